@@ -16,12 +16,17 @@ PAGE_TOKENS = 64  # a sequence's keys and values are stored in pages of this man
 @dataclass(frozen=True)
 class KVNeed:
     """Keys and values of every position, or of the last ``window`` positions. ``value_dim``: the values' width
-    where it differs from the keys' (None: the same)."""
+    where it differs from the keys' (None: the same; 0: rows of one kind only, kept where the keys are)."""
 
     num_kv_heads: int
     head_dim: int
     window: int | None = None
     value_dim: int | None = None
+
+    @property
+    def values(self) -> int:
+        """The width of a position's values."""
+        return self.head_dim if self.value_dim is None else self.value_dim
 
 
 @dataclass(frozen=True)

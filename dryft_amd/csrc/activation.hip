@@ -202,3 +202,94 @@ DRYFT_API int dryft_blend_columns(void* a, int64_t a_stride, const void* b, int6
                        b_stride, lam, width);
   return DRYFT_LAUNCH_CHECK();
 }
+
+// A polynomial of a row and its element-wise powers, each divided by its own root mean square over the row:
+//
+//   y = c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3,   N(u) = u / sqrt(mean(u^2) + eps)
+//
+// z is a row in the activation dtype or the float partial sums of a matrix product, added up on the way in; c holds the
+// four numbers on the device. Float arithmetic, rounded once. A workgroup a row; HELD keeps the row in LDS (dynamic
+// shared memory of `width` floats) between the two passes, else it is read twice. V values a thread and access.
+#define POLY_HELD_WIDTH 16384
+
+template <typename T, typename D, int V, bool HELD>
+__global__ __launch_bounds__(512) void poly_norm_kernel(const D* __restrict__ z, int64_t z_stride, int n_partials,
+                                                        int64_t partial_stride, const float* __restrict__ c,
+                                                        T* __restrict__ y, int width, float eps) {
+  extern __shared__ __attribute__((aligned(16))) float held[];
+  __shared__ float part[3][8];
+  const int64_t row = blockIdx.x;
+  const D* zr = z + row * z_stride;
+  auto read = [&](int i, float (&v)[V]) {
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[j] = 0.f;
+    for (int p = 0; p < n_partials; ++p) {
+      float t[V];
+      if constexpr (V == 8) load8_as_float(zr + p * partial_stride + i, t);
+      else t[0] = load_as_float(zr + p * partial_stride + i);
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[j] += t[j];
+    }
+  };
+  float s2 = 0.f, s4 = 0.f, s6 = 0.f;
+  for (int i = threadIdx.x * V; i < width; i += blockDim.x * V) {
+    float v[V];
+    read(i, v);
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      if (HELD) held[i + j] = v[j];
+      const float q = v[j] * v[j];
+      s2 += q;
+      s4 += q * q;
+      s6 += q * q * q;
+    }
+  }
+  const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE, waves = blockDim.x / WAVE;
+  s2 = wave_sum(s2);
+  s4 = wave_sum(s4);
+  s6 = wave_sum(s6);
+  if (lane == 0) { part[0][wave] = s2; part[1][wave] = s4; part[2][wave] = s6; }
+  __syncthreads();
+  s2 = s4 = s6 = 0.f;
+  for (int w = 0; w < waves; ++w) { s2 += part[0][w]; s4 += part[1][w]; s6 += part[2][w]; }
+  const float n = (float)width, a = c[0] / sqrtf(s2 / n + eps), b = c[1] / sqrtf(s4 / n + eps),
+              d = c[2] / sqrtf(s6 / n + eps), e = c[3];
+  for (int i = threadIdx.x * V; i < width; i += blockDim.x * V) {
+    float v[V];
+    if (HELD) {
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[j] = held[i + j];
+    } else {
+      read(i, v);
+    }
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[j] = ((d * v[j] + b) * v[j] + a) * v[j] + e;
+    if constexpr (V == 8) store8_from_float(y + row * width + i, v);
+    else store_from_float(y + row * width + i, v[0]);
+  }
+}
+
+// kind: 1 = z in the activation dtype, rows z_stride apart; 2 = float partial sums
+DRYFT_API int dryft_poly_norm(const void* z, int kind, int64_t z_stride, int n_partials, int64_t partial_stride,
+                              const float* c, void* y, int n_rows, int width, float eps, int is_f32, hipStream_t stream) {
+  if (n_rows <= 0) return 0;
+  if (width <= 0 || n_partials < 1) return -1;
+  const bool wide = width % 8 == 0 && z_stride % 8 == 0 && partial_stride % 4 == 0 &&
+                    (((uintptr_t)z | (uintptr_t)y) & 15) == 0;
+  const bool held = width <= POLY_HELD_WIDTH;
+  const int threads = width >= 4096 ? 512 : 256;
+#define PN(TT, DD, V, H)                                                                                             \
+  hipLaunchKernelGGL((poly_norm_kernel<TT, DD, V, H>), dim3(n_rows), dim3(threads), H ? (size_t)width * sizeof(float) : 0, \
+                     stream, (const DD*)z, z_stride, n_partials, partial_stride, c, (TT*)y, width, eps)
+#define PNH(TT, DD)                                                                                                  \
+  if (wide && held) { PN(TT, DD, 8, true); }                                                                         \
+  else if (wide) { PN(TT, DD, 8, false); }                                                                           \
+  else if (held) { PN(TT, DD, 1, true); }                                                                            \
+  else { PN(TT, DD, 1, false); }
+  if (is_f32) { PNH(float, float) }
+  else if (kind == 2) { PNH(bf16_t, float) }
+  else { PNH(bf16_t, bf16_t) }
+#undef PNH
+#undef PN
+  return DRYFT_LAUNCH_CHECK();
+}

@@ -56,7 +56,7 @@ __global__ __launch_bounds__(256) void latent_rope_kv_kernel(
     const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rot, const int* __restrict__ row_slot,
     const int* __restrict__ row_pos, T* __restrict__ q_out, T* __restrict__ k_pages, T* __restrict__ v_pages,
     const int* __restrict__ page_table, int max_pages, int write_kv, int n_heads, int plain, int rot_dim, int v_dim,
-    int page_dv, int pairs) {
+    int page_dv, int pairs, int page_dk) {
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int64_t row = blockIdx.x;
   const int job = blockIdx.y * 4 + wave;
@@ -64,7 +64,7 @@ __global__ __launch_bounds__(256) void latent_rope_kv_kernel(
   const int kind = job / n_heads, head = job % n_heads, key_dim = plain + rot_dim;
   const int slot = row_slot[row], pos = row_pos[row];
   if (kind == 0 && slot < 0) {
-    for (int i = lane; i < key_dim; i += WAVE) store_from_float(q_out + (row * n_heads + head) * key_dim + i, 0.f);
+    for (int i = lane; i < page_dk; i += WAVE) store_from_float(q_out + (row * n_heads + head) * page_dk + i, 0.f);
     return;
   }
   if (kind != 0 && (slot < 0 || !write_kv)) return;
@@ -80,8 +80,8 @@ __global__ __launch_bounds__(256) void latent_rope_kv_kernel(
     for (int i = lane; i < v_dim; i += WAVE) dst[(int64_t)i * PAGE_TOKENS] = src[i];
     return;
   }
-  T* dst = kind == 0 ? q_out + (row * n_heads + head) * key_dim
-                     : k_pages + (((int64_t)page * n_heads + head) * PAGE_TOKENS + in_page) * key_dim;
+  T* dst = kind == 0 ? q_out + (row * n_heads + head) * page_dk
+                     : k_pages + (((int64_t)page * n_heads + head) * PAGE_TOKENS + in_page) * page_dk;
   const T* src_plain = kind == 0 ? q_raw + (row * n_heads + head) * key_dim
                                  : kv + row * (int64_t)(n_heads * (plain + v_dim)) + (int64_t)head * plain;
   const T* src_rot = kind == 0 ? src_plain + plain : down + row * down_stride + krot_col;
@@ -95,26 +95,28 @@ __global__ __launch_bounds__(256) void latent_rope_kv_kernel(
     store_from_float(dst + plain + ib, b * c + a * s);
   }
   for (int i = rot + lane; i < rot_dim; i += WAVE) dst[plain + i] = src_rot[i];
+  for (int i = key_dim + lane; kind == 0 && i < page_dk; i += WAVE) store_from_float(dst + i, 0.f);
 }
 
 DRYFT_API int dryft_latent_rope_kv(const void* q_raw, const void* kv, const void* down, int64_t down_stride, int krot_col,
                                    const float* cos_t, const float* sin_t, int rot, const int* row_slot,
                                    const int* row_pos, void* q_out, void* k_pages, void* v_pages, const int* page_table,
                                    int max_pages, int write_kv, int n_rows, int n_heads, int plain, int rot_dim, int v_dim,
-                                   int page_dv, int pairs, int is_f32, hipStream_t stream) {
+                                   int page_dv, int pairs, int page_dk, int is_f32, hipStream_t stream) {
   if (n_rows <= 0) return 0;
-  if (rot < 0 || rot % 2 || rot > rot_dim || n_heads <= 0 || v_dim > page_dv) return -1;
+  if (rot < 0 || rot % 2 || rot > rot_dim || n_heads <= 0 || v_dim > page_dv || plain + rot_dim > page_dk)
+    return -1;
   dim3 grid(n_rows, (3 * n_heads + 3) / 4), block(256);
   if (is_f32)
     hipLaunchKernelGGL(latent_rope_kv_kernel<float>, grid, block, 0, stream, (const float*)q_raw, (const float*)kv,
                        (const float*)down, down_stride, krot_col, cos_t, sin_t, rot, row_slot, row_pos, (float*)q_out,
                        (float*)k_pages, (float*)v_pages, page_table, max_pages, write_kv, n_heads, plain, rot_dim, v_dim,
-                       page_dv, pairs);
+                       page_dv, pairs, page_dk);
   else
     hipLaunchKernelGGL(latent_rope_kv_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)q_raw, (const bf16_t*)kv,
                        (const bf16_t*)down, down_stride, krot_col, cos_t, sin_t, rot, row_slot, row_pos, (bf16_t*)q_out,
                        (bf16_t*)k_pages, (bf16_t*)v_pages, page_table, max_pages, write_kv, n_heads, plain, rot_dim,
-                       v_dim, page_dv, pairs);
+                       v_dim, page_dv, pairs, page_dk);
   return DRYFT_LAUNCH_CHECK();
 }
 

@@ -192,7 +192,32 @@ DRYFT_API int dryft_add_rows(const void* a, const void* b, void* out, int64_t n,
 // shared memory of `width` floats), and a thread touches the same elements in every pass.
 // `form` chooses other norms: bit 0, the branch's norm takes the mean off first (a layer norm without bias:
 // (d - mean) * rsqrt(mean((d - mean)^2) + eps) * wb); bit 1, the same for y; bit 2, y is x_new itself, only rounded
-// (a sublayer that reads the stream as it is).
+// (a sublayer that reads the stream as it is). With `groups` > 1 the norm of y is an rms norm taken in that many equal
+// consecutive parts of the row, each divided by its own root mean square.
+#define STREAM_NORM_MAX_GROUPS 256
+
+// Sums of squares of a row's parts from its values in LDS, by the block's four waves: parts of a row of fewer than
+// four are cut further so that every wave has work. Part g's sum is sums[g * cuts] + ... (`cuts` is returned).
+__device__ __forceinline__ int part_squares(const float* held, int width, int groups, float* sums) {
+  const int cuts = groups >= 4 ? 1 : 4 / groups, len = width / groups;
+  const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
+  __syncthreads();                           // the row has been written
+  for (int u = wave; u < groups * cuts; u += 4) {
+    const float* part = held + (u / cuts) * len;
+    float ss = 0.f;
+    for (int i = (u % cuts) * WAVE + lane; i < len; i += cuts * WAVE) ss += part[i] * part[i];
+    ss = wave_sum(ss);
+    if (lane == 0) sums[u] = ss;
+  }
+  __syncthreads();
+  return cuts;
+}
+__device__ __forceinline__ float part_inverse(const float* sums, int cuts, int g, int len, float eps) {
+  float ss = 0.f;
+  for (int c = 0; c < cuts; ++c) ss += sums[g * cuts + c];
+  return rsqrtf(ss / (float)len + eps);
+}
+
 template <typename T, typename D>
 __global__ __launch_bounds__(256) void stream_norm_kernel(const void* __restrict__ x_in, int x_kind,
                                                           const D* __restrict__ delta, int n_partials,
@@ -201,9 +226,9 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(const void* __restrict
                                                           const void* __restrict__ vec, int vec_f32,
                                                           const void* __restrict__ w, int w_f32,
                                                           float* __restrict__ x_out, T* __restrict__ y, int width,
-                                                          float eps, int form) {
+                                                          float eps, int form, int groups) {
   extern __shared__ __attribute__((aligned(16))) float held[];
-  __shared__ float scratch[16];
+  __shared__ float scratch[16], sums[STREAM_NORM_MAX_GROUPS];
   const int64_t base = (int64_t)blockIdx.x * width;
   float inv_d = 1.f, mean_d = 0.f;
   if (n_partials > 0) {
@@ -242,6 +267,12 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(const void* __restrict
     for (int i = threadIdx.x; i < width; i += blockDim.x) store_from_float(y + base + i, held[i]);
     return;
   }
+  if (groups > 1) {
+    const int cuts = part_squares(held, width, groups, sums), len = width / groups;
+    for (int i = threadIdx.x; i < width; i += blockDim.x)
+      store_from_float(y + base + i, held[i] * part_inverse(sums, cuts, i / len, len, eps) * load_vector(w, i, w_f32));
+    return;
+  }
   float mean = 0.f;
   if (form & 2) {
     mean = block_sum(sv, scratch) / (float)width;
@@ -264,9 +295,9 @@ __global__ __launch_bounds__(256) void stream_norm_vec_kernel(const void* __rest
                                                               const void* __restrict__ vec, int vec_f32,
                                                               const void* __restrict__ w, int w_f32,
                                                               float* __restrict__ x_out, T* __restrict__ y, int width,
-                                                              float eps, int form) {
+                                                              float eps, int form, int groups) {
   extern __shared__ __attribute__((aligned(16))) float held[];
-  __shared__ float scratch[16];
+  __shared__ float scratch[16], sums[STREAM_NORM_MAX_GROUPS];
   const int64_t base = (int64_t)blockIdx.x * width;
   float inv_d = 1.f, mean_d = 0.f;
   if (n_partials > 0) {
@@ -348,6 +379,24 @@ __global__ __launch_bounds__(256) void stream_norm_vec_kernel(const void* __rest
     }
     return;
   }
+  if (groups > 1) {
+    const int cuts = part_squares(held, width, groups, sums), len = width / groups;
+    for (int i = threadIdx.x * 8; i < width; i += blockDim.x * 8) {
+      float v[8], wv[8];
+      load8_as_float(held + i, v);
+      if (w_f32) load8_as_float((const float*)w + i, wv); else load8_as_float((const bf16_t*)w + i, wv);
+      if (len % 8 == 0) {                    // eight neighbours lie in one part
+        const float inv = part_inverse(sums, cuts, i / len, len, eps);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v[j] *= inv * wv[j];
+      } else {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v[j] *= part_inverse(sums, cuts, (i + j) / len, len, eps) * wv[j];
+      }
+      store8_from_float(y + base + i, v);
+    }
+    return;
+  }
   float mean = 0.f;
   if (form & 2) {
     mean = block_sum(sv, scratch) / (float)width;
@@ -377,8 +426,10 @@ __global__ __launch_bounds__(256) void stream_norm_vec_kernel(const void* __rest
 DRYFT_API int dryft_stream_norm(const void* x_in, int x_kind, const void* delta, int delta_kind, int n_partials,
                                 int64_t partial_stride, const void* wb, int wb_f32, const void* extra,
                                 const void* vec, int vec_f32, const void* w, int w_f32, float* x_out, void* y,
-                                int n_rows, int width, float eps, int is_f32, int form, hipStream_t stream) {
+                                int n_rows, int width, float eps, int is_f32, int form, int groups,
+                                hipStream_t stream) {
   if (n_rows <= 0) return 0;
+  if (groups < 1 || groups > STREAM_NORM_MAX_GROUPS || width % groups || (groups > 1 && (form & 2))) return -1;
   if (width <= 0 || width > STREAM_NORM_MAX_WIDTH || (y != nullptr && w == nullptr && !(form & 4))) return -1;
   if (delta_kind == 0) n_partials = 0;
   dim3 grid(n_rows), block(256);
@@ -386,11 +437,11 @@ DRYFT_API int dryft_stream_norm(const void* x_in, int x_kind, const void* delta,
 #define SN(TT, DD)                                                                                                   \
   hipLaunchKernelGGL((stream_norm_kernel<TT, DD>), grid, block, lds, stream, x_in, x_kind, (const DD*)delta,        \
                      n_partials, partial_stride, wb, wb_f32, (const TT*)extra, vec, vec_f32, w, w_f32, x_out,       \
-                     (TT*)y, width, eps, form)
+                     (TT*)y, width, eps, form, groups)
 #define SNV(TT, DD)                                                                                                  \
   hipLaunchKernelGGL((stream_norm_vec_kernel<TT, DD>), grid, block, lds, stream, x_in, x_kind, (const DD*)delta,    \
                      n_partials, partial_stride, wb, wb_f32, (const TT*)extra, vec, vec_f32, w, w_f32, x_out,       \
-                     (TT*)y, width, eps, form)
+                     (TT*)y, width, eps, form, groups)
   const bool aligned = (((uintptr_t)x_in | (uintptr_t)delta | (uintptr_t)wb | (uintptr_t)extra | (uintptr_t)vec |
                          (uintptr_t)w | (uintptr_t)x_out | (uintptr_t)y) & 15) == 0 && partial_stride % 4 == 0;
   if (width % 8 == 0 && aligned) {
@@ -458,5 +509,59 @@ DRYFT_API int dryft_rms_pair_mean(const void* a, int a_kind, int a_parts, int64_
   else if (fb) PM(bf16_t, float);
   else PM(bf16_t, bf16_t);
 #undef PM
+  return DRYFT_LAUNCH_CHECK();
+}
+
+// Two branches, each times a number: out = sa * (sum_p A[p] + bias_a) + sb * (sum_p B[p] + bias_b), float32. A thread takes
+// `V` neighbouring values.
+template <typename DA, typename DB, int V>
+__global__ __launch_bounds__(256) void scaled_pair_kernel(const DA* __restrict__ a, int a_parts, int64_t a_stride,
+                                                          const float* __restrict__ a_bias, float sa,
+                                                          const DB* __restrict__ b, int b_parts, int64_t b_stride,
+                                                          const float* __restrict__ b_bias, float sb,
+                                                          float* __restrict__ out, int64_t total, int width) {
+  const int64_t i = ((int64_t)blockIdx.x * blockDim.x + threadIdx.x) * V;
+  if (i >= total) return;
+  float x[8], y[8], t[8];
+#pragma unroll
+  for (int j = 0; j < V; ++j) {
+    x[j] = a_bias ? a_bias[(i + j) % width] : 0.f;
+    y[j] = b_bias ? b_bias[(i + j) % width] : 0.f;
+  }
+  for (int p = 0; p < a_parts; ++p) {
+    if constexpr (V == 8) load8_as_float(a + p * a_stride + i, t); else t[0] = load_as_float(a + p * a_stride + i);
+#pragma unroll
+    for (int j = 0; j < V; ++j) x[j] += t[j];
+  }
+  for (int p = 0; p < b_parts; ++p) {
+    if constexpr (V == 8) load8_as_float(b + p * b_stride + i, t); else t[0] = load_as_float(b + p * b_stride + i);
+#pragma unroll
+    for (int j = 0; j < V; ++j) y[j] += t[j];
+  }
+#pragma unroll
+  for (int j = 0; j < V; ++j) x[j] = sa * x[j] + sb * y[j];
+  if constexpr (V == 8) store8_from_float(out + i, x); else out[i] = x[0];
+}
+
+// kinds, parts and strides as for dryft_rms_pair_mean
+DRYFT_API int dryft_scaled_pair(const void* a, int a_kind, int a_parts, int64_t a_stride, const float* a_bias, float sa,
+                                const void* b, int b_kind, int b_parts, int64_t b_stride, const float* b_bias, float sb,
+                                float* out, int n_rows, int width, int is_f32, hipStream_t stream) {
+  if (n_rows <= 0) return 0;
+  if (width <= 0 || a_parts < 1 || b_parts < 1) return -1;
+  const int64_t total = (int64_t)n_rows * width;
+  const bool fa = is_f32 || a_kind == 2, fb = is_f32 || b_kind == 2;
+  const bool wide = width % 8 == 0 && (((uintptr_t)a | (uintptr_t)b | (uintptr_t)out) & 15) == 0;
+#define SP(DA, DB, V)                                                                                                 \
+  hipLaunchKernelGGL((scaled_pair_kernel<DA, DB, V>), dim3((unsigned)((total / V + 255) / 256)), dim3(256), 0, stream,  \
+                     (const DA*)a, a_parts, a_stride, a_bias, sa, (const DB*)b, b_parts, b_stride, b_bias, sb, out, total, \
+                     width)
+#define SPV(DA, DB) if (wide) { SP(DA, DB, 8); } else { SP(DA, DB, 1); }
+  if (fa && fb) { SPV(float, float) }
+  else if (fa) { SPV(float, bf16_t) }
+  else if (fb) { SPV(bf16_t, float) }
+  else { SPV(bf16_t, bf16_t) }
+#undef SPV
+#undef SP
   return DRYFT_LAUNCH_CHECK();
 }

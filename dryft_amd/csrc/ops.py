@@ -24,12 +24,14 @@ _SIGNATURES = {
               "dryft_embed_scaled": [_P, _P, _P, _I, _I, _I, _F, _I, _P]},
     "norm": {"dryft_add_rmsnorm": [_P, _P, _I, _I, _L, _P, _I, _P, _P, _I, _I, _F, _I, _P],
              "dryft_add_rows": [_P, _P, _P, _L, _I, _P],
-             "dryft_stream_norm": [_P, _I, _P, _I, _I, _L, _P, _I, _P, _P, _I, _P, _I, _P, _P, _I, _I, _F, _I, _I, _P],
+             "dryft_stream_norm": [_P, _I, _P, _I, _I, _L, _P, _I, _P, _P, _I, _P, _I, _P, _P, _I, _I, _F, _I, _I, _I, _P],
+             "dryft_scaled_pair": [_P, _I, _I, _L, _P, _F, _P, _I, _I, _L, _P, _F, _P, _I, _I, _I, _P],
              "dryft_rms_pair_mean": [_P, _I, _I, _L, _P, _P, _P, _I, _I, _L, _P, _P, _P, _I, _I, _F, _I, _P]},
     "activation": {"dryft_silu_mul": [_P, _P, _I, _I, _L, _I, _P],
                    "dryft_glu_clamped": [_P, _P, _I, _I, _L, _F, _F, _I, _P],
                    "dryft_sigmoid_gate": [_P, _L, _P, _L, _P, _I, _I, _I, _P],
                    "dryft_relu_squared": [_P, _L, _P, _I, _I, _I, _P],
+                   "dryft_poly_norm": [_P, _I, _L, _I, _L, _P, _P, _I, _I, _F, _I, _P],
                    "dryft_token_gate": [_P, _L, _P, _P, _L, _I, _I, _P, _I, _I, _I, _P],
                    "dryft_blend_columns": [_P, _L, _P, _L, _P, _I, _I, _I, _P]},
     "mlstm": {"dryft_mlstm_steps": [_P, _L, _I, _I, _I, _P, _P, _P, _F, _P, _P, _P, _I, _P, _P, _P, _P, _I, _I, _I, _F,
@@ -49,7 +51,7 @@ _SIGNATURES = {
                 "dryft_rope_pairs_kv": [_P, _L, _I, _I, _I, _P, _P, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I,
                                         _I, _I, _P],
                 "dryft_norm_rope_half_kv": [_P, _L, _I, _I, _I, _P, _P, _F, _P, _P, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I,
-                                            _I, _I, _I, _I, _I, _I, _P],
+                                            _I, _I, _I, _I, _I, _I, _I, _P],
                 "dryft_rows_to_cache_takes": [_I, _I, _I, _I],
                 "dryft_rows_to_cache_parts": [_P, _I, _L, _P, _P, _I, _I, _F, _P, _P, _I, _P, _P, _P, _P, _P, _P, _I, _I,
                                               _I, _I, _I, _P]},
@@ -82,12 +84,13 @@ _SIGNATURES = {
     "hyper": {"dryft_hyper_norm": [_P, _I, _I, _P, _I, _I, _L, _P, _P, _P, _P, _P, _P, _I, _I, _I, _F, _I, _P]},
     "wkv": {"dryft_wkv_blend": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _P],
             "dryft_wkv_decay": [_P, _P, _P, _P, _I, _I, _I, _I, _P],
+            "dryft_log_decay": [_P, _P, _P, _P, _I, _I, _I, _F, _I, _P],
             "dryft_wkv_steps": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _P, _I, _I, _P, _P, _I,
                                 _P],
             "dryft_wkv_out": [_P, _P, _P, _P, _I, _I, _I, _F, _L, _I, _P]},
     "latent": {"dryft_rms_segments": [_P, _L, _I, _P, _P, _I, _P, _P, _I, _F, _I, _I, _P],
                "dryft_latent_rope_kv": [_P, _P, _P, _L, _I, _P, _P, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I,
-                                        _I, _I, _I, _I, _P],
+                                        _I, _I, _I, _I, _I, _P],
                "dryft_head_gate": [_P, _P, _L, _I, _P, _I, _I, _I, _I, _I, _I, _P]},
     "moe": {"dryft_moe_route": [_P, _L, _P, _I, _I, _I, _I, _F, _P, _P, _I, _I, _I, _I, _P],
             "dryft_moe_plan": [_P, _I, _I, _P, _P, _P, _P, _P, _P, _I, _P],
@@ -104,6 +107,16 @@ _SIGNATURES = {
     "delta": {"dryft_delta_max_dim": [],
               "dryft_delta_steps": [_P, _L, _I, _I, _I, _P, _L, _I, _I, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I,
                                     _F, _F, _I, _P, _I, _I, _P, _P, _I, _P]},
+    "linattn": {"dryft_linattn_max_dim": [],
+                "dryft_linattn_token": [_P, _L, _I, _I, _I, _I, _F, _F, _P, _P, _I, _P, _P, _P, _P, _P, _P, _I, _P, _P, _F, _P,
+                                        _I, _I, _I, _I, _I, _P],
+                "dryft_linattn_chunk": [_P, _L, _I, _I, _I, _F, _F, _P, _P, _I, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I,
+                                        _I, _P, _I, _I, _P, _P, _I, _P]},
+    "mla": {"dryft_latent_rows_in": [_P, _I, _L, _I, _L, _P, _P, _I, _P, _P, _I, _I, _P, _P, _I, _I, _F, _P, _P, _P, _P, _I, _I,
+                                     _I, _I, _I, _P],
+            "dryft_head_product": [_P, _L, _I, _I, _P, _I, _I, _I, _I, _P, _L, _I, _I, _I, _I, _P, _P, _I, _I, _P, _I, _P],
+            "dryft_latent_split": [_P, _P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _F, _P, _P, _I, _P, _P],
+            "dryft_latent_attend_f32": [_P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _F, _P]},
     "sampling": {"dryft_argmax_rows": [_P, _I, _I, _L, _P, _I, _P, _P, _P],
                  "dryft_sample_rows": [_P, _I, _I, _L, _F, _P, _P, _I, _P, _P, _P]},
 }
@@ -263,17 +276,24 @@ def add_rows(a: torch.Tensor, b: torch.Tensor, out: torch.Tensor) -> torch.Tenso
     return out
 
 
+STREAM_NORM_MAX_GROUPS = 256
+
+
 def stream_norm(x, delta, post_weight, extra, vec, weight, eps: float, x_out, y, act: torch.dtype,
-                post_centred: bool = False, centred: bool = False, plain_read: bool = False) -> None:
+                post_centred: bool = False, centred: bool = False, plain_read: bool = False, groups: int = 1) -> None:
     """The norms of a float32 residual stream in one launch, per row (``post_centred`` / ``centred``: the norm of
     ``d`` / of ``x_out`` takes the mean off first and divides by the standard deviation, a layer norm without bias;
     ``plain_read``: ``y`` is ``x_out`` itself in the activation dtype, no weight):
     ``d = delta`` (a tensor in the activation dtype, or ``[n, rows, width]`` float32 partial sums as ``(data, n)``);
     ``x_out = x + rmsnorm(d) * post_weight + extra + vec`` (each term optional; without ``post_weight`` ``d`` is added
     as it is); ``y = rmsnorm(x_out) * weight`` in the activation dtype (optional). ``x`` is float32, or in the
-    activation dtype ``act`` (a stream that starts), or None; ``x_out`` is float32 (may be ``x`` itself) or None."""
+    activation dtype ``act`` (a stream that starts), or None; ``x_out`` is float32 (may be ``x`` itself) or None.
+    ``groups`` > 1: the norm of ``y`` is taken in so many equal consecutive parts of the row, each by itself."""
     ref = y if y is not None else (x_out if x_out is not None else x)
     rows, width = ref.shape
+    if groups < 1 or groups > STREAM_NORM_MAX_GROUPS or width % groups or (groups > 1 and centred):
+        raise KernelError(f"stream_norm: {width} values do not split into {groups} equal parts (at most "
+                          f"{STREAM_NORM_MAX_GROUPS}, and without a mean taken off)")
     x_kind = 0
     if x is not None:
         _gpu(x, "x")
@@ -319,7 +339,7 @@ def stream_norm(x, delta, post_weight, extra, vec, weight, eps: float, x_out, y,
     _check(_fn("norm", "dryft_stream_norm")(
         _ptr(x), x_kind, _ptr(delta), kind, n_partials, stride, _ptr(post_weight), flag(post_weight), _ptr(extra),
         _ptr(vec), flag(vec), _ptr(weight), flag(weight), _ptr(x_out), _ptr(y), rows, width, float(eps), is_f32,
-        (1 if post_centred else 0) | (2 if centred else 0) | (4 if plain_read else 0), _stream()), "stream_norm")
+        (1 if post_centred else 0) | (2 if centred else 0) | (4 if plain_read else 0), int(groups), _stream()), "stream_norm")
 
 
 # -------------------------------------------------------------------------------------- activation
@@ -361,6 +381,29 @@ def relu_squared(x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
         raise KernelError("relu_squared: x [rows, width] with unit column stride, out contiguous")
     _check(_fn("activation", "dryft_relu_squared")(_ptr(x), x.stride(0), _ptr(out), rows, width, _float_flag(x, "x"),
                                                    _stream()), "relu_squared")
+    return out
+
+
+def poly_norm(z, coefficients: torch.Tensor, eps: float, out: torch.Tensor) -> torch.Tensor:
+    """``out = c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3`` per row, powers element by element and ``N`` the division by the row's
+    root mean square; ``coefficients`` float32 ``[4]`` on the device. ``z`` is ``[rows, width]`` in the dtype of ``out``
+    (unit column stride) or float32 partial sums ``(data [n, rows, width], n)``."""
+    _gpu(out, "out")
+    is_f32 = _float_flag(out, "out")
+    rows, width = out.shape
+    if isinstance(z, tuple):
+        data, kind, n, stride = _branch(z, rows, width, out.dtype, "z")
+        row_stride = width
+    else:
+        _gpu(z, "z", out.dtype)
+        if not (z.shape == out.shape and z.stride(1) == 1):
+            raise KernelError("poly_norm: z must be [rows, width] with unit column stride")
+        data, kind, n, stride, row_stride = z, 1, 1, 0, z.stride(0)
+    if not out.is_contiguous():
+        raise KernelError("poly_norm: out must be contiguous")
+    _f32_vector(coefficients, "coefficients", 4)
+    _check(_fn("activation", "dryft_poly_norm")(_ptr(data), kind, row_stride, n, stride, _ptr(coefficients), _ptr(out), rows,
+                                                width, float(eps), is_f32, _stream()), "poly_norm")
     return out
 
 
@@ -1491,6 +1534,22 @@ def wkv_decay(low, up, bias, decay) -> None:
                                          _float_flag(up, "up"), _stream()), "wkv_decay")
 
 
+def log_decay(low, up, bias, decay, factor: float) -> None:
+    """``decay = log(sigmoid(low @ up.T + bias)) * factor``, the logarithm of ``sigmoid(.)^factor``; operands as above."""
+    _gpu(low, "low", torch.float32)
+    _gpu(up, "up")
+    rows, rank = low.shape
+    n = up.shape[0]
+    if not (low.is_contiguous() and up.is_contiguous() and up.shape == (n, rank)):
+        raise KernelError(f"log_decay: low contiguous [rows, {rank}], up contiguous [n, {rank}], got {tuple(up.shape)}")
+    _f32_vector(bias, "bias", n)
+    _gpu(decay, "decay", torch.float32)
+    if not (decay.shape == (rows, n) and decay.is_contiguous()):
+        raise KernelError("log_decay: decay must be contiguous float32 [rows, n]")
+    _check(_fn("wkv", "dryft_log_decay")(_ptr(low), _ptr(up), _ptr(bias), _ptr(decay), rows, n, rank, float(factor),
+                                         _float_flag(up, "up"), _stream()), "log_decay")
+
+
 WKV_GROUP = 16          # tokens the recurrence's kernel takes at a time; segments are multiples of it
 
 
@@ -1584,11 +1643,12 @@ def rms_segments(src, col: int, w_a, out_a, n_a: int, w_b, out_b, eps: float) ->
 
 def latent_rope_kv(q_raw, kv, down, krot_col: int, cos, sin, rot: int, row_slot, row_pos, q_out, k_pages, v_pages,
                    page_table, write_kv: bool, n_heads: int, plain: int, rot_dim: int, v_dim: int, page_dv: int,
-                   pairs: bool = False) -> None:
+                   pairs: bool = False, page_dk: int = 0) -> None:
     """Queries ``[plain | rotated]`` per head from ``q_raw``; keys ``[that head's plain part of kv | the one rotated
     part at column krot_col of down]``; values from ``kv`` after the keys. The rotated parts' first ``rot`` features
     turn, feature ``i`` with ``i + rot/2`` (with ``pairs``: feature ``2i`` with ``2i + 1``), with float32 tables; keys
-    and values go to their pages (values ``page_dv`` wide, of which ``v_dim`` are written)."""
+    and values go to their pages (values ``page_dv`` wide, of which ``v_dim`` are written). ``page_dk``: the width of the
+    keys' pages and of the rows of ``q_out`` where it is more than ``plain + rot_dim`` (zeros behind a head's own)."""
     _gpu(q_raw, "q_raw")
     is_f32 = _float_flag(q_raw, "q_raw")
     rows, key_dim = q_raw.shape[0], plain + rot_dim
@@ -1609,11 +1669,12 @@ def latent_rope_kv(q_raw, kv, down, krot_col: int, cos, sin, rot: int, row_slot,
             if not (t.dim() == 2 and t.shape[1] == rot // 2 and t.is_contiguous()):
                 raise KernelError(f"{name}: must be contiguous float32 [positions, {rot // 2}]")
     _gpu(q_out, "q_out", q_raw.dtype)
-    if not (q_out.is_contiguous() and q_out.numel() == rows * n_heads * key_dim):
-        raise KernelError("latent_rope_kv: q_out must be [rows, heads, key_dim]")
+    page_dk = int(page_dk) or key_dim
+    if not (page_dk >= key_dim and q_out.is_contiguous() and q_out.numel() == rows * n_heads * page_dk):
+        raise KernelError("latent_rope_kv: q_out must be [rows, heads, width of the keys' pages]")
     if not v_dim <= page_dv:
         raise KernelError("latent_rope_kv: the values' pages are narrower than the values")
-    _check_pages(k_pages, v_pages, page_table, n_heads, key_dim, q_raw.dtype, page_dv)
+    _check_pages(k_pages, v_pages, page_table, n_heads, page_dk, q_raw.dtype, page_dv)
     for name, t in (("row_slot", row_slot), ("row_pos", row_pos)):
         _gpu(t, name, torch.int32)
         if not (t.numel() >= rows):
@@ -1621,7 +1682,7 @@ def latent_rope_kv(q_raw, kv, down, krot_col: int, cos, sin, rot: int, row_slot,
     _check(_fn("latent", "dryft_latent_rope_kv")(
         _ptr(q_raw), _ptr(kv), _ptr(down), down.stride(0), krot_col, _ptr(cos), _ptr(sin), rot, _ptr(row_slot),
         _ptr(row_pos), _ptr(q_out), _ptr(k_pages), _ptr(v_pages), _ptr(page_table), page_table.shape[1],
-        int(bool(write_kv)), rows, n_heads, plain, rot_dim, v_dim, page_dv, int(bool(pairs)), is_f32, _stream()),
+        int(bool(write_kv)), rows, n_heads, plain, rot_dim, v_dim, page_dv, int(bool(pairs)), page_dk, is_f32, _stream()),
         "latent_rope_kv")
 
 
@@ -1825,6 +1886,23 @@ def rms_pair_mean(a, a_bias, a_weight, b, b_bias, b_weight, eps: float, out: tor
     return out
 
 
+def scaled_pair(a, a_bias, a_scale: float, b, b_bias, b_scale: float, out: torch.Tensor, act: torch.dtype) -> torch.Tensor:
+    """``out = a_scale * (a + a_bias) + b_scale * (b + b_bias)``, float32; operands as for ``rms_pair_mean``."""
+    _gpu(out, "out", torch.float32)
+    rows, width = out.shape
+    if not out.is_contiguous():
+        raise KernelError("scaled_pair: out must be contiguous")
+    pa, ka, na, sa = _branch(a, rows, width, act, "a")
+    pb, kb, nb, sb = _branch(b, rows, width, act, "b")
+    for name, t in (("a_bias", a_bias), ("b_bias", b_bias)):
+        if t is not None:
+            _f32_vector(t, name, width)
+    _check(_fn("norm", "dryft_scaled_pair")(_ptr(pa), ka, na, sa, _ptr(a_bias), float(a_scale), _ptr(pb), kb, nb, sb,
+                                            _ptr(b_bias), float(b_scale), _ptr(out), rows, width,
+                                            1 if act == torch.float32 else 0, _stream()), "scaled_pair")
+    return out
+
+
 # --------------------------------------------------------------------------------------- short causal convolution
 CONV_MAX_TAPS = 16
 
@@ -1899,13 +1977,16 @@ def conv_tail(u, col: int, channels: int, in_bias, taps: int, seq_slot, cu_rows,
 # ------------------------------------------------------------------------- norm per head, rotation over halves, append
 def norm_rope_half_kv(src, q_col: int, k_col: int, v_col: int, q_weight, k_weight, eps: float, cos, sin, rot: int,
                       row_slot, row_pos, q_out, k_pages, v_pages, page_table, write_kv: bool, n_heads: int, n_kv: int,
-                      head_dim: int, v_dim: int, page_dim: int = 0) -> None:
+                      head_dim: int, v_dim: int, page_dim: int = 0, unit_after: bool = False) -> None:
     """Every q and k head of ``src`` divided by its root mean square and multiplied by ``q_weight`` / ``k_weight``
     (float32 ``[head_dim]``; None: the head passes), then feature ``i`` of its first ``rot`` turned with feature
     ``i + rot / 2`` by float32 tables ``[positions, rot / 2]``; queries to ``q_out [rows, heads, head_dim]`` and, when
     ``write_kv``, keys and (untouched) values of width ``v_dim`` to their pages. ``page_dim`` > 0: pages and the rows of
     ``q_out`` are that wide for keys and values alike (at least as wide as either); what lies behind a head's own
-    features is not written, so ``q_out`` and the pages must have started as zeros."""
+    features is not written, so ``q_out`` and the pages must have started as zeros. ``unit_after``: every q and k head is
+    divided by its root mean square after the turn (no weight), and what comes before the turn has no norm."""
+    if unit_after and (q_weight is not None or k_weight is not None):
+        raise KernelError("norm_rope_half_kv: a norm before the turn or one after it")
     _gpu(src, "src")
     is_f32 = _float_flag(src, "src")
     rows = src.shape[0]
@@ -1935,8 +2016,8 @@ def norm_rope_half_kv(src, q_col: int, k_col: int, v_col: int, q_weight, k_weigh
     _check(_fn("rope_kv", "dryft_norm_rope_half_kv")(
         _ptr(src), src.stride(0), q_col, k_col, v_col, _ptr(q_weight), _ptr(k_weight), float(eps), _ptr(cos), _ptr(sin),
         rot, _ptr(row_slot), _ptr(row_pos), _ptr(q_out), _ptr(k_pages), _ptr(v_pages), _ptr(page_table),
-        page_table.shape[1], int(bool(write_kv)), rows, n_heads, n_kv, head_dim, v_dim, page_dim, is_f32, _stream()),
-        "norm_rope_half_kv")
+        page_table.shape[1], int(bool(write_kv)), rows, n_heads, n_kv, head_dim, v_dim, page_dim, int(bool(unit_after)),
+        is_f32, _stream()), "norm_rope_half_kv")
 
 
 # ------------------------------------------------------------------------------------------ state-space mixer
@@ -2065,3 +2146,237 @@ def delta_steps(qkv, q_col: int, k_col: int, v_col: int, gates, a_col: int, b_co
         _ptr(a_log), _ptr(seq_slot), _ptr(cu_rows), _ptr(q_len), _ptr(state), _ptr(out), n_seqs, n_heads, n_groups,
         key_dim, value_dim, float(q_scale), float(unit_eps), int(bool(write_state)), _ptr(seg_cu), max_segs, seg_rows,
         _ptr(seg_state), _ptr(seg_trans), _float_flag(qkv, "qkv"), _stream()), "delta_steps")
+
+
+# ------------------------------------------------------------------------------------------ linear attention
+LINEAR_MAX_DIM = 256
+LINEAR_CHUNK = 16       # tokens the chunk kernel takes at a time; segments are multiples of it
+
+
+def _linear_facts(who: str, proj, q_col: int, k_col: int, v_col: int, tables, row_pos, log_decays, head_decays, seq_slot,
+                  cu_rows, q_len, n_seqs: int, state, n_heads: int, dim: int, v_dim: int):
+    """Checks what both kernels of linear attention read; returns (cos, sin, rotated width)."""
+    _gpu(proj, "proj")
+    rows = proj.shape[0]
+    if not (proj.dim() == 2 and proj.stride(1) == 1 and min(q_col, k_col, v_col) >= 0 and
+            max(q_col + n_heads * dim, k_col + n_heads * dim, v_col + n_heads * v_dim) <= proj.shape[1]):
+        raise KernelError(f"{who}: q, k or v lie outside the columns of the projection")
+    cos, sin, rot = tables if tables is not None else (None, None, 0)
+    if rot % 2 or not 0 <= rot <= dim:
+        raise KernelError(f"{who}: the rotated width must be even and at most {dim}, got {rot}")
+    if rot:
+        for name, t in (("cos", cos), ("sin", sin)):
+            _gpu(t, name, torch.float32)
+            if not (t.dim() == 2 and t.shape[1] == rot // 2 and t.is_contiguous()):
+                raise KernelError(f"{name}: must be contiguous float32 [positions, {rot // 2}]")
+    _row_facts(rows, row_pos=row_pos)
+    if (log_decays is None) == (head_decays is None):
+        raise KernelError(f"{who}: decays per channel and token, or one per head")
+    if log_decays is not None:
+        _gpu(log_decays, "log_decays", torch.float32)
+        if not (log_decays.shape == (rows, n_heads * dim) and log_decays.is_contiguous()):
+            raise KernelError(f"{who}: log_decays must be contiguous float32 [rows, {n_heads * dim}]")
+    else:
+        _f32_vector(head_decays, "head_decays", n_heads)
+    _seq_facts(seq_slot, cu_rows, q_len, n_seqs)
+    _gpu(state, "state", torch.float32)
+    if not (state.dim() == 4 and state.shape[1:] == (n_heads, dim, v_dim) and state.is_contiguous()):
+        raise KernelError(f"{who}: state must be contiguous float32 [slots, {n_heads}, {dim}, {v_dim}]")
+    if not (0 < dim <= LINEAR_MAX_DIM and 0 < v_dim <= LINEAR_MAX_DIM):
+        raise KernelError(f"{who}: dim and v_dim must lie in 1..{LINEAR_MAX_DIM}")
+    return cos, sin, int(rot)
+
+
+def linear_token(proj, q_col: int, k_col: int, v_col: int, g_col: int, q_scale: float, k_scale: float, tables, row_pos,
+                 log_decays, head_decays, seq_slot, cu_rows, q_len, n_seqs: int, state, weight, eps: float, out, n_heads: int,
+                 dim: int, v_dim: int, write_state: bool) -> None:
+    """Per sequence and head, row by row from ``state [slots, heads, dim, v_dim]`` (float32): ``S <- diag(decay) S + k v^T``,
+    ``o = S^T q``, ``out = o / rms(o) * weight * silu(gate)`` in the activation dtype. ``q``, ``k``, ``v`` and the gate are
+    runs of columns of ``proj``; ``tables = (cos, sin, rotated width)`` turns q and k over halves first (None: no
+    rotation). Decays: ``log_decays`` float32 ``[rows, heads * dim]``, or ``head_decays`` float32 ``[heads]`` (the decays
+    themselves). ``weight`` float32 ``[v_dim]`` or None. Meant for steps of one row a sequence."""
+    cos, sin, rot = _linear_facts("linear_token", proj, q_col, k_col, v_col, tables, row_pos, log_decays, head_decays, seq_slot,
+                                  cu_rows, q_len, n_seqs, state, n_heads, dim, v_dim)
+    _gpu(out, "out", proj.dtype)
+    if not (0 <= g_col and g_col + n_heads * v_dim <= proj.shape[1] and out.shape == (proj.shape[0], n_heads * v_dim) and
+            out.is_contiguous()):
+        raise KernelError("linear_token: the gate a run of columns of the projection, out contiguous [rows, heads * v_dim]")
+    if weight is not None:
+        _f32_vector(weight, "weight", v_dim)
+    _check(_fn("linattn", "dryft_linattn_token")(
+        _ptr(proj), proj.stride(0), q_col, k_col, v_col, g_col, float(q_scale), float(k_scale), _ptr(cos), _ptr(sin), rot,
+        _ptr(row_pos), _ptr(log_decays), _ptr(head_decays), _ptr(seq_slot), _ptr(cu_rows), _ptr(q_len), n_seqs, _ptr(state),
+        _ptr(weight), float(eps), _ptr(out), n_heads, dim, v_dim, int(bool(write_state)), _float_flag(proj, "proj"),
+        _stream()), "linear_token")
+
+
+def linear_chunks(proj, q_col: int, k_col: int, v_col: int, q_scale: float, k_scale: float, tables, row_pos, log_decays,
+                  head_log_decays, seq_slot, cu_rows, q_len, n_seqs: int, state, o_raw, n_heads: int, dim: int, v_dim: int,
+                  write_state: bool, segments=None) -> None:
+    """The same recurrence sixteen tokens at a time on the matrix cores in 32-bit precision, up to the raw read-outs
+    ``o_raw`` (float32 ``[rows, heads * v_dim]``). The decays of heads come as logarithms too. ``segments``: as for
+    ``ssm_scan`` (multiples of 16 rows; the rows of sequences that sit out are then not written)."""
+    cos, sin, rot = _linear_facts("linear_chunks", proj, q_col, k_col, v_col, tables, row_pos, log_decays, head_log_decays,
+                                  seq_slot, cu_rows, q_len, n_seqs, state, n_heads, dim, v_dim)
+    _gpu(o_raw, "o_raw", torch.float32)
+    if not (o_raw.shape == (proj.shape[0], n_heads * v_dim) and o_raw.is_contiguous()):
+        raise KernelError("linear_chunks: o_raw must be contiguous float32 [rows, heads * v_dim]")
+    seg_rows, seg_cu, max_segs = _segment_facts("linear_chunks", segments, n_seqs, write_state)
+    seg_state = seg_decay = None
+    if segments is not None:
+        if seg_rows % LINEAR_CHUNK:
+            raise KernelError(f"linear_chunks: segments of a multiple of {LINEAR_CHUNK} rows")
+        if max_segs <= 0:
+            return
+        seg_state = torch.empty((max_segs, n_heads, dim, v_dim), dtype=torch.float32, device=proj.device)
+        seg_decay = torch.empty((max_segs, n_heads, dim), dtype=torch.float32, device=proj.device)
+    _check(_fn("linattn", "dryft_linattn_chunk")(
+        _ptr(proj), proj.stride(0), q_col, k_col, v_col, float(q_scale), float(k_scale), _ptr(cos), _ptr(sin), rot,
+        _ptr(row_pos), _ptr(log_decays), _ptr(head_log_decays), _ptr(seq_slot), _ptr(cu_rows), _ptr(q_len), n_seqs,
+        _ptr(state), _ptr(o_raw), n_heads, dim, v_dim, int(bool(write_state)), _ptr(seg_cu), max_segs, seg_rows,
+        _ptr(seg_state), _ptr(seg_decay), _float_flag(proj, "proj"), _stream()), "linear_chunks")
+
+
+# ------------------------------------------------------------------------------------------ attention to cached latents
+LATENT_MAX_WIDTH = 960      # features of a cached row (latent, rotated key part, padding)
+
+
+def _latent_pages(who: str, pages, page_table, dtype) -> int:
+    _gpu(pages, "pages", dtype)
+    _gpu(page_table, "page_table", torch.int32)
+    if not (pages.dim() == 4 and pages.shape[1] == 1 and pages.shape[2] == 64 and pages.is_contiguous() and
+            pages.shape[3] % 32 == 0 and pages.shape[3] <= LATENT_MAX_WIDTH and page_table.dim() == 2 and
+            page_table.is_contiguous()):
+        raise KernelError(f"{who}: pages must be contiguous [pages, 1, 64, width], the width a multiple of 32 and at most "
+                          f"{LATENT_MAX_WIDTH}")
+    return pages.shape[3]
+
+
+def _turn_tables(who: str, tables, row_pos, rows: int, rot_dim: int):
+    """``(cos, sin, rotated width, by pairs)`` checked; zeros for no rotation."""
+    cos, sin, rot, pairs = tables if tables is not None else (None, None, 0, False)
+    if rot % 2 or not 0 <= rot <= rot_dim:
+        raise KernelError(f"{who}: the rotated width must be even and at most {rot_dim}, got {rot}")
+    if rot:
+        for name, t in (("cos", cos), ("sin", sin)):
+            _gpu(t, name, torch.float32)
+            if not (t.dim() == 2 and t.shape[1] == rot // 2 and t.is_contiguous()):
+                raise KernelError(f"{name}: must be contiguous float32 [positions, {rot // 2}]")
+    _row_facts(rows, row_pos=row_pos)
+    return cos, sin, int(rot), int(bool(pairs))
+
+
+def latent_rows_in(src, w_q, c_q, w_kv, c_out, rot_dim: int, tables, eps: float, row_slot, row_pos, pages, page_table,
+                   write_kv: bool) -> None:
+    """``src [rows, q_rank | rank | rot_dim]`` (activation dtype, unit column stride, or float32 partial sums ``(data,
+    n)``): ``c_q = rms(.) * w_q``; the latent ``rms(.) * w_kv`` and the key part behind it, turned by ``tables = (cos, sin,
+    rotated width, by pairs)``, go to the row's place in its page, the latent also to ``c_out`` when that is given.
+    ``w_kv`` None: only ``c_q``."""
+    _gpu(c_q, "c_q")
+    is_f32 = _float_flag(c_q, "c_q")
+    rows, q_rank = c_q.shape
+    rank = w_kv.numel() if w_kv is not None else 0
+    rot_dim = int(rot_dim) if rank else 0
+    total = q_rank + rank + rot_dim
+    if isinstance(src, tuple):
+        data, n = src
+        _gpu(data, "src", torch.float32)
+        if not (data.dim() == 3 and data.shape[1] == rows and data.shape[2] >= total and data.is_contiguous() and
+                data.shape[0] >= n >= 1):
+            raise KernelError("latent_rows_in: partial sums must be contiguous float32 [n, rows, columns]")
+        kind, stride, part_stride = 2, data.shape[2], rows * data.shape[2]
+    else:
+        data, n, kind, part_stride = src, 1, 1, 0
+        _gpu(data, "src", c_q.dtype)
+        if not (data.dim() == 2 and data.shape[0] == rows and data.shape[1] >= total and data.stride(1) == 1):
+            raise KernelError("latent_rows_in: src must be [rows, columns] with unit column stride")
+        stride = data.stride(0)
+    if not c_q.is_contiguous():
+        raise KernelError("latent_rows_in: c_q must be contiguous")
+    _f32_vector(w_q, "w_q", q_rank)
+    cos = sin = None
+    rot = pairs = width = max_pages = 0
+    if rank:
+        _f32_vector(w_kv, "w_kv", rank)
+        width = _latent_pages("latent_rows_in", pages, page_table, c_q.dtype)
+        if rank + rot_dim > width:
+            raise KernelError("latent_rows_in: the pages are narrower than what is kept")
+        max_pages = page_table.shape[1]
+        if c_out is not None:
+            _gpu(c_out, "c_out", c_q.dtype)
+            if not (c_out.shape == (rows, rank) and c_out.is_contiguous()):
+                raise KernelError("latent_rows_in: c_out must be contiguous [rows, rank]")
+        cos, sin, rot, pairs = _turn_tables("latent_rows_in", tables, row_pos, rows, rot_dim)
+        _row_facts(rows, row_slot=row_slot)
+    else:
+        c_out = pages = page_table = None
+    _check(_fn("mla", "dryft_latent_rows_in")(
+        _ptr(data), kind, stride, n, part_stride, _ptr(w_q), _ptr(c_q), q_rank, _ptr(w_kv), _ptr(c_out), rank, rot_dim,
+        _ptr(cos), _ptr(sin), rot, pairs, float(eps), _ptr(row_slot), _ptr(row_pos), _ptr(pages), _ptr(page_table), max_pages,
+        width, int(bool(write_kv)), rows, is_f32, _stream()), "latent_rows_in")
+
+
+def head_product(x, x_col: int, x_head: int, matrices, k: int, n: int, out, rot_dim: int = 0, tables=None, row_pos=None) -> None:
+    """``out[row, h, :n] = M[h] @ x[row, x_col + h * x_head : + k]`` with ``matrices [heads, n padded to 16, k padded to 32]``
+    (zeros behind), ``out [rows, heads, width]`` contiguous. ``rot_dim`` > 0: the ``rot_dim`` features that follow a head's
+    ``k`` in ``x`` go to ``out[.., n:]``, turned by ``tables = (cos, sin, rotated width, by pairs)``, with zeros up to the
+    width."""
+    _gpu(x, "x")
+    is_f32 = _float_flag(x, "x")
+    _gpu(matrices, "matrices", x.dtype)
+    _gpu(out, "out", x.dtype)
+    rows, heads = x.shape[0], matrices.shape[0]
+    if not (x.dim() == 2 and x.stride(1) == 1 and x_col >= 0 and x_col + (heads - 1) * x_head + k + rot_dim <= x.shape[1]):
+        raise KernelError("head_product: the heads lie outside the columns of x")
+    if not (matrices.dim() == 3 and matrices.is_contiguous() and matrices.shape[1] % 16 == 0 and matrices.shape[2] % 32 == 0 and
+            0 < n <= matrices.shape[1] and 0 < k <= matrices.shape[2] and matrices.data_ptr() % 16 == 0):
+        raise KernelError("head_product: matrices must be contiguous [heads, n padded to 16, k padded to 32]")
+    if not (out.dim() == 3 and out.shape[:2] == (rows, heads) and out.is_contiguous() and out.shape[2] >= n + rot_dim):
+        raise KernelError("head_product: out must be contiguous [rows, heads, >= n + rot_dim]")
+    cos = sin = None
+    rot = pairs = 0
+    if rot_dim:
+        cos, sin, rot, pairs = _turn_tables("head_product", tables, row_pos, rows, rot_dim)
+    _check(_fn("mla", "dryft_head_product")(
+        _ptr(x), x.stride(0), x_col, x_head, _ptr(matrices), k, matrices.shape[2], n, matrices.shape[1], _ptr(out),
+        heads * out.shape[2], out.shape[2], rows, heads, int(rot_dim), _ptr(cos), _ptr(sin), rot, pairs, _ptr(row_pos), is_f32,
+        _stream()), "head_product")
+
+
+def latent_tile_rows(heads: int) -> int:
+    """Rows of a sequence that one workgroup of ``latent_attend`` takes (its tiles, for ``ctx.tiles``)."""
+    return 16 // min(heads, 16)
+
+
+def latent_attend(q, pages, page_table, seq_slot, cu_rows, q_len, seq_start, tile_cu, n_seqs: int, max_tiles: int, row_slot,
+                  row_pos, out, rank: int, scale: float, splits: int) -> None:
+    """Causal attention of ``q [rows, heads, width]`` to the cached rows ``pages [pages, 1, 64, width]``: ``out [rows, heads,
+    rank]`` is the weighted sum of the rows' first ``rank`` numbers. bfloat16 on the matrix cores (a tile of
+    ``latent_tile_rows`` rows of a sequence and one of ``splits`` runs of its pages a workgroup), float32 in plain
+    arithmetic."""
+    _gpu(q, "q")
+    is_f32 = _float_flag(q, "q")
+    width = _latent_pages("latent_attend", pages, page_table, q.dtype)
+    rows, heads = q.shape[:2]
+    if not (q.dim() == 3 and q.shape[2] == width and q.is_contiguous() and q.data_ptr() % 16 == 0):
+        raise KernelError(f"latent_attend: q must be contiguous [rows, heads, {width}]")
+    _gpu(out, "out", q.dtype)
+    if not (out.shape == (rows, heads, rank) and out.is_contiguous() and 0 < rank <= width):
+        raise KernelError("latent_attend: out must be contiguous [rows, heads, rank]")
+    _row_facts(rows, row_slot=row_slot, row_pos=row_pos)
+    if is_f32:
+        _check(_fn("mla", "dryft_latent_attend_f32")(_ptr(q), _ptr(pages), _ptr(page_table), page_table.shape[1], _ptr(row_slot),
+                                                     _ptr(row_pos), _ptr(out), rows, heads, width, rank, float(scale),
+                                                     _stream()), "latent_attend")
+        return
+    _seq_facts(seq_slot, cu_rows, q_len, n_seqs)
+    for name, t, need in (("seq_start", seq_start, n_seqs), ("tile_cu", tile_cu, n_seqs + 1)):
+        _gpu(t, name, torch.int32)
+        if t.numel() < need:
+            raise KernelError(f"{name}: needs {need} entries")
+    part_o = torch.empty((rows, heads, splits, rank), dtype=torch.float32, device=q.device)
+    part_ml = torch.empty((rows, heads, splits, 2), dtype=torch.float32, device=q.device)
+    _check(_fn("mla", "dryft_latent_split")(
+        _ptr(q), _ptr(pages), _ptr(page_table), page_table.shape[1], _ptr(seq_slot), _ptr(cu_rows), _ptr(q_len),
+        _ptr(seq_start), _ptr(tile_cu), n_seqs, max_tiles, _ptr(row_slot), rows, heads, width, rank, float(scale), _ptr(part_o),
+        _ptr(part_ml), int(splits), _ptr(out), _stream()), "latent_attend")

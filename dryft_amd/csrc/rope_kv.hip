@@ -671,7 +671,7 @@ __global__ __launch_bounds__(256) void norm_rope_half_kv_kernel(
     const float* __restrict__ k_w, float eps, const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rot,
     const int* __restrict__ row_slot, const int* __restrict__ row_pos, T* __restrict__ q_out, T* __restrict__ k_pages,
     T* __restrict__ v_pages, const int* __restrict__ page_table, int max_pages, int write_kv, int n_heads, int n_kv,
-    int head_dim, int v_dim, int skip_v, int page_dim) {
+    int head_dim, int v_dim, int skip_v, int page_dim, int unit_after) {
   __shared__ float held[4][NRH_MAX_DIM];
   const int k_wide = page_dim > 0 ? page_dim : head_dim, v_wide = page_dim > 0 ? page_dim : v_dim;
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
@@ -719,17 +719,28 @@ __global__ __launch_bounds__(256) void norm_rope_half_kv_kernel(
   // each lane reads below what another lane of its wave wrote above
   __builtin_amdgcn_fence(__ATOMIC_SEQ_CST, "workgroup");
   __builtin_amdgcn_wave_barrier();
-  for (int i = lane; i < head_dim; i += WAVE) {
+  auto turned = [&](int i) {
     const float x = mine[i] * inv * (w != nullptr ? w[i] : 1.f);
-    float o = x;
-    if (i < rot) {
-      const int j = i < half ? i + half : i - half, f = i < half ? i : i - half;
-      const float other = mine[j] * inv * (w != nullptr ? w[j] : 1.f);
-      const float c = cos_t[(int64_t)pos * half + f], s = sin_t[(int64_t)pos * half + f];
-      o = i < half ? x * c - other * s : x * c + other * s;
-    }
-    store_from_float(dst + i, o);
+    if (i >= rot) return x;
+    const int j = i < half ? i + half : i - half, f = i < half ? i : i - half;
+    const float other = mine[j] * inv * (w != nullptr ? w[j] : 1.f);
+    const float c = cos_t[(int64_t)pos * half + f], s = sin_t[(int64_t)pos * half + f];
+    return i < half ? x * c - other * s : x * c + other * s;
+  };
+  if (!unit_after) {
+    for (int i = lane; i < head_dim; i += WAVE) store_from_float(dst + i, turned(i));
+    return;
   }
+  float o[NRH_MAX_DIM / WAVE], sq = 0.f;
+#pragma unroll
+  for (int n = 0; n < NRH_MAX_DIM / WAVE; ++n) {
+    o[n] = n * WAVE + lane < head_dim ? turned(n * WAVE + lane) : 0.f;
+    sq += o[n] * o[n];
+  }
+  const float unit = rsqrtf(wave_sum(sq) / (float)head_dim + eps);
+#pragma unroll
+  for (int n = 0; n < NRH_MAX_DIM / WAVE; ++n)
+    if (n * WAVE + lane < head_dim) store_from_float(dst + n * WAVE + lane, o[n] * unit);
 }
 
 DRYFT_API int dryft_norm_rope_half_kv(const void* src, int64_t src_stride, int q_col, int k_col, int v_col,
@@ -737,7 +748,7 @@ DRYFT_API int dryft_norm_rope_half_kv(const void* src, int64_t src_stride, int q
                                       const float* sin_t, int rot, const int* row_slot, const int* row_pos, void* q_out,
                                       void* k_pages, void* v_pages, const int* page_table, int max_pages, int write_kv,
                                       int n_rows, int n_heads, int n_kv, int head_dim, int v_dim, int page_dim,
-                                      int is_f32, hipStream_t stream) {
+                                      int unit_after, int is_f32, hipStream_t stream) {
   if (n_rows <= 0) return 0;
   if (rot < 0 || rot % 2 || rot > head_dim || head_dim > NRH_MAX_DIM || n_kv <= 0 || q_out == nullptr) return -1;
   if (page_dim != 0 && (page_dim < head_dim || page_dim < v_dim)) return -1;
@@ -749,12 +760,13 @@ DRYFT_API int dryft_norm_rope_half_kv(const void* src, int64_t src_stride, int q
   if (is_f32)
     hipLaunchKernelGGL(norm_rope_half_kv_kernel<float>, grid, block, 0, stream, (const float*)src, src_stride, q_col,
                        k_col, v_col, q_w, k_w, eps, cos_t, sin_t, rot, row_slot, row_pos, (float*)q_out, (float*)k_pages,
-                       (float*)v_pages, page_table, max_pages, write_kv, n_heads, n_kv, head_dim, v_dim, skip_v, page_dim);
+                       (float*)v_pages, page_table, max_pages, write_kv, n_heads, n_kv, head_dim, v_dim, skip_v, page_dim,
+                       unit_after);
   else
     hipLaunchKernelGGL(norm_rope_half_kv_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)src, src_stride, q_col,
                        k_col, v_col, q_w, k_w, eps, cos_t, sin_t, rot, row_slot, row_pos, (bf16_t*)q_out,
                        (bf16_t*)k_pages, (bf16_t*)v_pages, page_table, max_pages, write_kv, n_heads, n_kv, head_dim,
-                       v_dim, skip_v, page_dim);
+                       v_dim, skip_v, page_dim, unit_after);
   int rc = DRYFT_LAUNCH_CHECK();
   if (rc || !skip_v) return rc;
   dim3 vgrid((n_rows + V_TILE_ROWS - 1) / V_TILE_ROWS, n_kv);

@@ -45,17 +45,20 @@ DRYFT_API int dryft_wkv_blend(const void* h, const float* previous, const float*
 }
 
 // ---------------------------------------------------------------------------------------------------
-// The decay: w = exp(-exp(W_up tanh(low) + bias)), with `low` [rows, rank] the float accumulators of
-// the first projection. R rows a workgroup share each weight row they read; a thread owns outputs n, n + 256, ...
-template <typename W, int R>
+// A decay per key channel from a low-rank projection whose first half left its float accumulators in `low` [rows, rank]:
+//   w = exp(-exp(W_up tanh(low) + bias))                       (LOGSIG false)
+//   w = log(sigmoid(W_up low + bias)) * factor                 (LOGSIG true: the logarithm of sigmoid(.)^factor)
+// R rows a workgroup share each weight row they read; a thread owns outputs n, n + 256, ...
+template <typename W, int R, bool LOGSIG>
 __global__ __launch_bounds__(256) void wkv_decay_kernel(const float* __restrict__ low, const W* __restrict__ up,
                                                         const float* __restrict__ bias, float* __restrict__ decay,
-                                                        int rows, int n_out, int rank) {
+                                                        int rows, int n_out, int rank, float factor) {
   extern __shared__ float t_low[];           // [R][rank]
   const int64_t row0 = (int64_t)blockIdx.x * R;
   for (int i = threadIdx.x; i < R * rank; i += blockDim.x) {
     const int64_t row = row0 + i / rank;
-    t_low[i] = row < rows ? tanhf(low[row * rank + i % rank]) : 0.f;
+    const float x = row < rows ? low[row * rank + i % rank] : 0.f;
+    t_low[i] = LOGSIG ? x : tanhf(x);
   }
   __syncthreads();
   for (int n = blockIdx.y * blockDim.x + threadIdx.x; n < n_out; n += gridDim.y * blockDim.x) {
@@ -82,34 +85,42 @@ __global__ __launch_bounds__(256) void wkv_decay_kernel(const float* __restrict_
     const float b = bias[n];
 #pragma unroll
     for (int r = 0; r < R; ++r)
-      if (row0 + r < rows) decay[(row0 + r) * n_out + n] = expf(-expf(acc[r] + b));
+      if (row0 + r < rows) {
+        const float z = acc[r] + b;
+        // log(sigmoid(z)) = min(z, 0) - log(1 + exp(-|z|))
+        decay[(row0 + r) * n_out + n] = LOGSIG ? (fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * factor : expf(-expf(z));
+      }
   }
+}
+
+template <bool LOGSIG>
+static int launch_decay(const float* low, const void* up, const float* bias, float* decay, int rows, int n_out, int rank,
+                        float factor, int up_is_f32, hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (rank <= 0 || rank > 2048) return -1;
+  const bool many = rows >= 64;
+  const size_t lds = (size_t)(many ? 8 : 1) * rank * sizeof(float);
+  // few rows: a workgroup per 256 outputs, so that the chip has work
+  const dim3 grid = many ? dim3((rows + 7) / 8, 1) : dim3(rows, (n_out + 255) / 256);
+#define DK(WW, R)                                                                                                     \
+  hipLaunchKernelGGL((wkv_decay_kernel<WW, R, LOGSIG>), grid, dim3(256), lds, stream, low, (const WW*)up, bias, decay,   \
+                     rows, n_out, rank, factor)
+  if (many && up_is_f32) DK(float, 8);
+  else if (many) DK(bf16_t, 8);
+  else if (up_is_f32) DK(float, 1);
+  else DK(bf16_t, 1);
+#undef DK
+  return DRYFT_LAUNCH_CHECK();
 }
 
 DRYFT_API int dryft_wkv_decay(const float* low, const void* up, const float* bias, float* decay, int rows, int n_out,
                               int rank, int up_is_f32, hipStream_t stream) {
-  if (rows <= 0) return 0;
-  if (rank <= 0 || rank > 2048) return -1;
-  if (rows >= 64) {
-    const size_t lds = (size_t)8 * rank * sizeof(float);
-    dim3 grid((rows + 7) / 8, 1);
-    if (up_is_f32)
-      hipLaunchKernelGGL((wkv_decay_kernel<float, 8>), grid, dim3(256), lds, stream, low, (const float*)up, bias, decay,
-                         rows, n_out, rank);
-    else
-      hipLaunchKernelGGL((wkv_decay_kernel<bf16_t, 8>), grid, dim3(256), lds, stream, low, (const bf16_t*)up, bias, decay,
-                         rows, n_out, rank);
-  } else {
-    const size_t lds = (size_t)rank * sizeof(float);
-    dim3 grid(rows, (n_out + 255) / 256);          // few rows: a workgroup per 256 outputs, so that the chip has work
-    if (up_is_f32)
-      hipLaunchKernelGGL((wkv_decay_kernel<float, 1>), grid, dim3(256), lds, stream, low, (const float*)up, bias,
-                         decay, rows, n_out, rank);
-    else
-      hipLaunchKernelGGL((wkv_decay_kernel<bf16_t, 1>), grid, dim3(256), lds, stream, low, (const bf16_t*)up, bias,
-                         decay, rows, n_out, rank);
-  }
-  return DRYFT_LAUNCH_CHECK();
+  return launch_decay<false>(low, up, bias, decay, rows, n_out, rank, 1.f, up_is_f32, stream);
+}
+
+DRYFT_API int dryft_log_decay(const float* low, const void* up, const float* bias, float* decay, int rows, int n_out,
+                              int rank, float factor, int up_is_f32, hipStream_t stream) {
+  return launch_decay<true>(low, up, bias, decay, rows, n_out, rank, factor, up_is_f32, stream);
 }
 
 // ---------------------------------------------------------------------------------------------------

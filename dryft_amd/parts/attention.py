@@ -22,8 +22,9 @@ positions, runs counted from position 0); a learned bias by distance added to th
 half on a logarithmic scale that reaches the last row at ``far``); one output gate per head instead of one per
 feature (``output_gate="head"``); and values that lean on those of an earlier layer (``value_mix = (name, first)``:
 the first layer of that name leaves its values of the step's rows in the step context, every later one takes ``(1 -
-l) v + l v_first`` with its own learned ``l``, tensor ``vmix``, before anything is cached). Any of these takes the
-step down ``_forward_general``.
+l) v + l v_first`` with its own learned ``l``, tensor ``vmix``, before anything is cached); and q and k divided by their
+root mean square per head after the rotation, without a weight (``qk_unit_eps``). Any of these takes the step down
+``_forward_general``.
 
 ``pad_pages``: in bfloat16, heads whose keys and values differ in width (or whose width is no multiple of 16) keep
 pages of one width for both, the next multiple of 16 that holds either, with zeros behind a head's own features: the
@@ -84,7 +85,7 @@ class GQAAttention(Mixer):
                  float_weights: bool = False, bias: bool = False, conv_taps: int | None = None,
                  sink_value: float | None = None, chunk: int | None = None,
                  distance_bias: tuple[int, int] | None = None, value_mix: tuple[str, bool] | None = None,
-                 pad_pages: bool = False):
+                 pad_pages: bool = False, qk_unit_eps: float | None = None):
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} query heads cannot share {num_kv_heads} kv heads evenly")
         if not 0 < head_dim <= MAX_HEAD_DIM:
@@ -117,8 +118,9 @@ class GQAAttention(Mixer):
                              f"distance beyond half of them, got {self.distance_bias}")
         self.value_mix = (str(value_mix[0]), bool(value_mix[1])) if value_mix else None
         self.pad_pages = bool(pad_pages)
-        if self.pad_pages and positions:
-            raise ValueError("pages of one padded width go with mixers that do not rotate")
+        self.qk_unit_eps = None if qk_unit_eps is None else float(qk_unit_eps)
+        if self.qk_unit_eps is not None and qk_norm_eps is not None:
+            raise ValueError("q and k are normed before the rotation (qk_norm_eps) or after it (qk_unit_eps), not both")
         self.q_dim, self.kv_dim = self.n_heads * self.head_dim, self.n_kv * self.head_dim
         self.v_dim, self.o_dim = self.n_kv * self.value_dim, self.n_heads * self.value_dim
         self.has_bias, self.conv_taps = bool(bias), int(conv_taps) if conv_taps else 0
@@ -127,7 +129,7 @@ class GQAAttention(Mixer):
         self.g_dim = (self.n_heads if self.head_gate else self.o_dim) if self.output_gate else 0
         self.extended = bool(self.value_dim != self.head_dim or self.softcap or self.has_sink or self.output_gate or
                              self.float_weights or self.has_bias or self.conv_taps or self.sink_value is not None or
-                             self.chunk or self.distance_bias or self.value_mix)
+                             self.chunk or self.distance_bias or self.value_mix or self.qk_unit_eps is not None)
         self.conv_channels = self.q_dim + self.kv_dim + self.v_dim
         self.w_qkv = self.w_o = self.q_norm = self.k_norm = self.sink = None
         self.in_bias = self.o_bias = self.conv_w = self.conv_wt = self.rel = self.vmix = self.w_o_padded = None
@@ -253,14 +255,16 @@ class GQAAttention(Mixer):
         q = torch.zeros((rows, H, wide), dtype=h.dtype, device=h.device) if wide else \
             torch.empty((rows, H, D), dtype=h.dtype, device=h.device)
         if isinstance(table, PairRotaryPositions):
-            if self.qk_norm_eps is not None:
-                raise NotImplementedError("per-head q/k norms do not go with the rotation over neighbouring pairs")
+            if self.qk_norm_eps is not None or self.qk_unit_eps is not None or wide:
+                raise NotImplementedError("per-head q/k norms and padded pages do not go with the rotation over "
+                                          "neighbouring pairs")
             ops.rope_pairs_kv(src, 0, self.q_dim, self.q_dim + self.kv_dim, cos, sin, rot, ctx.row_slot, ctx.row_pos, q,
                               line.k, line.v, line.page_table, writes_cache, H, G, D, Dv)
         else:
             ops.norm_rope_half_kv(src, 0, self.q_dim, self.q_dim + self.kv_dim, self.q_norm, self.k_norm,
-                                  self.qk_norm_eps or 0.0, cos, sin, rot, ctx.row_slot, ctx.row_pos, q, line.k, line.v,
-                                  line.page_table, writes_cache, H, G, D, Dv, page_dim=wide)
+                                  self.qk_unit_eps or self.qk_norm_eps or 0.0, cos, sin, rot, ctx.row_slot, ctx.row_pos, q,
+                                  line.k, line.v, line.page_table, writes_cache, H, G, D, Dv, page_dim=wide,
+                                  unit_after=self.qk_unit_eps is not None)
         # bfloat16 on the matrix cores where they take the sizes (keys and values of one width, a multiple of 16, as
         # they are or padded); float32, and the other sizes, on the kernel that takes one (row, head) a workgroup
         matrix_cores = h.dtype == torch.bfloat16 and (wide or (D == Dv and D % MATRIX_CORE_HEAD_STEP == 0))

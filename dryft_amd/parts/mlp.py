@@ -9,8 +9,9 @@ from __future__ import annotations
 import torch
 
 from ..csrc import ops
+from ..weights.spec import VECTOR
 from . import register_part
-from .base import FeedForward, matrix
+from .base import FeedForward, Partials, matrix
 from .linear import STREAM_ROWS, few_rows_ok, linear, panel_swiglu_ok, tall_swiglu_ok
 
 
@@ -98,6 +99,34 @@ class SquaredReLU(FeedForward):
         return linear(act, self.w_down, allow_partials=True)
 
 
+class PolyNormMLP(FeedForward):
+    """``down( c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3 )`` with ``z = up(h)``, powers element by element and ``N`` the division
+    of a token's vector by its root mean square (``eps`` inside the root); dense, no bias. Tensor ``act`` holds the four
+    numbers. ``z`` reaches the polynomial as the float partial sums of its product where that is split over K."""
+
+    def __init__(self, hidden_size: int, intermediate_size: int, eps: float):
+        self.hidden, self.inter, self.eps = int(hidden_size), int(intermediate_size), float(eps)
+        self.w_up = self.w_down = self.act = None
+
+    def tensor_specs(self):
+        return {"up_proj": matrix((self.inter, self.hidden)), "down_proj": matrix((self.hidden, self.inter)),
+                "act": ((4,), VECTOR, "ones")}
+
+    def load(self, tensors):
+        self.w_up, self.w_down = tensors["up_proj"], tensors["down_proj"]
+        self.act = tensors["act"].float().contiguous()
+
+    def kernel_modules(self, dtype):
+        return ("gemm", "activation")
+
+    def forward(self, h, ctx):
+        z = linear(h, self.w_up, allow_partials=True)
+        act = torch.empty((h.shape[0], self.inter), dtype=h.dtype, device=h.device)
+        ops.poly_norm((z.data, z.count) if isinstance(z, Partials) else z, self.act, self.eps, act)
+        return linear(act, self.w_down, allow_partials=True)
+
+
 register_part("swiglu", SwiGLU)
+register_part("poly_norm_mlp", PolyNormMLP)
 register_part("squared_relu", SquaredReLU)
 register_part("clamped_glu", ClampedGLU)

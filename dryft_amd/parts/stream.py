@@ -33,13 +33,17 @@ from .linear import linear
 
 class StreamRMSNorm(Norm):
     """``offset``: what the stored weight is counted from (1 for weights stored around zero); ``scale``: a factor on
-    the whole weight (a head's factor on its logits rides here). A stream of several copies ``[copies, rows, width]``
+    the whole weight (a head's factor on its logits rides here); ``groups``: the norm is taken in so many equal consecutive
+    parts of the vector, each divided by its own root mean square. A stream of several copies ``[copies, rows, width]``
     (``parts/hyper.py``) is normed as the sum of its copies."""
 
     centred = False           # does the norm take the mean off first (a layer norm without bias)?
 
-    def __init__(self, size: int, eps: float, offset: float = 0.0, scale: float = 1.0):
+    def __init__(self, size: int, eps: float, offset: float = 0.0, scale: float = 1.0, groups: int = 1):
         self.size, self.eps, self.offset, self.scale = int(size), float(eps), float(offset), float(scale)
+        self.groups = int(groups)
+        if not 1 <= self.groups <= ops.STREAM_NORM_MAX_GROUPS or self.size % self.groups:
+            raise ValueError(f"{size} values do not split into {groups} equal parts (1..{ops.STREAM_NORM_MAX_GROUPS})")
         self.weight: torch.Tensor | None = None
 
     def tensor_specs(self):
@@ -55,7 +59,8 @@ class StreamRMSNorm(Norm):
         if x.dim() == 3:
             return self.add_forward(x, None, dtype)[1]
         y = torch.empty(x.shape, dtype=dtype or self.compute_dtype or x.dtype, device=x.device)
-        ops.stream_norm(x, None, None, None, None, self.weight, self.eps, None, y, y.dtype, centred=self.centred)
+        ops.stream_norm(x, None, None, None, None, self.weight, self.eps, None, y, y.dtype, centred=self.centred,
+                        groups=self.groups)
         return y
 
     def add_forward(self, res: torch.Tensor, delta, dtype: torch.dtype | None = None, in_place: bool = True):
@@ -65,12 +70,14 @@ class StreamRMSNorm(Norm):
         pending = as_deferred(delta)
         act = dtype or self.compute_dtype or _activation_dtype(res, pending)
         if res.dim() == 3 or pending.route is not None:
+            if self.groups > 1:
+                raise NotImplementedError("a norm in parts does not go with a stream of several copies")
             from .hyper import read_streams
             return read_streams(res, pending, None, self, act, keep=False)
         own = in_place and res.dtype == torch.float32 and res.is_contiguous()
         out = res if own else torch.empty(res.shape, dtype=torch.float32, device=res.device)
         y = torch.empty(res.shape, dtype=act, device=res.device)
-        _launch(res, pending, self.weight, self.eps, out, y, act, centred=self.centred)
+        _launch(res, pending, self.weight, self.eps, out, y, act, centred=self.centred, groups=self.groups)
         return out, y
 
 
@@ -95,15 +102,19 @@ def _activation_dtype(x: torch.Tensor, pending: Deferred) -> torch.dtype:
     return x.dtype
 
 
-def _launch(x, pending: Deferred, weight, eps, x_out, y, act, centred: bool = False, plain_read: bool = False) -> None:
+def _launch(x, pending: Deferred, weight, eps, x_out, y, act, centred: bool = False, plain_read: bool = False,
+            groups: int = 1) -> None:
     delta = pending.delta
     if isinstance(delta, Partials):
         delta = (delta.data, delta.count)
     post = pending.norm.weight if pending.norm is not None else None
+    if getattr(pending.norm, "groups", 1) > 1:
+        raise NotImplementedError("a norm in parts stands in front of a reader, not behind a sublayer")
     if pending.norm is not None and pending.norm.eps != eps:
         raise ValueError("the norms around one residual sum differ in eps; one launch takes one")
     ops.stream_norm(x, delta, post, pending.rows, pending.vector, weight, eps, x_out, y, act,
-                    post_centred=bool(getattr(pending.norm, "centred", False)), centred=centred, plain_read=plain_read)
+                    post_centred=bool(getattr(pending.norm, "centred", False)), centred=centred, plain_read=plain_read,
+                    groups=groups)
 
 
 def read_plain(x: torch.Tensor, pending, act: torch.dtype):
