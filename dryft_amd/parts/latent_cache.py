@@ -120,18 +120,19 @@ class CachedLatentAttention(Mixer):
         rows, H = h.shape[0], self.n_heads
         tables = self._tables(ctx)
         # only steps that the host knows have so many rows, and what their sequences start from is part of the step
-        expand = self._page_dim() > 0 and ctx.max_q_len > 1 and rows > _EXPANDED_FROM and ctx.host is not None and \
+        many = h.dtype == torch.bfloat16 and ctx.max_q_len > 1 and rows > _EXPANDED_FROM and ctx.host is not None and \
             not any(start for slot, start in zip(ctx.host.slots, ctx.host.starts) if slot >= 0)
-        down = linear(h, self.w_down, allow_partials=not expand)
+        leaves = many and self.own_latent
+        down = linear(h, self.w_down, allow_partials=not leaves)
         c_q = torch.empty((rows, self.q_rank), dtype=h.dtype, device=h.device)
-        c_kv = torch.empty((rows, self.kv_rank), dtype=h.dtype, device=h.device) if expand and self.own_latent else None
+        c_kv = torch.empty((rows, self.kv_rank), dtype=h.dtype, device=h.device) if leaves else None
         ops.latent_rows_in((down.data, down.count) if isinstance(down, Partials) else down, self.q_norm, c_q,
                            self.kv_norm, c_kv, self.rot_dim, tables, self.norm_eps, ctx.row_slot, ctx.row_pos, line.k,
                            line.page_table, writes_cache)
         q_raw = linear(c_q, self.w_uq)
-        if expand:
-            if self.own_latent:
-                ctx.shared["latent:" + self.name] = (c_kv, down, self.q_rank + self.kv_rank)
+        if leaves:
+            ctx.shared["latent:" + self.name] = (c_kv, down, self.q_rank)
+        if many and self._page_dim():
             return self._with_keys(q_raw, ctx, tables)
         q = torch.empty((rows, H, self.width), dtype=h.dtype, device=h.device)
         ops.head_product(q_raw, 0, self.key_dim, self.w_absorb, self.plain, self.kv_rank, q, self.rot_dim, tables, ctx.row_pos)
@@ -154,7 +155,7 @@ class CachedLatentAttention(Mixer):
         found = ctx.shared.get("latent:" + self.name)
         if found is None or found[0].shape != (rows, self.kv_rank):
             raise ValueError(f"latent {self.name!r}: no earlier layer of this step has left one of this width")
-        c_kv, down, rot_col = found
+        c_kv, down, lat_col = found                                         # of the layer that writes the line
         table, n_pages = self._step_pages(ctx)
         wide = self._page_dim()
         # zeros once a step: a layer's pages are overwritten by the next one's, finite wherever no row is
@@ -164,7 +165,7 @@ class CachedLatentAttention(Mixer):
         kv = linear(c_kv, w_ukv)                                            # plain keys of all heads | values of all heads
         q = torch.empty((rows, H, wide), dtype=q_raw.dtype, device=dev)
         cos, sin, rot, pairs = tables if tables is not None else (None, None, 0, False)
-        ops.latent_rope_kv(q_raw, kv, down, rot_col, cos, sin, rot, ctx.row_slot, ctx.row_pos, q, k, v, table, True, H,
+        ops.latent_rope_kv(q_raw, kv, down, lat_col + self.kv_rank, cos, sin, rot, ctx.row_slot, ctx.row_pos, q, k, v, table, True, H,
                            self.plain, self.rot_dim, self.value_dim, wide, pairs=pairs, page_dk=wide)
         out = ctx.kept_zeros((rows, H, wide), q_raw.dtype) if ctx.some_sit_out() else \
             torch.empty((rows, H, wide), dtype=q_raw.dtype, device=dev)
