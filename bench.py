@@ -135,7 +135,9 @@ def compare_fetedra(args, design: str = "fetedra", relative: str = "piralix") ->
     ``--prompt-len`` tokens and ``--batch`` sequences decoding. One JSON line. ``--design barilix`` does the same for
     Barilix beside the Fetedra preset of the same width (recurrent and windowed-attention layers with experts on a
     float32 stream, as many layers of the same widths), ``--design podenex`` for Podenex beside it (three kinds of
-    windowed or chunked attention, one of them Fetedra's latent kind, with routed experts on a float32 stream)."""
+    windowed or chunked attention, one of them Fetedra's latent kind, with routed experts on a float32 stream),
+    ``--design fubinex`` for Fubinex beside Barilix (attention and a recurrence side by side, and a second recurrent
+    kind, on a float32 stream)."""
     import torch
 
     from dryft_amd import Engine
@@ -163,9 +165,10 @@ def compare_fetedra(args, design: str = "fetedra", relative: str = "piralix") ->
 def main() -> int:
     global PROMPT, SLOT
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", default=None, choices=["piralix", "fetedra", "barilix", "podenex"],
+    ap.add_argument("--design", default=None, choices=["piralix", "fetedra", "barilix", "podenex", "fubinex"],
                     help="instead of the default workload: that design beside its closest relative in the library at "
-                         "equal size (Piralix beside Qwen3, Fetedra beside Piralix, Barilix and Podenex beside Fetedra; one JSON line)")
+                         "equal size (Piralix beside Qwen3, Fetedra beside Piralix, Barilix and Podenex beside Fetedra, Fubinex beside "
+                         "Barilix; one JSON line)")
     ap.add_argument("--sizes", default=None, help="presets for --design (default: the design's presets)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=128)
@@ -190,9 +193,12 @@ def main() -> int:
         args.sizes = args.sizes or {"piralix": "piralix-w1024,piralix-w2048,piralix-w2560",
                                     "fetedra": "fetedra-w1024,fetedra-w2048",
                                     "barilix": "barilix-w1024,barilix-w2048",
-                                    "podenex": "podenex-w1024,podenex-w2048"}[args.design]
+                                    "podenex": "podenex-w1024,podenex-w2048",
+                                    "fubinex": "fubinex-w1024,fubinex-w2048"}[args.design]
         if args.design in ("barilix", "podenex"):
             return compare_fetedra(args, args.design, "fetedra")
+        if args.design == "fubinex":
+            return compare_fetedra(args, "fubinex", "barilix")
         return compare_fetedra(args) if args.design == "fetedra" else compare_designs(args)
     if args.gpus != 1:
         print(f"bench.py measures one GPU only (asked for {args.gpus}); this library has no multi-GPU path")

@@ -21,7 +21,8 @@
 
 #define LIN_CHUNK 16
 #define LIN_MAX_DIM 256
-#define LIN_STRONG (-60.f)
+#define LIN_STRONG (-86.f)               // in powers of two, as all logarithms inside the chunk kernel
+#define LIN_LOG2E 1.4426950408889634f
 
 // Feature i of a head turned by the row's position: feature i of the first `rot` with feature i + rot/2.
 template <typename T>
@@ -190,37 +191,44 @@ __global__ __launch_bounds__(256) void linattn_chunk_kernel(
       S[m][r] = (MODE != 1 && i < D && col < Dv) ? s_from[(int64_t)i * Dv + col] : 0.f;
     }
   const int ch = tid % DP, part = tid / DP;                         // the thread's channel, its run of TT tokens
-  const float hl = CHAN ? 0.f : ld_head[head];
+  const float hl = CHAN ? 0.f : ld_head[head] * LIN_LOG2E;
   const int half = rot / 2, twin = ch < half ? ch + half : ch - half, freq = ch < half ? ch : ch - half;
   const bool turns = ROT && ch < rot;
-  float fq[TT], fk[TT], fq2[TT], fk2[TT], fc[TT], fs[TT], fl[LIN_CHUNK], fv[4];
+  const float sign = ch < half ? -1.f : 1.f;
+  // What a chunk brings stays as it was loaded until it is used (a conversion here would wait for the loads), and every
+  // load goes to a place that exists: a token beyond the last reads the last, a channel beyond D the last.
+  const int chc = min(ch, D - 1), twc = turns ? twin : chc, frc = turns ? freq : 0, vcc = min(col, Dv - 1);
+  const int step = (int)stride, wide = H * D;
+  const T* base = proj + first * stride;
+  const int64_t pos0 = ROT ? row_pos[first] : 0;                    // a sequence's rows stand at consecutive positions
+  T fq[TT], fk[TT], fq2[TT], fk2[TT], fv[4];
+  float fc[TT], fs[TT], fl[LIN_CHUNK];
   auto fetch = [&](int t0) {
+    const int last = n - 1 - t0;
+    const T* qc = base + (int64_t)t0 * stride + q_col + head * D;
+    const T* kc = base + (int64_t)t0 * stride + k_col + head * D;
+    const T* vc = base + (int64_t)t0 * stride + v_col + head * Dv;
+    const float* cc = cos_t + (pos0 + t0) * half;
+    const float* sc = sin_t + (pos0 + t0) * half;
 #pragma unroll
     for (int u = 0; u < TT; ++u) {
-      const int t = t0 + part * TT + u;
-      const bool in = t < n && ch < D;
-      const T* p = proj + (first + (in ? t : 0)) * stride + head * D;
-      if (MODE != 1) fq[u] = in ? load_as_float(p + q_col + ch) : 0.f;
-      fk[u] = in ? load_as_float(p + k_col + ch) : 0.f;
+      const int t = min(part * TT + u, last);
+      if (MODE != 1) fq[u] = qc[t * step + chc];
+      fk[u] = kc[t * step + chc];
       if (ROT) {
-        const bool both = in && turns;
-        const int64_t pos = both ? row_pos[first + t] : 0;
-        if (MODE != 1) fq2[u] = both ? load_as_float(p + q_col + twin) : 0.f;
-        fk2[u] = both ? load_as_float(p + k_col + twin) : 0.f;
-        fc[u] = both ? cos_t[pos * half + freq] : 1.f;
-        fs[u] = both ? (ch < half ? -1.f : 1.f) * sin_t[pos * half + freq] : 0.f;
+        if (MODE != 1) fq2[u] = qc[t * step + twc];
+        fk2[u] = kc[t * step + twc];
+        fc[u] = cc[t * half + frc];
+        fs[u] = sc[t * half + frc];
       }
     }
     if (CHAN) {
+      const float* lc = ld + (first + t0) * wide + head * D;
 #pragma unroll
-      for (int t = 0; t < LIN_CHUNK; ++t)
-        fl[t] = (t0 + t < n && ch < D) ? ld[((first + t0 + t) * H + head) * D + ch] : 0.f;
+      for (int t = 0; t < LIN_CHUNK; ++t) fl[t] = lc[min(t, last) * wide + chc];
     }
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int t = t0 + 4 * g + j;
-      fv[j] = (t < n && col < Dv) ? load_as_float(proj + (first + t) * stride + v_col + head * Dv + col) : 0.f;
-    }
+    for (int j = 0; j < 4; ++j) fv[j] = vc[min(4 * g + j, last) * step + vcc];
   };
   float total = 0.f;
   fetch(0);
@@ -231,31 +239,45 @@ __global__ __launch_bounds__(256) void linattn_chunk_kernel(
     float* Kh = Qt + LIN_CHUNK * LD;                                // [16][LD]
     float* Kt = Kh + LIN_CHUNK * LD;                                // [DP][LIN_KT]
     float* eb = Kt + DP * LIN_KT;                                   // [DP]
+    const int left = n - t0;                                        // tokens of the sequence from here on
     {
       float own[TT], run = 0.f;
 #pragma unroll
       for (int t = 0; t < LIN_CHUNK; ++t) {
-        run += CHAN ? fl[t] : (t0 + t < n ? hl : 0.f);
+        if (t < left) run += CHAN ? fl[t] * LIN_LOG2E : hl;
         if (t / TT == part) own[t % TT] = run;
       }
+      const float grow = __builtin_amdgcn_exp2f(-run);              // k^ = k~ e^(-b_16)
+      float kt[TT];
 #pragma unroll
       for (int u = 0; u < TT; ++u) {
         const int t = part * TT + u;
-        const float k = (ROT ? fk[u] * fc[u] + fk2[u] * fs[u] : fk[u]) * k_scale;
+        const bool in = t < left && ch < D;
+        float k = load_as_float(&fk[u]);
+        if (ROT && turns) k = k * fc[u] + load_as_float(&fk2[u]) * (sign * fs[u]);
+        kt[u] = in ? k * k_scale * __builtin_amdgcn_exp2f(run - own[u]) : 0.f;
         if (MODE != 1) {
-          const float q = (ROT ? fq[u] * fc[u] + fq2[u] * fs[u] : fq[u]) * q_scale;
-          Qt[t * LD + ch] = q * expf(own[u]);
-          Kh[t * LD + ch] = k * expf(-own[u]);
+          float q = load_as_float(&fq[u]);
+          if (ROT && turns) q = q * fc[u] + load_as_float(&fq2[u]) * (sign * fs[u]);
+          Qt[t * LD + ch] = in ? q * q_scale * __builtin_amdgcn_exp2f(own[u]) : 0.f;
+          Kh[t * LD + ch] = kt[u] * grow;
         }
-        Kt[ch * LIN_KT + t] = k * expf(run - own[u]);
       }
-      if (part == 0) eb[ch] = expf(run);
+      if constexpr (TT % 4 == 0) {
+#pragma unroll
+        for (int u = 0; u < TT; u += 4)
+          *(vf4*)(Kt + ch * LIN_KT + part * TT + u) = vf4{kt[u], kt[u + 1], kt[u + 2], kt[u + 3]};
+      } else {
+#pragma unroll
+        for (int u = 0; u < TT; ++u) Kt[ch * LIN_KT + part * TT + u] = kt[u];
+      }
+      if (part == 0) eb[ch] = __builtin_amdgcn_exp2f(run);
       if (MODE == 1) total += run;
-      if (MODE != 1 && run < LIN_STRONG) strong[flag] = 1;
+      if (MODE != 1 && ch < D && run < LIN_STRONG) strong[flag] = 1;
     }
     vf4 v;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) v[j] = fv[j];
+    for (int j = 0; j < 4; ++j) v[j] = 4 * g + j < left && col < Dv ? load_as_float(&fv[j]) : 0.f;
     __syncthreads();
     if (tid == 0) strong[flag == 0 ? 2 : flag - 1] = 0;             // read by everyone before this barrier, set after the next
     if (t0 + LIN_CHUNK < n) fetch(t0 + LIN_CHUNK);
@@ -284,7 +306,7 @@ __global__ __launch_bounds__(256) void linattn_chunk_kernel(
           for (int i = 0; i < D; ++i) {
             float run = 0.f, bt = 0.f, bs[4] = {0.f, 0.f, 0.f, 0.f};
             for (int t = 0; t <= c; ++t) {
-              run += CHAN ? ld[((first + t0 + t) * H + head) * D + i] : hl;
+              run += CHAN ? ld[((first + t0 + t) * H + head) * D + i] * LIN_LOG2E : hl;
 #pragma unroll
               for (int r = 0; r < 4; ++r)
                 if (t == 4 * g + r) bs[r] = run;
@@ -295,7 +317,7 @@ __global__ __launch_bounds__(256) void linattn_chunk_kernel(
             for (int r = 0; r < 4; ++r)
               if (4 * g + r <= c) {
                 const T* pk = proj + (first + t0 + 4 * g + r) * stride + head * D;
-                a[r] += q * turned(pk + k_col, i, rot, cos_t, sin_t, pos + 4 * g + r) * k_scale * expf(bt - bs[r]);
+                a[r] += q * turned(pk + k_col, i, rot, cos_t, sin_t, pos + 4 * g + r) * k_scale * __builtin_amdgcn_exp2f(bt - bs[r]);
               }
           }
         }
@@ -318,7 +340,7 @@ __global__ __launch_bounds__(256) void linattn_chunk_kernel(
     }
   }
   if (MODE == 1 && blockIdx.z == 0 && part == 0 && ch < D)
-    seg_decay[((int64_t)blockIdx.x * H + head) * D + ch] = expf(total);
+    seg_decay[((int64_t)blockIdx.x * H + head) * D + ch] = __builtin_amdgcn_exp2f(total);
   if (MODE == 2 && seg != n_segs - 1) return;                       // the last segment leaves the sequence's state
   if (MODE != 1 && !write_state) return;
   float* s_to = MODE == 1 ? s_seg : s_mine;

@@ -13,7 +13,7 @@ typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 typedef __attribute__((ext_vector_type(8))) uint16_t u16x8;
 #define MFMA16(a, b, c) __builtin_amdgcn_mfma_f32_16x16x32_bf16((a), (b), (c), 0, 0, 0)
 
-#define MLA_MAX_WIDTH 960          // a page, a tile of queries and its weights fit the 160 KB of LDS up to here
+#define MLA_MAX_WIDTH 960          // features of a cached row; half a page and a tile of queries wait in LDS
 
 // ---------------------------------------------------------------------------------------------------
 // What a step's rows bring: `src` holds, per row, the queries' latent | the keys' latent | the key part to be rotated (the
@@ -34,7 +34,15 @@ __global__ __launch_bounds__(256) void latent_rows_in_kernel(
   float sq = 0.f, sk = 0.f;
   for (int i = threadIdx.x; i < total; i += blockDim.x) {
     float v = 0.f;
-    for (int p = 0; p < n_partials; ++p) v += load_as_float(src + p * partial_stride + row * stride + i);
+    int p = 0;
+    for (; p + 4 <= n_partials; p += 4) {                            // four loads in flight; added in the order 0, 1, ...
+      float t[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) t[u] = load_as_float(src + (p + u) * partial_stride + row * stride + i);
+#pragma unroll
+      for (int u = 0; u < 4; ++u) v += t[u];
+    }
+    for (; p < n_partials; ++p) v += load_as_float(src + p * partial_stride + row * stride + i);
     held[i] = v;
     if (i < q_rank) sq += v * v;
     else if (i < q_rank + rank) sk += v * v;
@@ -137,6 +145,7 @@ __global__ __launch_bounds__(256) void head_product_kernel(
   const bf16_t* xr = x + row * x_stride + x_col + (int64_t)head * x_head;
   const bf16_t* mr = m + ((int64_t)head * Np + n0 + c) * Kp + 8 * g;
   vf4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 8
   for (int k0 = 0; k0 < Kp; k0 += 32) {
     const int k = k0 + 8 * g;
     const bf16x8 a = *(const bf16x8*)(mr + k0);
@@ -200,11 +209,16 @@ DRYFT_API int dryft_head_product(const void* x, int64_t x_stride, int x_col, int
 
 // ---------------------------------------------------------------------------------------------------
 // bfloat16: a workgroup takes a tile of up to 16 (row, head) pairs of one sequence (all heads of one row, or several
-// rows' where a row has few) and one run of the sequence's pages. The pairs are the 16 columns of both products: S^T = K
-// Q^T, where a wave takes 16 of a page's 64 positions, and O^T = C^T P^T, where the waves deal out the latent's features.
-// A page lies in LDS row by row; the second product's first operand gathers 8 positions of a feature from it. Each
-// run of pages leaves its maximum, sum and weighted sum of latents (float); `latent_combine` joins them in order.
-template <int NT>
+// rows' where a row has few) and one run of the sequence's half pages (32 positions). The pairs are the 16 columns of both
+// products. S^T = K Q^T: a wave takes 16 of the 32 positions and half of the features, and leaves its part of the scores
+// in LDS, from where every lane takes the scores of exactly the 8 positions that it contributes to the second product,
+// O^T = C^T P^T, whose features the waves deal out among themselves. Half a page lies in LDS row by row; the second
+// product's first operand gathers 8 positions of a feature from it. The next half page's loads are in flight
+// meanwhile. Each run leaves its maximum, sum and weighted sum of latents (float); `latent_combine` joins them in order.
+#define LATENT_KEYS 32
+
+// NT: feature tiles of 16 a wave owns at most; NL: 16-byte pieces of half a page a thread brings in at most
+template <int NT, int NL>
 __global__ __launch_bounds__(256) void latent_split_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ pages, const int* __restrict__ page_table, int max_pages,
     const int* __restrict__ seq_slot, const int* __restrict__ cu_rows, const int* __restrict__ q_len,
@@ -212,10 +226,9 @@ __global__ __launch_bounds__(256) void latent_split_kernel(
     float* __restrict__ part_o, float* __restrict__ part_ml, int splits) {
   extern __shared__ __attribute__((aligned(16))) char lds_raw[];
   const int ws = width + 8;
-  bf16_t* page_s = (bf16_t*)lds_raw;                     // [64][ws]
-  bf16_t* q_s = page_s + 64 * ws;                        // [16][ws]
-  bf16_t* p_s = q_s + 16 * ws;                           // [16][72]
-  float* red = (float*)(p_s + 16 * 72);                  // [4][16]
+  vf4* s_part = (vf4*)lds_raw;                           // [4 waves][64 lanes]
+  bf16_t* page_s = (bf16_t*)(s_part + 256);              // [32][ws]
+  bf16_t* q_s = page_s + LATENT_KEYS * ws;               // [16][ws]
   if ((int)blockIdx.x >= tile_cu[n_seqs]) return;
   int seq = 0;
   while (tile_cu[seq + 1] <= (int)blockIdx.x) ++seq;
@@ -229,9 +242,19 @@ __global__ __launch_bounds__(256) void latent_split_kernel(
   const bool live = c / hc < rt && my_row < rows_here && my_head < H;
   const int my_pos = start + my_row;
   const int last_pos = start + min(r0 + rt, rows_here) - 1;
-  const int n_pages = last_pos / PAGE_TOKENS + 1, per = (n_pages + splits - 1) / splits;
-  const int first_page = blockIdx.z * per, end_page = min(n_pages, first_page + per);
-  const int chunks = width / 8;
+  const int n_halves = last_pos / LATENT_KEYS + 1, per = (n_halves + splits - 1) / splits;
+  const int begin = blockIdx.z * per, end = min(n_halves, begin + per);
+  const int chunks = width / 8, pieces = LATENT_KEYS * chunks;
+  vu4 next[NL];
+  int page_ok = 0;
+  auto fetch = [&](int half) {                                       // rows of a page lie end to end
+    const int page = page_table[(int64_t)slot * max_pages + half / 2];
+    page_ok = page >= 0;
+    const vu4* src = (const vu4*)(pages + ((int64_t)(page < 0 ? 0 : page) * PAGE_TOKENS + half % 2 * LATENT_KEYS) * width);
+#pragma unroll
+    for (int u = 0; u < NL; ++u) next[u] = src[min(tid + 256 * u, pieces - 1)];
+  };
+  if (begin < end) fetch(begin);
   for (int e = tid; e < 16 * chunks; e += 256) {                     // the tile's queries, zeros for columns without a pair
     const int col = e / chunks, k = (e % chunks) * 8;
     const int row = r0 + col / hc, head = h0 + col % hc;
@@ -242,101 +265,151 @@ __global__ __launch_bounds__(256) void latent_split_kernel(
   vf4 O[NT];
 #pragma unroll
   for (int t = 0; t < NT; ++t) O[t] = vf4{0.f, 0.f, 0.f, 0.f};
+  const int blocks = width / 32, k_from = wave < 2 ? 0 : blocks / 2, k_to = wave < 2 ? blocks / 2 : blocks;
+  const bf16_t* k_row = page_s + (16 * (wave & 1) + c) * ws + 8 * g;
+  const bf16_t* q_row = q_s + c * ws + 8 * g;
   float m = -INFINITY, l = 0.f;
-  for (int pg = first_page; pg < end_page; ++pg) {
-    const int page = page_table[(int64_t)slot * max_pages + pg];
-    const bf16_t* src = pages + (int64_t)(page < 0 ? 0 : page) * PAGE_TOKENS * width;
-    __syncthreads();                                                 // the page before has been read
-    for (int e = tid; e < 64 * chunks; e += 256) {
-      const int pos = e / chunks, k = (e % chunks) * 8;
-      *(vu4*)(page_s + pos * ws + k) = *(const vu4*)(src + (int64_t)pos * width + k);
-    }
-    __syncthreads();
-    vf4 s = {0.f, 0.f, 0.f, 0.f};
-    for (int k = 8 * g; k < width; k += 32)
-      s = MFMA16(*(const bf16x8*)(page_s + (16 * wave + c) * ws + k), *(const bf16x8*)(q_s + c * ws + k), s);
-    float top = -INFINITY;
+  for (int half = begin; half < end; ++half) {
+    __syncthreads();                                                 // the half page before has been read
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int pos = pg * PAGE_TOKENS + 16 * wave + 4 * g + r;
-      s[r] = (live && pos <= my_pos && page >= 0) ? s[r] * scale : -INFINITY;
-      top = fmaxf(top, s[r]);
+    for (int u = 0; u < NL; ++u) {
+      const int e = tid + 256 * u;
+      if (e < pieces) *(vu4*)(page_s + (e / chunks) * ws + (e % chunks) * 8) = next[u];
+    }
+    const bool seen = page_ok != 0;
+    __syncthreads();
+    if (half + 1 < end) fetch(half + 1);
+    vf4 part = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int k = k_from; k < k_to; ++k) part = MFMA16(*(const bf16x8*)(k_row + 32 * k), *(const bf16x8*)(q_row + 32 * k), part);
+    s_part[wave * WAVE + lane] = part;
+    __syncthreads();
+    // positions 8g .. 8g + 7 of the half page: of 16-position tile g / 2, held by its lane groups 2 (g % 2) and the next
+    float s[8], top = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int at = (g / 2) * WAVE + (2 * (g % 2) + i) * 16 + c;
+      const vf4 lo = s_part[at], hi = s_part[2 * WAVE + at];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int pos = half * LATENT_KEYS + 8 * g + 4 * i + r;
+        s[4 * i + r] = (live && seen && pos <= my_pos) ? (lo[r] + hi[r]) * scale : -INFINITY;
+        top = fmaxf(top, s[4 * i + r]);
+      }
     }
     top = fmaxf(top, __shfl_xor(top, 16, WAVE));
     top = fmaxf(top, __shfl_xor(top, 32, WAVE));
-    if (g == 0) red[wave * 16 + c] = top;
-    __syncthreads();
-    float m_new = m;
-#pragma unroll
-    for (int w = 0; w < 4; ++w) m_new = fmaxf(m_new, red[w * 16 + c]);
+    const float m_new = fmaxf(m, top);
     const float base = m_new == -INFINITY ? 0.f : m_new;             // a column that has seen no key yet keeps weight 0
     const float alpha = expf(m - base);
+    m = m_new;
     float sum = 0.f;
-    uint32_t packed[2];
+    u16x8 pb;
 #pragma unroll
-    for (int r = 0; r < 4; r += 2) {
-      const bf16_t p0 = float_to_bf16(expf(s[r] - base)), p1 = float_to_bf16(expf(s[r + 1] - base));
-      sum += bf16_to_float(p0) + bf16_to_float(p1);
-      packed[r / 2] = (uint32_t)p0.bits | ((uint32_t)p1.bits << 16);
+    for (int e = 0; e < 8; ++e) {
+      const bf16_t p = float_to_bf16(expf(s[e] - base));
+      sum += bf16_to_float(p);
+      pb[e] = p.bits;
     }
     l = l * alpha + sum;
-    m = m_new;
-    *(uint64_t*)(p_s + c * 72 + 16 * wave + 4 * g) = (uint64_t)packed[0] | ((uint64_t)packed[1] << 32);
-    __syncthreads();
-    bf16x8 pb[2];
-    pb[0] = *(const bf16x8*)(p_s + c * 72 + 8 * g);
-    pb[1] = *(const bf16x8*)(p_s + c * 72 + 32 + 8 * g);
 #pragma unroll
     for (int t = 0; t < NT; ++t) {
       const int f = 16 * (wave + 4 * t) + c;                         // the lane's feature as a row of the first operand
       if (16 * (wave + 4 * t) < rank) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) O[t][r] *= alpha;
+        u16x8 a;
 #pragma unroll
-        for (int kb = 0; kb < 2; ++kb) {
-          u16x8 a;
-#pragma unroll
-          for (int e = 0; e < 8; ++e) a[e] = page_s[(32 * kb + 8 * g + e) * ws + f].bits;
-          O[t] = MFMA16(__builtin_bit_cast(bf16x8, a), pb[kb], O[t]);
-        }
+        for (int e = 0; e < 8; ++e) a[e] = page_s[(8 * g + e) * ws + f].bits;
+        O[t] = MFMA16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, pb), O[t]);
       }
     }
   }
   l += __shfl_xor(l, 16, WAVE);
   l += __shfl_xor(l, 32, WAVE);
-  __syncthreads();
-  if (g == 0) red[wave * 16 + c] = l;
-  __syncthreads();
   if (!live) return;
-  l = red[c] + red[16 + c] + red[32 + c] + red[48 + c];
   const int64_t at = (((row_base + my_row) * H + my_head) * splits + blockIdx.z);
   if (wave == 0 && g == 0) { part_ml[2 * at] = m; part_ml[2 * at + 1] = l; }
 #pragma unroll
   for (int t = 0; t < NT; ++t) {
     const int f = 16 * (wave + 4 * t) + 4 * g;
+    if (rank % 4 == 0) {
+      if (f < rank) *(vf4*)(part_o + at * rank + f) = O[t];
+    } else {
 #pragma unroll
-    for (int r = 0; r < 4; ++r)
-      if (f + r < rank) part_o[at * rank + f + r] = O[t][r];
+      for (int r = 0; r < 4; ++r)
+        if (f + r < rank) part_o[at * rank + f + r] = O[t][r];
+    }
   }
 }
 
-// The runs of a (row, head) joined in order; rows of sequences that sit out give zeros.
+// The runs of a (row, head) joined in order; rows of sequences that sit out give zeros. Thread tid holds four features
+// (V = 4) or one; groups of threads take every `groups`-th run and are added up in order through LDS.
+#define LATENT_MAX_SPLITS 64
+
+template <int V>
 __global__ __launch_bounds__(256) void latent_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                                                              const int* __restrict__ row_slot, bf16_t* __restrict__ out,
                                                              int H, int rank, int splits) {
+  __shared__ float weight[LATENT_MAX_SPLITS], sums[256 * V];
   const int64_t at = (int64_t)blockIdx.x * H + blockIdx.y;
+  const int tid = threadIdx.x, per = rank / V;                       // threads that hold a run's features
   if (row_slot[blockIdx.x] < 0) {
-    for (int f = threadIdx.x; f < rank; f += 256) out[at * rank + f] = float_to_bf16(0.f);
+    for (int f = tid; f < rank; f += 256) out[at * rank + f] = float_to_bf16(0.f);
     return;
   }
-  float m = -INFINITY, l = 0.f;
-  for (int s = 0; s < splits; ++s) m = fmaxf(m, part_ml[2 * (at * splits + s)]);
-  for (int s = 0; s < splits; ++s) l += part_ml[2 * (at * splits + s) + 1] * expf(part_ml[2 * (at * splits + s)] - m);
-  const float inv = 1.f / l;
-  for (int f = threadIdx.x; f < rank; f += 256) {
-    float o = 0.f;
-    for (int s = 0; s < splits; ++s) o += part_o[(at * splits + s) * rank + f] * expf(part_ml[2 * (at * splits + s)] - m);
-    out[at * rank + f] = float_to_bf16(o * inv);
+  if (tid < WAVE) {
+    float m = -INFINITY, l = 0.f;
+    if (tid < splits) { m = part_ml[2 * (at * splits + tid)]; l = part_ml[2 * (at * splits + tid) + 1]; }
+    const float top = wave_max(m), w = expf(m - top);                // some run holds a key: top is finite
+    const float total = wave_sum(l * w);
+    weight[tid] = w / total;
+  }
+  __syncthreads();
+  const int groups = per < 256 ? 256 / per : 1;
+  for (int p0 = 0; p0 < per; p0 += 256) {
+    const int group = groups > 1 ? tid / per : 0, p = groups > 1 ? tid % per : p0 + tid;
+    float o[V];
+#pragma unroll
+    for (int j = 0; j < V; ++j) o[j] = 0.f;
+    if (group < groups && p < per) {
+      const float* src = part_o + at * splits * rank + (int64_t)p * V;
+      for (int s0 = group; s0 < splits; s0 += 8 * groups) {
+        float x[8][V];
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+          const int s = s0 + u * groups;
+          if constexpr (V == 4) {
+            const vf4 t = s < splits ? *(const vf4*)(src + (int64_t)s * rank) : vf4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int j = 0; j < 4; ++j) x[u][j] = t[j];
+          } else {
+            x[u][0] = s < splits ? src[(int64_t)s * rank] : 0.f;
+          }
+        }
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+          const float w = s0 + u * groups < splits ? weight[s0 + u * groups] : 0.f;
+#pragma unroll
+          for (int j = 0; j < V; ++j) o[j] += w * x[u][j];
+        }
+      }
+    }
+    if (groups == 1) {
+      if (p < per)
+#pragma unroll
+        for (int j = 0; j < V; ++j) out[at * rank + p * V + j] = float_to_bf16(o[j]);
+      continue;
+    }
+    if (group < groups)
+#pragma unroll
+      for (int j = 0; j < V; ++j) sums[(group * per + p) * V + j] = o[j];
+    __syncthreads();
+    for (int f = tid; f < rank; f += 256) {
+      float sum = 0.f;
+      for (int q = 0; q < groups; ++q) sum += sums[q * rank + f];
+      out[at * rank + f] = float_to_bf16(sum);
+    }
   }
 }
 
@@ -346,30 +419,38 @@ DRYFT_API int dryft_latent_split(const void* q, const void* pages, const int* pa
                                  int width, int rank, float scale, float* part_o, float* part_ml, int splits, void* out,
                                  hipStream_t stream) {
   if (n_rows <= 0) return 0;
-  if (H <= 0 || width % 32 || width > MLA_MAX_WIDTH || rank <= 0 || rank > width || splits <= 0) return -1;
-  const size_t lds = (size_t)80 * (width + 8) * 2 + 16 * 72 * 2 + 4 * 16 * 4;
+  if (H <= 0 || width % 32 || width > MLA_MAX_WIDTH || rank <= 0 || rank > width || splits <= 0 ||
+      splits > LATENT_MAX_SPLITS)
+    return -1;
+  const size_t lds = (size_t)(LATENT_KEYS + 16) * (width + 8) * sizeof(bf16_t) + 256 * sizeof(vf4);
   if (max_tiles > 0) {
     const dim3 grid(max_tiles, (H + 15) / 16, splits);
-#define LS(NN)                                                                                                       \
+#define LS(NN, LL)                                                                                                   \
   {                                                                                                                  \
-    if (lds > 64 * 1024 && hipFuncSetAttribute((const void*)latent_split_kernel<NN>,                                 \
+    if (lds > 64 * 1024 && hipFuncSetAttribute((const void*)latent_split_kernel<NN, LL>,                             \
                                                hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)  \
       return -2;                                                                                                     \
-    hipLaunchKernelGGL(latent_split_kernel<NN>, grid, dim3(256), lds, stream, (const bf16_t*)q, (const bf16_t*)pages,  \
-                       page_table, max_pages, seq_slot, cu_rows, q_len, seq_start, tile_cu, n_seqs, H, width, rank,    \
-                       scale, part_o, part_ml, splits);                                                              \
+    hipLaunchKernelGGL((latent_split_kernel<NN, LL>), grid, dim3(256), lds, stream, (const bf16_t*)q,                \
+                       (const bf16_t*)pages, page_table, max_pages, seq_slot, cu_rows, q_len, seq_start, tile_cu,    \
+                       n_seqs, H, width, rank, scale, part_o, part_ml, splits);                                      \
   }
-    if (rank <= 64) LS(1)
-    else if (rank <= 128) LS(2)
-    else if (rank <= 256) LS(4)
-    else if (rank <= 512) LS(8)
-    else LS(15)
+#define LSW(NN) if (width <= 256) LS(NN, 4) else if (width <= 576) LS(NN, 9) else LS(NN, 15)
+    if (rank <= 64) { LSW(1) }
+    else if (rank <= 128) { LSW(2) }
+    else if (rank <= 256) { LSW(4) }
+    else if (rank <= 512) { LSW(8) }
+    else { LS(15, 15) }
+#undef LSW
 #undef LS
     const int rc = DRYFT_LAUNCH_CHECK();
     if (rc) return rc;
   }
-  hipLaunchKernelGGL(latent_combine_kernel, dim3(n_rows, H), dim3(256), 0, stream, part_o, part_ml, row_slot, (bf16_t*)out,
-                     H, rank, splits);
+  if (rank % 4 == 0)
+    hipLaunchKernelGGL(latent_combine_kernel<4>, dim3(n_rows, H), dim3(256), 0, stream, part_o, part_ml, row_slot,
+                       (bf16_t*)out, H, rank, splits);
+  else
+    hipLaunchKernelGGL(latent_combine_kernel<1>, dim3(n_rows, H), dim3(256), 0, stream, part_o, part_ml, row_slot,
+                       (bf16_t*)out, H, rank, splits);
   return DRYFT_LAUNCH_CHECK();
 }
 

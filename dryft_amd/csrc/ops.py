@@ -2238,6 +2238,8 @@ def linear_chunks(proj, q_col: int, k_col: int, v_col: int, q_scale: float, k_sc
 
 
 # ------------------------------------------------------------------------------------------ attention to cached latents
+LATENT_MAX_SPLITS = 64      # runs that a sequence's keys are cut into at most
+LATENT_KEYS = 32            # keys the kernel takes at a time
 LATENT_MAX_WIDTH = 960      # features of a cached row (latent, rotated key part, padding)
 
 
@@ -2374,6 +2376,8 @@ def latent_attend(q, pages, page_table, seq_slot, cu_rows, q_len, seq_start, til
         _gpu(t, name, torch.int32)
         if t.numel() < need:
             raise KernelError(f"{name}: needs {need} entries")
+    if not 1 <= splits <= LATENT_MAX_SPLITS:
+        raise KernelError(f"latent_attend: 1..{LATENT_MAX_SPLITS} runs of pages, got {splits}")
     part_o = torch.empty((rows, heads, splits, rank), dtype=torch.float32, device=q.device)
     part_ml = torch.empty((rows, heads, splits, 2), dtype=torch.float32, device=q.device)
     _check(_fn("mla", "dryft_latent_split")(

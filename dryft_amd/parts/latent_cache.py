@@ -35,8 +35,7 @@ from .linear import linear
 from .rope import PairRotaryPositions
 
 _EXPANDED_FROM = 512           # prompts' steps of more rows than this form keys and values (captured steps have fewer)
-_WORKGROUPS = 512              # of the kernel that attends to latents: how many a decoding step is cut into at most
-_MAX_SPLITS = 32
+_WORKGROUPS = 512              # of the kernel that attends to latents: about how many a step is cut into at most
 
 
 def _padded(w: torch.Tensor, rows_to: int, cols_to: int) -> torch.Tensor:
@@ -146,9 +145,11 @@ class CachedLatentAttention(Mixer):
         return linear(out.view(rows, H * self.value_dim), self.w_o, allow_partials=True)
 
     def _splits(self, tiles: int, max_kv_len: int) -> int:
-        """Into how many runs a sequence's pages are cut: as many as fill the chip, at most one a page."""
-        blocks = max(1, tiles) * -(-self.n_heads // 16)
-        return max(1, min(_WORKGROUPS // blocks, _MAX_SPLITS, pages_for(max_kv_len)))
+        """Into how many runs a sequence's keys are cut: as many as fill the chip, at most one per run of keys that the
+        kernel takes at a time, and no more than the runs of equal length that this leaves need."""
+        blocks, pieces = max(1, tiles) * -(-self.n_heads // 16), -(-max_kv_len // ops.LATENT_KEYS)
+        most = max(1, min(_WORKGROUPS // blocks, ops.LATENT_MAX_SPLITS, pieces))
+        return -(-pieces // -(-pieces // most))
 
     def _with_keys(self, q_raw: torch.Tensor, ctx: StepContext, tables):
         rows, H, dev = q_raw.shape[0], self.n_heads, q_raw.device
