@@ -103,7 +103,10 @@ def tensors_for(cfg: dict, seed: int) -> dict[str, torch.Tensor]:
 
     def linear(p, m):
         H, D, Dv = m["heads"], m["dim"], m["vdim"]
-        mat(p + "q", H * D, W, 1.4); mat(p + "k", H * D, W, 1.4); mat(p + "v", H * Dv, W, 1.4)
+        # a key leans on the query of its own token: q . k of a token stays away from zero, where the read-out, which is
+        # divided by its own size, would turn on the last bit of either
+        mat(p + "q", H * D, W, 1.4); mat(p + "k", H * D, W, 0.8); mat(p + "v", H * Dv, W, 1.4)
+        out[p + "k"] += out[p + "q"]
         mat(p + "g", H * Dv, W, 2.0); mat(p + "o", W, H * Dv)
 
     out["embed"] = torch.randn(V, W, generator=g)

@@ -1,0 +1,823 @@
+"""Fubinex on the GPU against the plain implementation (float64), in float32 and bfloat16: each new kernel and mechanism
+alone, then whole models of three configurations through the step function (whole prompts, portions down to two
+tokens, one token at a time, unequal batches, slots used again, long decoding), configurations drawn at random, greedy
+generation through the entry point with captured steps, and the trace program. In bfloat16 the layers that attend to
+latents have two ways through a prompt (on the latents, and with keys and values formed for the step); the tests that
+run prompts run them both ways (``ways``)."""
+
+import json
+import os
+import subprocess
+import sys
+
+import numpy as np
+import pytest
+import torch
+
+from fubinex_cases import (CASES, YARN, chunks, config, double, gated, latent, parallel, random_config, retention, tensors_for,
+                           write_dir)
+from helpers import collect_positions, trace_batches
+from plain import fubinex_plain as P
+from test_piralix_gpu import CUTS, MIXER_TOL, TOL, feed, rel_err, run_mixer
+
+pytestmark = pytest.mark.gpu
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+DEV = "cuda:0"
+DTYPES = ["float32", "bfloat16"]
+TORCH = {"float32": torch.float32, "bfloat16": torch.bfloat16}
+EPS = 1e-5
+# rows of logits in bfloat16: the worst of a thousand rows lies at 0.03 to 0.06 of the logits' size (as it does for the
+# plain implementation with every product rounded to 8 bits); a lost state, a key or a decay that is off by one moves rows
+# by 0.1 to 1 (the tests that build such cases say so)
+TOL = {"float32": TOL["float32"], "bfloat16": 0.1}
+MORE_CUTS = CUTS + ([1, 2, 3, 4, 5, 6, 8],)
+
+
+def i32(x):
+    return torch.tensor(x, dtype=torch.int32, device=DEV)
+
+
+@pytest.fixture(params=["latents", "keys"])
+def ways(request, monkeypatch):
+    """Prompts on the latents, and with keys and values formed from the second row on."""
+    from dryft_amd.parts import latent_cache
+    if request.param == "keys":
+        monkeypatch.setattr(latent_cache, "_EXPANDED_FROM", 1)
+    return request.param
+
+
+# ------------------------------------------------------------------------------------------ kernels alone
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("width,groups", [(60, 3), (75, 5), (256, 2), (256, 256), (1000, 8), (2048, 4), (320, 1), (36, 9)])
+def test_stream_norm_in_parts(dtype, width, groups):
+    from dryft_amd.csrc import ops
+    T = TORCH[dtype]
+    g = torch.Generator().manual_seed(width)
+    rows = 7
+    x = 3 * torch.randn(rows, width, generator=g) * (0.2 + torch.arange(width) / width)     # parts of different sizes
+    d, w = torch.randn(2, rows, width, generator=g), torch.randn(width, generator=g)
+    x_out, y = torch.empty(rows, width, device=DEV), torch.empty(rows, width, dtype=T, device=DEV)
+    ops.stream_norm(x.to(DEV), (d.to(DEV), 2), None, None, None, w.to(DEV), EPS, x_out, y, T, groups=groups)
+    want = x.double() + d.double().sum(0)
+    assert torch.allclose(x_out.cpu().double(), want, atol=2e-5)
+    ref = P.group_norm(want, w.double(), groups, EPS)
+    assert rel_err(y, ref) <= (1e-6 if dtype == "float32" else 6e-3)
+    if groups > 1:
+        assert rel_err(P.group_norm(want, w.double(), 1, EPS), ref) > 0.05
+    ops.stream_norm(x.to(DEV), None, None, None, None, w.to(DEV), EPS, None, y, T, groups=groups)
+    assert rel_err(y, P.group_norm(x.double(), w.double(), groups, EPS)) <= (1e-6 if dtype == "float32" else 6e-3)
+
+
+def test_stream_norm_refuses_parts_that_do_not_fit():
+    from dryft_amd.csrc import ops
+    x, y, w = torch.zeros(2, 10, device=DEV), torch.zeros(2, 10, device=DEV), torch.ones(10, device=DEV)
+    for groups in (0, 3, 20):
+        with pytest.raises(ops.KernelError):
+            ops.stream_norm(x, None, None, None, None, w, EPS, None, y, torch.float32, groups=groups)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("width", [9, 64, 250, 4096, 16384, 16392])
+def test_poly_norm(dtype, width):
+    from dryft_amd.csrc import ops
+    T = TORCH[dtype]
+    g = torch.Generator().manual_seed(width)
+    rows = 5
+    wide = (2 * torch.randn(rows, width + 8, generator=g)).to(T)
+    parts = torch.randn(3, rows, width, generator=g)
+    act = torch.tensor([0.7, -0.4, 0.9, 0.2])
+    out = torch.empty(rows, width, dtype=T, device=DEV)
+    for z, given in ((wide[:, 8:].double(), wide.to(DEV)[:, 8:]), (parts.double().sum(0), (parts.to(DEV), 3))):
+        ops.poly_norm(given, act.to(DEV), EPS, out)
+        want = P.poly_norm(z, act.double(), EPS)
+        assert rel_err(out, want) <= (2e-6 if dtype == "float32" else 6e-3)
+        for i in range(4):                                            # each of the four numbers is at work
+            other = act.double().clone()
+            other[i] = 0
+            assert float((P.poly_norm(z, other, EPS) - want).abs().max()) > 0.1
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("width", [33, 128])
+def test_scaled_pair(dtype, width):
+    from dryft_amd.csrc import ops
+    T = TORCH[dtype]
+    g = torch.Generator().manual_seed(width)
+    a, b = torch.randn(6, width, generator=g).to(T), torch.randn(3, 6, width, generator=g)
+    bias = torch.randn(width, generator=g)
+    out = torch.empty(6, width, device=DEV)
+    ops.scaled_pair(a.to(DEV), bias.to(DEV), 0.7, (b.to(DEV), 3), None, -1.3, out, T)
+    assert torch.allclose(out.cpu().double(), 0.7 * (a.double() + bias.double()) - 1.3 * b.double().sum(0), atol=1e-5)
+    ops.scaled_pair((b.to(DEV), 3), None, -1.3, a.to(DEV), bias.to(DEV), 0.7, out, T)
+    assert torch.allclose(out.cpu().double(), 0.7 * (a.double() + bias.double()) - 1.3 * b.double().sum(0), atol=1e-5)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("head_dim,v_dim,rot,page", [(32, 32, 16, 0), (20, 12, 0, 0), (96, 96, 24, 0), (40, 72, 40, 80), (128, 128, 64, 0)])
+def test_norm_after_the_turn(dtype, head_dim, v_dim, rot, page):
+    from dryft_amd.csrc import ops
+    T = TORCH[dtype]
+    g = torch.Generator().manual_seed(head_dim)
+    rows, H, G = 70, 4, 2
+    src = (2 * torch.randn(rows, H * head_dim + G * (head_dim + v_dim), generator=g)).to(T)
+    pos = torch.arange(5, 5 + rows)
+    r = {"dims": rot, "base": 100.0} if rot else None
+    cos = sin = None
+    if rot:
+        f, _ = P.frequencies(r)
+        a = torch.arange(80).double()[:, None] * f
+        cos, sin = a.cos().float().to(DEV), a.sin().float().to(DEV)
+    kw, vw = page or head_dim, page or v_dim
+    k, v = torch.zeros(2, G, 64, kw, dtype=T, device=DEV), torch.zeros(2, G, vw, 64, dtype=T, device=DEV)
+    q = torch.zeros(rows, H, kw, dtype=T, device=DEV)
+    table = i32([[1, 0]])
+    ops.norm_rope_half_kv(src.to(DEV), 0, H * head_dim, (H + G) * head_dim, None, None, EPS, cos, sin, rot, i32([0] * rows),
+                          i32(pos.tolist()), q, k, v, table, True, H, G, head_dim, v_dim, page_dim=page, unit_after=True)
+    x = src.double()
+    tol = 2e-6 if dtype == "float32" else 6e-3
+    want = P.rms(P.rotate_halves(x[:, :H * head_dim].view(rows, H, head_dim), pos, r), EPS)
+    assert rel_err(q[..., :head_dim], want) <= tol and (page == 0 or float(q[..., head_dim:].abs().max()) == 0)
+    want = P.rms(P.rotate_halves(x[:, H * head_dim:(H + G) * head_dim].view(rows, G, head_dim), pos, r), EPS)
+    cache = torch.cat([k[1], k[0]], 1).transpose(0, 1)[5:5 + rows, :, :head_dim]
+    assert rel_err(cache, want) <= tol
+    with pytest.raises(ops.KernelError):
+        ops.norm_rope_half_kv(src.to(DEV), 0, H * head_dim, (H + G) * head_dim, torch.ones(head_dim, device=DEV), None, EPS, cos, sin,
+                              rot, i32([0] * rows), i32(pos.tolist()), q, k, v, table, True, H, G, head_dim, v_dim, page_dim=page,
+                              unit_after=True)
+
+
+def test_log_decay():
+    from dryft_amd.csrc import ops
+    g = torch.Generator().manual_seed(3)
+    for rows in (3, 100):
+        low, up, bias = 3 * torch.randn(rows, 5, generator=g), 4 * torch.randn(40, 5, generator=g), torch.randn(40, generator=g)
+        out = torch.empty(rows, 40, device=DEV)
+        ops.log_decay(low.to(DEV), up.to(DEV), bias.to(DEV), out, 0.25)
+        z = low.double() @ up.double().T + bias.double()
+        assert float(z.min()) < -20 and float(z.max()) > 20
+        want = 0.25 * torch.nn.functional.logsigmoid(z)
+        assert torch.allclose(out.cpu().double(), want, rtol=2e-5, atol=1e-7)
+
+
+def walk_case(H, D, Dv, lengths, decay, seed, rot=None):
+    """Inputs of a recurrence: ``decay`` 'channel' (spread over the whole range), 'strong' (channels that forget within a
+    token), or a list of one number per head."""
+    g = torch.Generator().manual_seed(seed)
+    T = sum(lengths)
+    proj = torch.randn(T, H * (2 * D + 2 * Dv), generator=g).to(torch.bfloat16).float()
+    logs = heads = None
+    if isinstance(decay, str):
+        logs = -torch.exp(-4 + 4 * torch.rand(T, H * D, generator=g))                      # e^-1 .. e^-0.02
+        if decay == "strong":
+            logs = torch.where(torch.rand(1, H * D, generator=g) < 0.3, -40 * torch.rand(T, H * D, generator=g), logs)
+        dec = logs.double().exp().view(T, H, D)
+    else:
+        heads = torch.tensor(decay)
+        dec = heads.double()[None, :, None].expand(T, H, D)
+    return proj, logs, heads, dec
+
+
+def plain_walk(proj, dec, H, D, Dv, lengths, starts, states, rot, q_scale, k_scale):
+    outs, ends, at = [], [], 0
+    for n, start, S in zip(lengths, starts, states):
+        x = proj[at:at + n].double()
+        pos = torch.arange(start, start + n)
+        q = P.rotate_halves(x[:, :H * D].view(n, H, D), pos, rot) * q_scale
+        k = P.rotate_halves(x[:, H * D:2 * H * D].view(n, H, D), pos, rot) * k_scale
+        o, S = P.linear_walk(q, k, x[:, 2 * H * D:2 * H * D + H * Dv].view(n, H, Dv), dec[at:at + n], S)
+        outs.append(o)
+        ends.append(S)
+        at += n
+    return outs, ends
+
+
+WALKS = [(1, 16, 16, "channel", None), (2, 24, 40, "channel", None), (3, 64, 65, "strong", None), (2, 128, 128, "channel", None),
+         (1, 256, 256, "strong", None), (2, 32, 48, [0.9, 0.02], 16), (2, 64, 64, [1.0, 0.999], 64), (1, 130, 20, [0.7], 130),
+         (2, 8, 8, [0.5, 0.99], 2), (1, 256, 30, [0.97], 128), (2, 20, 10, [1e-6, 0.3], None)]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,D,Dv,decay,rot_dims", WALKS)
+def test_linear_attention_kernels(H, D, Dv, decay, rot_dims, dtype):
+    """The chunk kernel whole and in segments, and the token kernel, from states that are not zero, beside a sequence
+    that sits out; in bfloat16 the inputs are rounded and everything after them is float arithmetic as in float32."""
+    from dryft_amd.csrc import ops
+    T = TORCH[dtype]
+    lengths, starts = [33, 1, 5, 150, 16], [3, 60, 0, 17, 64]
+    proj, logs, heads, dec = walk_case(H, D, Dv, lengths, decay, seed=D + Dv)
+    rot = {"dims": rot_dims, "base": 50.0} if rot_dims else None
+    tables = None
+    if rot:
+        a = torch.arange(256).double()[:, None] * P.frequencies(rot)[0]
+        tables = (a.cos().float().to(DEV), a.sin().float().to(DEV), rot_dims)
+    g = torch.Generator().manual_seed(9)
+    n_slots, slots = 7, [4, 1, -1, 0, 6]
+    state0 = torch.randn(n_slots, H, D, Dv, generator=g)
+    pos = [s + i for n, s in zip(lengths, starts) for i in range(n)]
+    cu = np.concatenate([[0], np.cumsum(lengths)]).tolist()
+    q_scale, k_scale = D ** -0.5, 0.8
+    want, ends = plain_walk(proj, dec, H, D, Dv, lengths, starts, [state0[s].double() for s in slots], rot, q_scale, k_scale)
+    dev = proj.to(T).to(DEV)
+    cols = (0, H * D, 2 * H * D)
+    common = (q_scale, k_scale, tables, i32(pos))
+    log_dev = logs.to(DEV) if logs is not None else None
+    facts = (i32(slots), i32(cu), i32(lengths), len(lengths))
+    per = [[-(-n // 32) if s >= 0 else 0 for n, s in zip(lengths, slots)], [-(-n // 64) if s >= 0 else 0 for n, s in zip(lengths, slots)]]
+    ways = [None] + [(rows, i32(np.concatenate([[0], np.cumsum(p)]).tolist()), sum(p) + 2) for rows, p in zip((32, 64), per)]
+    for segments in ways:
+        state = state0.to(DEV)
+        o = torch.zeros(sum(lengths), H * Dv, device=DEV)
+        ops.linear_chunks(dev, *cols, *common, log_dev, heads.double().log().float().to(DEV) if heads is not None else None, *facts,
+                          state, o, H, D, Dv, True, segments=segments)
+        for i, (slot, ref, end) in enumerate(zip(slots, want, ends)):
+            got = o[cu[i]:cu[i + 1]].view(-1, H, Dv).cpu()
+            if slot < 0:
+                assert float(got.abs().max()) == 0
+                continue
+            assert float((got.double() - ref).abs().max() / ref.pow(2).mean().sqrt()) <= 2e-5, (i, segments and segments[0])
+            assert float((state[slot].cpu().double() - end).abs().max() / end.pow(2).mean().sqrt()) <= 2e-5
+        assert torch.equal(state[2].cpu(), state0[2]) and torch.equal(state[5].cpu(), state0[5])
+    before = state.clone()
+    ops.linear_chunks(dev, *cols, *common, log_dev, heads.double().log().float().to(DEV) if heads is not None else None, *facts, state,
+                      o, H, D, Dv, False)
+    assert torch.equal(state, before)                                       # a run that does not write leaves the state
+    # token by token: the same rows through the kernel of decoding steps, with norm, weight and gate
+    weight = 1 + 0.3 * torch.randn(Dv, generator=g)
+    for w in (weight, None):
+        state = state0.to(DEV)
+        out = torch.full((sum(lengths), H * Dv), 7.0, dtype=T, device=DEV)
+        ops.linear_token(dev, *cols, 2 * H * D + H * Dv, *common, log_dev, heads.to(DEV) if heads is not None else None, *facts, state,
+                         w.to(DEV) if w is not None else None, EPS, out, H, D, Dv, True)
+        for i, (slot, ref, end) in enumerate(zip(slots, want, ends)):
+            gate = proj[cu[i]:cu[i + 1], 2 * H * D + H * Dv:].double()
+            ref = P.rms(ref, EPS) * (w.double() if w is not None else 1.0)
+            ref = ref.reshape(len(gate), H * Dv) * P.silu(gate)
+            got = out[cu[i]:cu[i + 1]].cpu().double()
+            if slot < 0:
+                assert float(got.abs().max()) == 0
+                continue
+            assert rel_err(got, ref) <= (2e-4 if dtype == "float32" else 8e-3), i
+            assert float((state[slot].cpu().double() - end).abs().max() / end.pow(2).mean().sqrt()) <= 2e-5
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("heads,k,n,rot_dim,pairs", [(3, 12, 14, 6, True), (20, 8, 40, 16, True), (2, 128, 512, 64, False), (5, 70, 33, 0, False)])
+def test_head_product(dtype, heads, k, n, rot_dim, pairs):
+    from dryft_amd.csrc import ops
+    from dryft_amd.parts.latent_cache import _padded
+    T = TORCH[dtype]
+    g = torch.Generator().manual_seed(k)
+    m = (torch.randn(heads, n, k, generator=g) / k ** 0.5).to(T)
+    rot = {"dims": rot_dim // 4 * 2, "base": 30.0} if rot_dim else None
+    tables = None
+    if rot:
+        a = torch.arange(64).double()[:, None] * P.frequencies(rot)[0]
+        tables = (a.cos().float().to(DEV), a.sin().float().to(DEV), rot["dims"], pairs)
+    width = -(-(n + rot_dim) // 32) * 32
+    for rows in (1, 16, 37):
+        x = torch.randn(rows, heads * (k + rot_dim), generator=g).to(T)
+        pos = torch.arange(20, 20 + rows)
+        out = torch.full((rows, heads, width if rot_dim else n), 5.0, dtype=T, device=DEV)
+        ops.head_product(x.to(DEV), 0, k + rot_dim, _padded(m, 16, 32).to(DEV), k, n, out, rot_dim, tables, i32(pos.tolist()))
+        xs = x.double().view(rows, heads, k + rot_dim)
+        want = torch.einsum("rhk,hnk->rhn", xs[..., :k], m.double())
+        assert rel_err(out[..., :n], want) <= (2e-6 if dtype == "float32" else 6e-3)
+        if rot_dim:
+            tail = (P.rotate_pairs if pairs else P.rotate_halves)(xs[..., k:], pos, rot)
+            assert rel_err(out[..., n:n + rot_dim], tail) <= (2e-6 if dtype == "float32" else 6e-3)
+            assert float(out[..., n + rot_dim:].abs().max() if width > n + rot_dim else 0) == 0
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("heads,rank,rot_dim", [(1, 12, 4), (3, 40, 8), (16, 128, 16), (20, 70, 24), (8, 512, 64), (2, 600, 32), (4, 928, 32)])
+def test_attention_to_latents(dtype, heads, rank, rot_dim):
+    """Rows deep inside, at and just behind borders of pages and of runs of 32 keys; keys anywhere that take most of a
+    row's weight; pages poisoned where no sequence reaches; a sequence that sits out; every number of runs."""
+    from dryft_amd.csrc import ops
+    T = TORCH[dtype]
+    g = torch.Generator().manual_seed(rank)
+    width = -(-(rank + rot_dim) // 32) * 32
+    ends, q_lens = [1, 31, 32, 33, 64, 65, 200, 130], [1, 3, 1, 2, 1, 1, 4, 17]
+    n_pages = sum(-(-e // 64) for e in ends) + 2
+    order = torch.randperm(n_pages, generator=g).tolist()
+    pages = torch.full((n_pages, 1, 64, width), 50.0)
+    table = torch.full((len(ends) + 1, 5), -1, dtype=torch.int32)
+    rows_of = []
+    for s, e in enumerate(ends):
+        lat = torch.randn(e, width, generator=g)
+        lat[:, rank + rot_dim:] = 0
+        rows_of.append(lat.to(T))
+        for p in range(-(-e // 64)):
+            page = order.pop()
+            table[s, p] = page
+            pages[page, 0, :min(64, e - 64 * p)] = lat[64 * p:64 * p + 64]
+    pages = pages.to(T)
+    q = torch.randn(sum(q_lens), heads, width, generator=g).to(T)
+    q[..., rank + rot_dim:] = 0
+    scale = 6.0 / (rank + rot_dim) ** 0.5                                     # scores of several units: few keys a row
+    dead = 4
+    slots = [s if s != dead else -1 for s in range(len(ends))]
+    starts = [e - n for e, n in zip(ends, q_lens)]
+    cu = np.concatenate([[0], np.cumsum(q_lens)]).tolist()
+    row_slot = [slots[s] for s, n in enumerate(q_lens) for _ in range(n)]
+    row_pos = [starts[s] + i for s, n in enumerate(q_lens) for i in range(n)]
+    rt = ops.latent_tile_rows(heads)
+    tiles = [-(-n // rt) if sl >= 0 else 0 for n, sl in zip(q_lens, slots)]
+    want = torch.zeros(sum(q_lens), heads, rank, dtype=torch.float64)
+    for s, lat in enumerate(rows_of):
+        if s == dead:
+            continue
+        for i in range(q_lens[s]):
+            p = starts[s] + i
+            sc = (q[cu[s] + i].double() @ lat[:p + 1].double().T) * scale
+            want[cu[s] + i] = torch.softmax(sc, -1) @ lat[:p + 1, :rank].double()
+    for splits in (1, 2, 3, 7, 64):
+        out = torch.full((sum(q_lens), heads, rank), 9.0, dtype=T, device=DEV)
+        ops.latent_attend(q.to(DEV), pages.to(DEV), table.to(DEV), i32(slots), i32(cu), i32(q_lens), i32(starts),
+                          i32(np.concatenate([[0], np.cumsum(tiles)]).tolist()), len(ends), sum(tiles) + 1, i32(row_slot), i32(row_pos), out,
+                          rank, scale, splits)
+        assert float(out[cu[dead]:cu[dead + 1]].abs().max()) == 0
+        d = (out.cpu().double() - want).pow(2).mean(-1).sqrt() / want.pow(2).mean().sqrt()
+        assert float(d.max()) <= (2e-5 if dtype == "float32" else 1.5e-2), (splits, float(d.max()))
+
+
+# ------------------------------------------------------------------------------------------ mixers alone
+def mixer_case(layer, width, seed):
+    from dryft_amd.config.fubinex import FubinexConfig
+    from dryft_amd.models.fubinex import fubinex_plan
+    cfg = config(width, 16, [layer], eps=EPS)
+    return cfg, tensors_for(cfg, seed), fubinex_plan(FubinexConfig.from_dict(cfg))
+
+
+def load_mixer(plan, t, dtype, max_len=256):
+    from dryft_amd.cache import CacheStore
+    from dryft_amd.parts import build_part
+    T = TORCH[dtype]
+    spec = plan.layers[0].parts["mixer"]
+    part = build_part(spec)
+    part.compute_dtype = T
+    part.load({logical: t[spec.tensors[logical]].to(DEV).to(T) for logical in part.tensor_specs()})
+    cache = CacheStore({0: part.cache_need()}, max_tokens=64 * 16, n_slots=4, max_len=max_len, dtype=T, device=DEV)
+    positions = {}
+    for name, ps in plan.positions.items():
+        positions[name] = part_of = build_part(ps)
+        part_of.prepare(max_len, T, DEV)
+    return part, cache, positions
+
+
+def inputs(dtype, width, lengths=(201, 9, 70), seed=12):
+    g = torch.Generator().manual_seed(seed)
+    return [torch.randn(n, width, generator=g).to(TORCH[dtype]).float() for n in lengths]
+
+
+def plain_mixer(layer, h, w, past=None):
+    run = {"parallel": P.parallel, "retention": P.retention, "latent_attention": P.latent_attention}[layer["type"]]
+    return run(h, w, layer["mixer"], EPS, past)[0]
+
+
+ONLY_LEFT, ONLY_RIGHT = dict(left_scale=1.0, right_scale=0.0), dict(left_scale=0.0, right_scale=1.0)
+SMALL_R, SMALL_L = gated(1, 8, 8, 2), chunks(1, 1, 8, 8)
+MIXER_SHAPES = {
+    "chunks-cores": parallel(chunks(4, 2, 32, 32, chunk=24, rot=16), SMALL_R, **ONLY_LEFT),
+    "chunks-page": parallel(chunks(4, 4, 64, 64, chunk=64, rot=64), SMALL_R, **ONLY_LEFT),
+    "chunks-page-and-one": parallel(chunks(2, 1, 16, 48, chunk=65, rot=4), SMALL_R, **ONLY_LEFT),
+    "chunks-odd": parallel(chunks(3, 3, 20, 12), SMALL_R, **ONLY_LEFT),
+    "chunks-itself": parallel(chunks(2, 2, 16, 16, chunk=1), SMALL_R, **ONLY_LEFT),
+    "chunks-128": parallel(chunks(4, 2, 128, 128, chunk=128, rot=64, scale=6.0 / 128), SMALL_R, **ONLY_LEFT),
+    "gated-small": parallel(SMALL_L, gated(2, 16, 24, 5, tau=8.0), **ONLY_RIGHT),
+    "gated-odd": parallel(SMALL_L, gated(3, 10, 6, 3, tau=1.0), **ONLY_RIGHT),
+    "gated-128": parallel(SMALL_L, gated(2, 128, 128, 16), **ONLY_RIGHT),
+    "both": parallel(chunks(4, 2, 32, 32, chunk=24, rot=16), gated(2, 16, 24, 5, tau=8.0), 0.7, -1.2),
+    "retention-small": retention(2, 16, 16, [0.9, 0.998], rot=16),
+    "retention-odd": retention(3, 20, 10, [0.02, 0.5, 1.0]),
+    "retention-part-rotated": retention(2, 64, 32, [0.97, 0.999], rot=24),
+    "retention-wide": retention(1, 136, 200, [0.99], rot=136),
+    "latent-small": latent(4, 16, 8, 40, 24, 32, rot=8, base=100.0, scaling=YARN),
+    "latent-odd": latent(3, 12, 6, 20, 10, 14),
+    "latent-many-heads": latent(20, 8, 16, 8, 32, 40, rot=16, base=5e3),
+    "latent-part-rotated": latent(2, 32, 32, 64, 48, 24, rot=24, base=1e4),
+    "latent-192": latent(2, 128, 64, 128, 96, 128, rot=64, base=5e5, scale=0.04),
+}
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("shape", sorted(MIXER_SHAPES))
+def test_mixer_alone(dtype, shape, ways):
+    layer = MIXER_SHAPES[shape]
+    if ways == "keys" and not (shape.startswith("latent") and dtype == "bfloat16"):
+        return                                                    # one way only
+    cfg, t, plan = mixer_case(layer, 64, seed=len(shape))
+    part, cache, positions = load_mixer(plan, t, dtype)
+    seqs = inputs(dtype, 64)
+    w = double(P.sub(t, "l0.mix."))
+    want = [plain_mixer(layer, s.double(), w) for s in seqs]
+    for cuts in MORE_CUTS:
+        for got, ref in zip(run_mixer(part, cache, positions, dtype, seqs, cuts), want):
+            assert rel_err(got, ref) <= MIXER_TOL[dtype], (shape, cuts[:3])
+
+
+SHOW_CUTS = ([], list(range(120, 200)), [64, 128], [2, 63, 65, 127, 129], [19, 20, 21], [1, 2, 3])
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("chunk", [None, 20, 64, 65, 130])
+def test_chunks_rotation_and_norm_show(dtype, chunk):
+    """A score scale large enough that a row gives most of its weight to one or two keys, wherever they are: then a chunk
+    that is one token off, a key lost behind a page's border, another rotation or a norm left out moves some row by far
+    more than the tolerance (the plain implementation with each of those faults shows it)."""
+    tol = {"float32": MIXER_TOL["float32"], "bfloat16": 2 * MIXER_TOL["bfloat16"]}[dtype]
+    layer = parallel(chunks(2, 1, 32, 32, chunk=chunk, rot=24, base=100.0, scale=0.4), SMALL_R, **ONLY_LEFT)
+    m = layer["mixer"]["left"]
+    cfg, t, plan = mixer_case(layer, 32, seed=3)
+    part, cache, positions = load_mixer(plan, t, dtype)
+    h = inputs(dtype, 32, (200,), seed=4)[0]
+    w = double(P.sub(t, "l0.mix.left."))
+
+    def plain(m2, x=h):
+        return P.chunked_attention(x.double(), w, m2, EPS)[0]
+    want = plain(m)
+    if chunk:
+        for off in (-1, 1):
+            assert rel_err(plain({**m, "mask": {"size": chunk + off}}), want) > 0.2
+    else:
+        assert rel_err(plain({**m, "mask": {"size": 64}})[150:], want[150:]) > 0.2     # keys before the last page matter
+    for fault in ({**m, "rot": None}, {**m, "rot": {"dims": 24, "base": 1e4}}, {**m, "rot": {"dims": 32, "base": 100.0}}):
+        assert rel_err(plain(fault), want) > 0.1
+    saved = P.rms
+    try:
+        P.rms = lambda x, eps: x                                       # q and k as they are
+        assert rel_err(plain(m), want) > 0.1
+    finally:
+        P.rms = saved
+    for cuts in SHOW_CUTS:
+        got = run_mixer(part, cache, positions, dtype, [h], cuts)[0]
+        assert rel_err(got, want) <= tol, cuts[:3]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("decay", [0.95, 0.9998, 0.05])
+def test_retention_state_shows(dtype, decay):
+    """A state that is lost between portions, a decay that is taken once too often or a rotation left out shows."""
+    tol = {"float32": MIXER_TOL["float32"], "bfloat16": 2 * MIXER_TOL["bfloat16"]}[dtype]
+    layer = retention(2, 32, 24, [decay, decay], rot=16, base=100.0)
+    cfg, t, plan = mixer_case(layer, 32, seed=5)
+    part, cache, positions = load_mixer(plan, t, dtype)
+    h = inputs(dtype, 32, (200,), seed=6)[0]
+    w = double(P.sub(t, "l0.mix."))
+    want = plain_mixer(layer, h.double(), w)
+    lost = torch.cat([plain_mixer(layer, h[:100].double(), w),
+                      P.retention(h[100:].double(), w, layer["mixer"], EPS, {"S": torch.zeros(2, 32, 24, dtype=torch.float64), "n": 100})[0]])
+    none = {**layer, "mixer": {**layer["mixer"], "rot": None}}
+    if decay > 0.5:                                        # else little is left of the token before
+        assert rel_err(lost, want) > 0.1
+        assert rel_err(plain_mixer(none, h.double(), w), want) > 0.05
+    late = torch.cat([plain_mixer(layer, h[:100].double(), w),                     # positions that start again
+                      P.retention(h[100:].double(), w, layer["mixer"], EPS, {**P.retention(h[:100].double(), w, layer["mixer"], EPS)[1], "n": 0})[0]])
+    if decay > 0.5:
+        assert rel_err(late, want) > 0.1
+    for cuts in SHOW_CUTS:
+        got = run_mixer(part, cache, positions, dtype, [h], cuts)[0]
+        assert rel_err(got, want) <= tol, cuts[:3]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_gated_decay_shows(dtype):
+    layer = parallel(SMALL_L, gated(2, 16, 24, 5, tau=4.0), **ONLY_RIGHT)
+    m = layer["mixer"]["right"]
+    cfg, t, plan = mixer_case(layer, 32, seed=7)
+    part, cache, positions = load_mixer(plan, t, dtype)
+    h = inputs(dtype, 32, (200,), seed=8)[0]
+    w = double(P.sub(t, "l0.mix.right."))
+    want = P.gated_linear_attention(h.double(), w, m, EPS)[0]
+    faults = {"no bias": ({**w, "a2.b": 0 * w["a2.b"]}, m), "another tau": (w, {**m, "tau": 2.0}), "no norm weight": ({**w, "norm": torch.ones_like(w["norm"])}, m),
+              "no gate": ({**w, "g": 0 * w["g"] + 1}, m), "decay of the input left out": ({**w, "a1": 0 * w["a1"]}, m)}
+    for what, (w2, m2) in faults.items():
+        assert rel_err(P.gated_linear_attention(h.double(), w2, m2, EPS)[0], want) > 0.1, what
+    for cuts in SHOW_CUTS:
+        got = run_mixer(part, cache, positions, dtype, [h], cuts)[0]
+        assert rel_err(got, want) <= 2 * MIXER_TOL[dtype], cuts[:3]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_latent_keys_far_away_show(dtype, ways):
+    tol = {"float32": MIXER_TOL["float32"], "bfloat16": 2 * MIXER_TOL["bfloat16"]}[dtype]
+    layer = latent(2, 16, 16, 32, 24, 20, rot=16, base=100.0, scaling=YARN, scale=0.4)
+    m = layer["mixer"]
+    cfg, t, plan = mixer_case(layer, 32, seed=9)
+    part, cache, positions = load_mixer(plan, t, dtype)
+    h = inputs(dtype, 32, (200,), seed=10)[0]
+    w = double(P.sub(t, "l0.mix."))
+    want = plain_mixer(layer, h.double(), w)
+    cut = P.latent_attention(h[:64].double(), w, m, EPS)[1]
+    moved = {k: torch.cat([v[:40], v[41:]]) for k, v in cut.items()}            # one key of the first page is lost
+    assert rel_err(P.latent_attention(h[64:].double(), w, m, EPS, moved)[0], want[64:]) > 0.05
+    faults = {"no rotation": (w, {**m, "rot": None}), "no scaling": (w, {**m, "rot": {"dims": 16, "base": 100.0}}),
+              "another factor": (w, {**m, "rot": {**m["rot"], "scaling": {**YARN, "factor": 2.0}}}),
+              "no latent norm weight": ({**w, "dkv.norm": torch.ones_like(w["dkv.norm"])}, m),
+              "no query norm weight": ({**w, "dq.norm": torch.ones_like(w["dq.norm"])}, m)}
+    for what, (w2, m2) in faults.items():
+        assert rel_err(P.latent_attention(h.double(), w2, m2, EPS)[0], want) > 0.05, what
+    saved = P.rotate_pairs
+    try:
+        P.rotate_pairs = P.rotate_halves
+        assert rel_err(plain_mixer(layer, h.double(), w), want) > 0.1
+    finally:
+        P.rotate_pairs = saved
+    for cuts in SHOW_CUTS:
+        got = run_mixer(part, cache, positions, dtype, [h], cuts)[0]
+        assert rel_err(got, want) <= tol, cuts[:3]
+
+
+# ------------------------------------------------------------------------------------------ whole models
+class Model:
+    def __init__(self, tmp, name, cfg=None, seed=None):
+        self.name, self.cfg = name, cfg or CASES[name]
+        self.tensors = tensors_for(self.cfg, seed=seed if seed is not None else ord(name[0]))
+        self.dir = write_dir(os.path.join(tmp, name), self.cfg, self.tensors)
+        self.vocab = self.cfg["vocab"]
+        self._plain, self._engines = {}, {}
+
+    def tokens(self, n, seed=0):
+        return [int(x) for x in np.random.default_rng(1000 * seed + n).integers(0, self.vocab, size=n)]
+
+    def plain(self, tokens) -> torch.Tensor:
+        key = tuple(tokens)
+        if key not in self._plain:
+            self._plain[key] = P.forward(self.cfg, double(self.tensors), list(tokens))[0]
+        return self._plain[key]
+
+    def engine(self, dtype, **kw):
+        from dryft_amd import Engine
+        key = (dtype, tuple(sorted(kw.items())))
+        if key not in self._engines:
+            args = dict(max_batch=4, max_len=320, max_tokens=64 * 24, use_graph=False)
+            args.update(kw)
+            self._engines[key] = Engine(self.dir, dtype=dtype, **args)
+        return self._engines[key]
+
+
+@pytest.fixture(scope="module")
+def models(tmp_path_factory):
+    tmp = str(tmp_path_factory.mktemp("fubinex"))
+    return {name: Model(tmp, name) for name in CASES}
+
+
+LENGTHS = [1, 2, 5, 63, 64, 65, 130]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", sorted(CASES))
+def test_whole_prompts_portions_and_single_tokens(models, name, dtype, ways):
+    model = models[name]
+    engine = model.engine(dtype)
+    requests = {f"r{n}": model.tokens(n) for n in LENGTHS}
+    for what, cuts_of in (("whole", lambda n: []), ("last tokens one by one", lambda n: list(range(max(1, n - 24), n))),
+                          ("portions", lambda n: [2, 4, 7, 64, 66, 129]), ("first tokens one by one", lambda n: [1, 2, 3])):
+        got = feed(engine, requests, cuts_of)
+        for rid, toks in requests.items():
+            assert rel_err(got[rid], model.plain(toks)) <= TOL[dtype], (name, what, rid)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["A", "C"])
+def test_layer_by_layer(models, name, dtype, ways):
+    """The residual stream after every layer against the plain one (float32 in both precisions)."""
+    from dryft_amd import SeqStep
+    model = models[name]
+    engine = model.engine(dtype)
+    toks = model.tokens(37)
+    want = P.forward(model.cfg, double(model.tensors), toks)[1]
+    got = []
+    slot = engine.acquire(1)[0]
+    engine.step([SeqStep(slot, toks, [36])], tap=lambda i, x: got.append(x.cpu()))
+    engine.release([slot])
+    assert len(got) == len(want) == len(model.cfg["layers"])
+    for i, (g, w) in enumerate(zip(got, want)):
+        assert g.dtype == torch.float32
+        assert rel_err(g, w) <= (2e-5 if dtype == "float32" else 5e-2), (name, i)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_borrowed_latents_reach_the_later_layers(models, dtype, ways):
+    """What the later layers read from the lender's line shows in the logits: with the latent of another token there the
+    plain model is far away, the library is not."""
+    model = models["A"]
+    toks = model.tokens(90, seed=4)
+    want = model.plain(toks)
+    saved = P.latent_attention
+
+    def shifted(h, w, c, eps, past=None, lent=None):
+        lent = {k: torch.roll(v, 1, 0) for k, v in lent.items()} if lent is not None else None
+        return saved(h, w, c, eps, past, lent)
+    try:
+        P.latent_attention = shifted
+        assert rel_err(P.forward(model.cfg, double(model.tensors), toks)[0], want) > 0.2
+    finally:
+        P.latent_attention = saved
+    got = feed(model.engine(dtype), {"r": toks}, lambda n: [40, 41, 89])["r"]
+    assert rel_err(got, want) <= TOL[dtype]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", sorted(CASES))
+def test_unequal_batches_and_slots_used_again(models, name, dtype, ways):
+    """Three batches one after another in the same slots and pages: unequal prompts start together and decode together,
+    the shorter ones end earlier. Against the plain implementation, and against each request alone."""
+    from dryft_amd import SeqStep
+    model = models[name]
+    engine = model.engine(dtype, max_batch=3, max_tokens=64 * 9)
+    batches = [{f"b{b}r{n}": (model.tokens(n, seed=b + 1), k) for n, k in sizes}
+               for b, sizes in enumerate([[(70, 6), (3, 2), (130, 20)], [(1, 0), (66, 65), (20, 3)], [(129, 1), (64, 10)]])]
+    records = list(trace_batches(batches))
+    slot_of, outputs = {}, {}
+    for rec in records:
+        seqs = []
+        for e in rec["entries"]:
+            if e["id"] not in slot_of:
+                slot_of[e["id"]] = engine.acquire(1)[0]
+            seqs.append(SeqStep(slot_of[e["id"]], e["tokens"], e["want"]))
+        outputs[rec["step"]] = engine.step(seqs).cpu()
+        engine.release([slot_of.pop(r) for r in rec["end"]])
+    got = collect_positions(records, outputs)
+    alone = feed(model.engine(dtype), {rid: toks for b in batches for rid, (toks, _) in b.items()}, lambda n: [])
+    for (rid, pos), row in got.items():
+        toks = next(b[rid][0] for b in batches if rid in b)
+        want = model.plain(toks)
+        assert rel_err(row[None], want[pos][None]) <= TOL[dtype], (name, rid, pos)
+        d = row.double() - alone[rid][pos].double()
+        assert float((d - d.mean()).pow(2).mean().sqrt() / want.pow(2).mean().sqrt()) <= (2e-5 if dtype == "float32" else TOL[dtype])
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_a_portion_beside_decoding_and_a_sequence_that_sits_out(models, dtype, ways):
+    from dryft_amd import SeqStep
+    model = models["C"]
+    engine = model.engine(dtype, max_batch=4)
+    a, b, c = model.tokens(100, seed=21), model.tokens(90, seed=22), model.tokens(40, seed=23)
+    sa, sb, sc = engine.acquire(3)
+    got = {"a": [], "b": [], "c": []}
+
+    def step(*entries):
+        out = engine.step([SeqStep(s, t, list(range(len(t)))) for _, s, t in entries]).cpu()
+        at = 0
+        for rid, s, t in entries:
+            if s >= 0:
+                got[rid].append(out[at:at + len(t)])
+                at += len(t)
+    step(("a", sa, a[:70]), ("b", sb, b[:3]))
+    step(("a", sa, a[70:71]), ("x", -1, [1, 2, 3]), ("b", sb, b[3:88]))
+    step(("b", sb, b[88:]), ("c", sc, c), ("a", sa, a[71:73]))
+    step(("x", -1, [5]), ("a", sa, a[73:]))
+    engine.release([sa, sb, sc])
+    for rid, toks in (("a", a), ("b", b), ("c", c)):
+        assert rel_err(torch.cat(got[rid]), model.plain(toks)) <= TOL[dtype], rid
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_long_decoding(models, dtype):
+    """300 tokens one at a time: every chunk of the model passes over decoded tokens several times."""
+    from dryft_amd import SeqStep
+    model = models["A"]
+    engine = model.engine(dtype)
+    toks = model.tokens(300, seed=7)
+    slot = engine.acquire(1)[0]
+    rows = [engine.step([SeqStep(slot, toks[:2], [1])])]
+    for t in toks[2:]:
+        rows.append(engine.step([SeqStep(slot, [t], [0])]))
+    engine.release([slot])
+    assert rel_err(torch.cat(rows), model.plain(toks)[1:]) <= TOL[dtype]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_a_long_prompt_in_segments(models, dtype):
+    """A prompt that the recurrences cut into segments and (in bfloat16) the latent layers run with keys, beside a short
+    one, then decoding; the middle of the long prompt is far from both ends."""
+    from dryft_amd import SeqStep
+    model = models["A"]
+    engine = model.engine(dtype, max_len=1024, max_tokens=64 * 40)
+    long, short = model.tokens(900, seed=11), model.tokens(20, seed=12)
+    want = [model.plain(long), model.plain(short)]
+    slots = engine.acquire(2)
+    out = engine.step([SeqStep(slots[0], long[:897], list(range(897))), SeqStep(slots[1], short[:17], list(range(17)))]).cpu()
+    got = [[out[:897]], [out[897:]]]
+    for k in range(3):
+        out = engine.step([SeqStep(slots[0], [long[897 + k]], [0]), SeqStep(slots[1], [short[17 + k]], [0])]).cpu()
+        got[0].append(out[:1])
+        got[1].append(out[1:])
+    engine.release(slots)
+    for mine, ref in zip(got, want):
+        assert rel_err(torch.cat(mine), ref) <= TOL[dtype]
+
+
+@pytest.mark.parametrize("seed", range(12))
+def test_random_configurations(seed, tmp_path, ways):
+    """Configurations drawn at random: three unequal prompts start together and decode together. float32 must agree with
+    the plain implementation to rounding in every row; in bfloat16 the typical row must (single rows of a deep random
+    model magnify rounding whatever computes them)."""
+    import random
+
+    from dryft_amd import Engine, SeqStep
+    cfg = random_config(random.Random(seed))
+    tensors = tensors_for(cfg, seed)
+    path = write_dir(str(tmp_path / "m"), cfg, tensors)
+    g = np.random.default_rng(seed)
+    reqs = [[int(x) for x in g.integers(0, cfg["vocab"], size=n)] for n in (1, 37, 150)]
+    want = [P.forward(cfg, double(tensors), r)[0] for r in reqs]
+    for dtype in DTYPES if ways == "latents" else ["bfloat16"]:
+        engine = Engine(path, dtype=dtype, max_batch=4, max_len=256, max_tokens=64 * 16, use_graph=False)
+        slots = engine.acquire(3)
+        heads = [max(1, len(r) - 6) for r in reqs]
+        got = [[] for _ in reqs]
+        out = engine.step([SeqStep(s, r[:h], list(range(h))) for s, r, h in zip(slots, reqs, heads)]).cpu()
+        at = 0
+        for i, h in enumerate(heads):
+            got[i].append(out[at:at + h])
+            at += h
+        for k in range(6):
+            live = [(i, s) for i, s in enumerate(slots) if heads[i] + k < len(reqs[i])]
+            if live:
+                out = engine.step([SeqStep(s, [reqs[i][heads[i] + k]], [0]) for i, s in live]).cpu()
+                for j, (i, _) in enumerate(live):
+                    got[i].append(out[j:j + 1])
+        engine.release(slots)
+        for mine, ref in zip(got, want):
+            d = torch.cat(mine).double() - ref
+            d = d - d.mean(-1, keepdim=True)
+            rows = d.pow(2).mean(-1).sqrt() / ref.pow(2).mean().sqrt()
+            if dtype == "float32":
+                assert float(rows.max()) <= TOL[dtype], (seed, float(rows.max()), cfg["layers"])
+            else:
+                assert float(rows.median()) <= 0.05 and float((rows > 0.2).double().mean()) <= 0.03, \
+                    (seed, float(rows.median()), float(rows.max()))
+
+
+def plain_greedy(model, prompt, n):
+    toks, out, logits = list(prompt), [], []
+    for _ in range(n):
+        row = P.forward(model.cfg, double(model.tensors), toks)[0][-1]
+        logits.append(row)
+        out.append(int(row.argmax()))
+        toks.append(out[-1])
+    return out, logits
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["A", "B", "C"])
+def test_greedy_generation_through_the_entry_point(models, name, dtype):
+    """``Engine.generate`` with captured steps: the scheduler, the sampler and the graphs serve this design as they serve
+    the others. Every token is the plain loop's, or one the plain logits leave within the tolerance of the best."""
+    model = models[name]
+    prompts = [model.tokens(n, seed=3) for n in (5, 17, 2)]
+    for use_graph in (True, False):
+        engine = model.engine(dtype, max_batch=4, max_len=64, max_tokens=64 * 4, use_graph=use_graph)
+        got = engine.generate_all(prompts, 8)
+        assert [len(g) for g in got] == [8, 8, 8]
+        for prompt, mine in zip(prompts, got):
+            want, logits = plain_greedy(model, prompt, 8)
+            for t in range(8):
+                if mine[t] != want[t]:
+                    spread = float(logits[t].max() - logits[t].min())
+                    assert float(logits[t].max() - logits[t][mine[t]]) <= 4 * TOL[dtype] * spread, (name, t)
+                    break
+    # a second generation in the same engine reuses slots, pages and captured steps, and repeats the first token for token
+    engine = model.engine(dtype, max_batch=4, max_len=64, max_tokens=64 * 4, use_graph=True)
+    first = engine.generate_all(prompts, 8)
+    assert engine.generate_all(prompts, 8) == first
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_captured_steps_equal_eager_ones(models, dtype):
+    """Many replays of captured decoding steps, with contexts that cross pages, chunks and the graphs' ranges."""
+    model = models["C"]
+    prompts = [model.tokens(n, seed=5) for n in (60, 3, 128, 250)]
+    eager = model.engine(dtype, max_batch=4, max_len=400, max_tokens=64 * 28, use_graph=False).generate_all(prompts, 40)
+    engine = model.engine(dtype, max_batch=4, max_len=400, max_tokens=64 * 28, use_graph=True)
+    for _ in range(2):
+        got = engine.generate_all(prompts, 40)
+        for prompt, a, b in zip(prompts, got, eager):
+            if a != b:                                        # keys cut into other runs round otherwise: a close call at most
+                t = next(i for i in range(40) if a[i] != b[i])
+                row = P.forward(model.cfg, double(model.tensors), prompt + b[:t])[0][-1]
+                assert float((row[a[t]] - row[b[t]]).abs()) <= 4 * TOL[dtype] * float(row.max() - row.min())
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_trace_program(models, dtype, tmp_path):
+    model = models["C"]
+    batches = [{f"r{n}": (model.tokens(n, seed=9), k) for n, k in [(40, 5), (2, 1), (90, 12)]}, {"s": (model.tokens(65, seed=2), 64)}]
+    records = list(trace_batches(batches))
+    live = max(sum(len(t) for t, _ in b.values()) for b in batches)
+    out_dir = str(tmp_path / "out")
+    cmd = [sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", model.dir, "--dtype", dtype, "--out", out_dir,
+           "--max-tokens", str(live)]
+    proc = subprocess.run(cmd, input="".join(json.dumps(r) + "\n" for r in records), capture_output=True, text=True, timeout=600)
+    assert proc.returncode == 0, proc.stderr[-2000:]
+    assert proc.stdout.split("\n")[:-1] == [f"done {r['step']}" for r in records]
+    outputs = {}
+    for r in records:
+        n_want = sum(len(e["want"]) for e in r["entries"])
+        if n_want:
+            outputs[r["step"]] = torch.from_numpy(np.fromfile(os.path.join(out_dir, f"{r['step']}.f32"), dtype="<f4").reshape(n_want, model.vocab))
+    for (rid, pos), row in collect_positions(records, outputs).items():
+        toks = next(b[rid][0] for b in batches if rid in b)
+        assert rel_err(row[None], model.plain(toks)[pos][None]) <= TOL[dtype], (rid, pos)
