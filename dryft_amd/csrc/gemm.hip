@@ -1400,6 +1400,72 @@ DRYFT_API int dryft_gemm_block_f32(const void* x, int64_t x_stride, const void* 
   }
 }
 
+// ------------------------------------------------------------------------------------------- narrow
+// y[M, N] = x . W^T in float32 for at most 64 outputs and any number of rows (gates, routers, low-rank projections): what
+// counts is to read x once and early. A workgroup takes 16 rows; its eight waves split K, four steps of 32 in flight each,
+// operands straight from memory in the matrix cores' layout (W is small and stays in the caches), and are added up
+// in order through LDS. Accumulator entry i of lane (c, g) is output 16 t + 4g + i of row c.
+template <int NT>
+__global__ __launch_bounds__(512) void gemm_narrow_kernel(const bf16_t* __restrict__ x, int64_t x_stride,
+                                                          const bf16_t* __restrict__ w, float* __restrict__ y, int M, int N,
+                                                          int K) {
+  __shared__ f32x4 red[8][NT][WAVE];
+  const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE, c = lane % 16, g = lane / 16;
+  const int64_t row0 = (int64_t)blockIdx.x * 16;
+  const bf16_t* xr = x + min(row0 + c, (int64_t)M - 1) * x_stride;
+  const bf16_t* wr[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t) wr[t] = w + (int64_t)min(16 * t + c, N - 1) * K;
+  f32x4 acc[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 32 * wave; k0 < K; k0 += 4 * 256) {
+    bf16x8 xv[4], wv[4][NT];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int k = k0 + 256 * u + 8 * g, kk = min(k, K - 8);      // beyond the end: the last piece, times zeros
+      xv[u] = *(const bf16x8*)(xr + kk);
+#pragma unroll
+      for (int t = 0; t < NT; ++t) wv[u][t] = *(const bf16x8*)(wr[t] + kk);
+      if (k >= K) xv[u] = zero8g();
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+#pragma unroll
+      for (int t = 0; t < NT; ++t) acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[u][t], xv[u], acc[t], 0, 0, 0);
+  }
+#pragma unroll
+  for (int t = 0; t < NT; ++t) red[wave][t][lane] = acc[t];
+  __syncthreads();
+  for (int e = threadIdx.x; e < NT * WAVE; e += 512) {
+    const int t = e / WAVE, l = e % WAVE;
+    f32x4 sum = red[0][t][l];
+#pragma unroll
+    for (int v = 1; v < 8; ++v) sum += red[v][t][l];
+    const int64_t row = row0 + l % 16;
+    if (row >= M) continue;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int n = 16 * t + 4 * (l / 16) + i;
+      if (n < N) y[row * N + n] = sum[i];
+    }
+  }
+}
+
+DRYFT_API int dryft_gemm_narrow_bf16(const void* x, int64_t x_stride, const void* w, float* y, int M, int N, int K,
+                                     hipStream_t stream) {
+  if (M <= 0 || N <= 0) return 0;
+  if (N > 64 || K < 8 || K % 8 || x_stride % 8) return -1;
+  const dim3 grid((M + 15) / 16), block(512);
+#define NR(T) hipLaunchKernelGGL(gemm_narrow_kernel<T>, grid, block, 0, stream, (const bf16_t*)x, x_stride, (const bf16_t*)w, y, M, N, K)
+  if (N <= 16) NR(1);
+  else if (N <= 32) NR(2);
+  else if (N <= 48) NR(3);
+  else NR(4);
+#undef NR
+  return DRYFT_LAUNCH_CHECK();
+}
+
 // ------------------------------------------------------------------------------------------- rows of 32-bit values
 // At most 16 rows of 32-bit values (decoding in the float32 path): bound by reading W once. A workgroup owns 8
 // weight rows, two per wave, and walks K in chunks of 256: the rows of x for a chunk are staged in LDS once for all

@@ -80,6 +80,7 @@ _SIGNATURES = {
              "dryft_gemm_block_f32": [_P, _L, _P, _P, _I, _I, _I, _I, _P],
              "dryft_gemm_rows_f32": [_P, _L, _P, _P, _I, _I, _I, _P],
              "dryft_gemm_wide_swiglu_bf16": [_P, _L, _P, _P, _I, _I, _I, _I, _I, _P],
+             "dryft_gemm_narrow_bf16": [_P, _L, _P, _P, _I, _I, _I, _P],
              "dryft_sum_partials": [_P, _P, _L, _I, _I, _P]},
     "hyper": {"dryft_hyper_norm": [_P, _I, _I, _P, _I, _I, _L, _P, _P, _P, _P, _P, _P, _I, _I, _I, _F, _I, _P]},
     "wkv": {"dryft_wkv_blend": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _P],
@@ -1075,6 +1076,28 @@ def gemm_block_bf16(x, w, out, swiglu: bool = False, shape: int | None = None) -
         raise KernelError("gemm_block: shape 0 or 1")
     _check(_fn("gemm", "dryft_gemm_block_bf16")(_ptr(x), x.stride(0), _ptr(w), _ptr(out), m, n, k, 1 if swiglu else 0,
                                                 1 if out.dtype == torch.float32 else 0, int(shape), _stream()), "gemm_block_bf16")
+    return out
+
+
+NARROW_OUTPUTS = 64     # the most outputs gemm_narrow takes
+
+
+def gemm_narrow_bf16(x, w, out) -> torch.Tensor:
+    """``x [M, K] @ w[N, K].T`` in float32 for at most ``NARROW_OUTPUTS`` outputs and any number of rows, K a multiple of 8."""
+    _gpu(x, "x", torch.bfloat16)
+    _gpu(w, "w", torch.bfloat16)
+    _gpu(out, "out", torch.float32)
+    m, k = x.shape
+    n = w.shape[0]
+    if not (w.dim() == 2 and w.shape[1] == k and w.is_contiguous() and x.stride(1) == 1):
+        raise KernelError("gemm_narrow: x [M,K] row-major, w [N,K] contiguous")
+    if not (n <= NARROW_OUTPUTS and k >= 8 and k % 8 == 0 and x.stride(0) % 8 == 0 and x.data_ptr() % 16 == 0 and
+            w.data_ptr() % 16 == 0):
+        raise KernelError(f"gemm_narrow: at most {NARROW_OUTPUTS} outputs, K a multiple of 8, operands 16-byte aligned")
+    if not (out.shape == (m, n) and out.is_contiguous()):
+        raise KernelError(f"gemm_narrow: out must be contiguous [{m},{n}]")
+    _check(_fn("gemm", "dryft_gemm_narrow_bf16")(_ptr(x), x.stride(0), _ptr(w), _ptr(out), m, n, k, _stream()),
+           "gemm_narrow_bf16")
     return out
 
 

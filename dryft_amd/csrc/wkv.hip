@@ -53,7 +53,7 @@ template <typename W, int R, bool LOGSIG>
 __global__ __launch_bounds__(256) void wkv_decay_kernel(const float* __restrict__ low, const W* __restrict__ up,
                                                         const float* __restrict__ bias, float* __restrict__ decay,
                                                         int rows, int n_out, int rank, float factor) {
-  extern __shared__ float t_low[];           // [R][rank]
+  extern __shared__ __attribute__((aligned(16))) float t_low[];           // [R][rank]
   const int64_t row0 = (int64_t)blockIdx.x * R;
   for (int i = threadIdx.x; i < R * rank; i += blockDim.x) {
     const int64_t row = row0 + i / rank;
@@ -72,9 +72,13 @@ __global__ __launch_bounds__(256) void wkv_decay_kernel(const float* __restrict_
         float w8[8];
         load8_as_float(w + j, w8);
 #pragma unroll
-        for (int e = 0; e < 8; ++e)
+        for (int r = 0; r < R; ++r) {
+          const vf4 a = *(const vf4*)(t_low + r * rank + j), b = *(const vf4*)(t_low + r * rank + j + 4);
 #pragma unroll
-          for (int r = 0; r < R; ++r) acc[r] += w8[e] * t_low[r * rank + j + e];
+          for (int e = 0; e < 4; ++e) acc[r] += w8[e] * a[e];
+#pragma unroll
+          for (int e = 0; e < 4; ++e) acc[r] += w8[4 + e] * b[e];
+        }
       }
     }
     for (; j < rank; ++j) {
@@ -101,7 +105,8 @@ static int launch_decay(const float* low, const void* up, const float* bias, flo
   const bool many = rows >= 64;
   const size_t lds = (size_t)(many ? 8 : 1) * rank * sizeof(float);
   // few rows: a workgroup per 256 outputs, so that the chip has work
-  const dim3 grid = many ? dim3((rows + 7) / 8, 1) : dim3(rows, (n_out + 255) / 256);
+  // and four of them for the rows that share what they read where there are many
+  const dim3 grid = many ? dim3((rows + 7) / 8, n_out > 1024 ? 4 : 1) : dim3(rows, (n_out + 255) / 256);
 #define DK(WW, R)                                                                                                     \
   hipLaunchKernelGGL((wkv_decay_kernel<WW, R, LOGSIG>), grid, dim3(256), lds, stream, low, (const WW*)up, bias, decay,   \
                      rows, n_out, rank, factor)

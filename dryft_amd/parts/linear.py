@@ -22,6 +22,8 @@ engine/dryft_qwen3/model.py:153, 179-180, 237, 258-261). Here:
 * bfloat16, 65 to 256 rows (short prompts, decoding at large batch) where the consumer adds partial sums and K is a
   multiple of 64: this library's kernel whose waves each own rows of x, operands straight into LDS (``tall_plan``);
   the fused gate/up product of as many rows goes to its other form (``tall_swiglu_ok``);
+* bfloat16, more than 16 rows, float32 results of at most 64 outputs (gates, routers, low-rank projections): this
+  library's kernel that reads the rows once and splits K over the waves of a workgroup;
 * bfloat16, otherwise (prompts, decoding at large batch): the vendor library through
   ``torch.mm``, as in the reference; float32 results of many rows and output sizes the
   library does not take are this library's block kernel (128 x 128 or 256 x 256 outputs
@@ -187,6 +189,8 @@ def linear(x: torch.Tensor, w: torch.Tensor, *, out_dtype: torch.dtype | None = 
                 return ops.gemm_block_f32(x, w, out, shape=0)
         return ops.gemm_tiled(x, w, out)
     few_ok = few_rows_ok(x, w)
+    if out_dtype == torch.float32 and not allow_partials and m > STREAM_ROWS and n <= ops.NARROW_OUTPUTS and few_ok:
+        return ops.gemm_narrow_bf16(x, w, torch.empty((m, n), dtype=torch.float32, device=x.device))
     library_ok = k % 8 == 0 and n % 8 == 0 and x.is_contiguous() and out_dtype == x.dtype
     if m <= STREAM_ROWS and few_ok:
         splits, group, depth = stream_plan(n, k, allow_partials)

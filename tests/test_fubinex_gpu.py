@@ -260,6 +260,18 @@ def test_linear_attention_kernels(H, D, Dv, decay, rot_dims, dtype):
             assert float((state[slot].cpu().double() - end).abs().max() / end.pow(2).mean().sqrt()) <= 2e-5
 
 
+@pytest.mark.parametrize("n,k", [(1, 8), (16, 72), (20, 2048), (33, 1000), (64, 4096)])
+def test_narrow_product(n, k):
+    from dryft_amd.csrc import ops
+    g = torch.Generator().manual_seed(n)
+    w = (torch.randn(n, k, generator=g) / k ** 0.5).to(torch.bfloat16)
+    for rows in (17, 64, 301):
+        x = torch.randn(rows, k + 8, generator=g).to(torch.bfloat16)
+        out = torch.full((rows, n), 3.0, device=DEV)
+        ops.gemm_narrow_bf16(x.to(DEV)[:, 8:], w.to(DEV), out)
+        assert torch.allclose(out.cpu().double(), x[:, 8:].double() @ w.double().T, atol=2e-5)
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("heads,k,n,rot_dim,pairs", [(3, 12, 14, 6, True), (20, 8, 40, 16, True), (2, 128, 512, 64, False), (5, 70, 33, 0, False)])
 def test_head_product(dtype, heads, k, n, rot_dim, pairs):
