@@ -11,6 +11,7 @@ from __future__ import annotations
 
 import json
 import os
+from dataclasses import dataclass
 from typing import Any, Callable
 
 _MISSING = object()
@@ -88,6 +89,42 @@ class KeyReader:
     def finish(self, what: str) -> None:
         if self.problems:
             raise ConfigError(what, self.problems)
+
+
+@dataclass(frozen=True)
+class LoopConfig:
+    """Layers ``start`` .. ``stop - 1`` run ``times`` times in a row with the same weights."""
+
+    start: int
+    stop: int
+    times: int
+
+    @classmethod
+    def read(cls, r: KeyReader, n_layers: int) -> "LoopConfig | None":
+        """The file's ``loop`` (absent or null: None), problems noted in ``r``."""
+        raw = r.raw.get("loop")
+        if raw is None:
+            return None
+        if not isinstance(raw, dict):
+            r.problems.append("loop: expected an object")
+            return None
+        lp = KeyReader(raw)
+        loop = cls(lp.integer("start", minimum=0), lp.integer("stop", minimum=0), lp.integer("times"))
+        r.problems += [f"loop.{p}" for p in lp.problems]
+        if not lp.problems and not 0 <= loop.start < loop.stop <= n_layers:
+            r.problems.append(f"loop: start {loop.start} .. stop {loop.stop} is no run of the {n_layers} layers")
+        return loop
+
+    def to_dict(self) -> dict[str, int]:
+        return {"start": self.start, "stop": self.stop, "times": self.times}
+
+
+def layer_order(n_layers: int, loop: LoopConfig | None) -> list[tuple[int, int | None]]:
+    """The layers as they run, each with the number of the pass that begins at it (None: none does)."""
+    if loop is None:
+        return [(i, None) for i in range(n_layers)]
+    passes = [(i, t if i == loop.start else None) for t in range(loop.times) for i in range(loop.start, loop.stop)]
+    return [(i, None) for i in range(loop.start)] + passes + [(i, None) for i in range(loop.stop, n_layers)]
 
 
 def read_config_json(model_dir: str) -> dict[str, Any]:

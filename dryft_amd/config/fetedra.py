@@ -15,11 +15,10 @@ from __future__ import annotations
 from dataclasses import dataclass
 from typing import Any
 
-from ..limits import MAX_HEAD_DIM
+from ..limits import MAX_HEAD_DIM, MAX_STREAMS
 from .base import ConfigError, KeyReader
 
 MIXER_TYPES = ("wkv", "latent_attention")
-MAX_STREAMS = 8          # what the stream kernel keeps in registers per column
 
 
 @dataclass(frozen=True)

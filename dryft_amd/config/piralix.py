@@ -14,7 +14,7 @@ from dataclasses import dataclass
 from typing import Any
 
 from ..limits import MAX_HEAD_DIM
-from .base import ConfigError, KeyReader
+from .base import ConfigError, KeyReader, LoopConfig
 
 MIXER_TYPES = ("attention", "mlstm", "rglru")
 
@@ -34,13 +34,6 @@ class LayerConfig:
 
     def mixer_dict(self) -> dict[str, Any]:
         return dict(self.mixer)
-
-
-@dataclass(frozen=True)
-class LoopConfig:
-    start: int
-    stop: int
-    times: int
 
 
 @dataclass(frozen=True)
@@ -84,13 +77,7 @@ class PiralixConfig:
                     mlp_items = (("kind", "dense"), ("ff", f.integer("ff")), ("limit", f.number("limit")))
                     r.problems += [f"{where}.mlp.{p}" for p in f.problems]
             layers.append(LayerConfig(entry["type"], tuple(mixer.items()), mlp_items))
-        loop = None
-        if raw.get("loop") is not None:
-            lp = _sub(r, raw, "loop")
-            loop = LoopConfig(lp.integer("start", minimum=0), lp.integer("stop", minimum=0), lp.integer("times"))
-            r.problems += [f"loop.{p}" for p in lp.problems]
-            if not lp.problems and not (0 <= loop.start < loop.stop <= len(layers_raw)):
-                r.problems.append(f"loop: start {loop.start} .. stop {loop.stop} is no run of the {len(layers_raw)} layers")
+        loop = LoopConfig.read(r, len(layers_raw))
         r.problems += [f"norm.{p}" for p in norm.problems]
         r.finish("unsupported or malformed Piralix config.json")
         return cls(vocab, width, eps, tuple(layers), loop, tuple(raw.items()))
@@ -108,7 +95,7 @@ class PiralixConfig:
                 mixer["rot"] = {"dims": rot.dims, "base": rot.base, "scaling": dict(rot.scaling) if rot.scaling else None}
             out["layers"].append({"type": layer.type, "mixer": mixer, "mlp": dict(layer.mlp) if layer.mlp else None})
         if self.loop:
-            out["loop"] = {"start": self.loop.start, "stop": self.loop.stop, "times": self.loop.times}
+            out["loop"] = self.loop.to_dict()
         return out
 
 

@@ -52,6 +52,67 @@ DRYFT_API int dryft_silu_mul(const void* gu, void* y, int n_rows, int inter, int
   return DRYFT_LAUNCH_CHECK();
 }
 
+// The same with relu in the place of silu: y = T( max(g, 0) * u ), in float, rounded once.
+template <typename T>
+__global__ void relu_mul_kernel(const T* __restrict__ gu, T* __restrict__ y, int inter, int64_t gu_stride) {
+  const int64_t row = blockIdx.x;
+  const int i = blockIdx.y * blockDim.x + threadIdx.x;
+  if (i >= inter) return;
+  const float g = load_as_float(gu + row * gu_stride + i), u = load_as_float(gu + row * gu_stride + inter + i);
+  store_from_float(y + row * inter + i, fmaxf(g, 0.f) * u);
+}
+
+// Eight values per thread with 16-byte loads and stores, for widths and strides that are multiples of 8.
+__global__ __launch_bounds__(256) void relu_mul_vec_kernel(const bf16_t* __restrict__ gu, bf16_t* __restrict__ y,
+                                                           int inter, int64_t gu_stride) {
+  const int64_t row = blockIdx.x;
+  const int i = (blockIdx.y * blockDim.x + threadIdx.x) * 8;
+  if (i >= inter) return;
+  float g[8], u[8];
+  load8_as_float(gu + row * gu_stride + i, g);
+  load8_as_float(gu + row * gu_stride + inter + i, u);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) g[j] = fmaxf(g[j], 0.f) * u[j];
+  store8_from_float(y + row * inter + i, g);
+}
+
+DRYFT_API int dryft_relu_mul(const void* gu, void* y, int n_rows, int inter, int64_t gu_stride, int is_f32,
+                             hipStream_t stream) {
+  if (n_rows <= 0) return 0;
+  if (!is_f32 && inter % 8 == 0 && gu_stride % 8 == 0 && (((uintptr_t)gu | (uintptr_t)y) & 15) == 0) {
+    dim3 vgrid(n_rows, (inter / 8 + 255) / 256);
+    hipLaunchKernelGGL(relu_mul_vec_kernel, vgrid, dim3(256), 0, stream, (const bf16_t*)gu, (bf16_t*)y, inter, gu_stride);
+    return DRYFT_LAUNCH_CHECK();
+  }
+  dim3 grid(n_rows, (inter + 255) / 256), block(256);
+  if (is_f32)
+    hipLaunchKernelGGL(relu_mul_kernel<float>, grid, block, 0, stream, (const float*)gu, (float*)y, inter, gu_stride);
+  else
+    hipLaunchKernelGGL(relu_mul_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)gu, (bf16_t*)y, inter, gu_stride);
+  return DRYFT_LAUNCH_CHECK();
+}
+
+// x <- cap * tanh(x / cap), float, in place: capped logits.
+__global__ __launch_bounds__(256) void cap_values_kernel(float* __restrict__ x, int64_t n, float cap) {
+  const int64_t stride = (int64_t)gridDim.x * blockDim.x, first = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+  vf4* x4 = (vf4*)x;                                         // a tensor starts at a multiple of 16 bytes (the host checks)
+  for (int64_t i = first; i < n / 4; i += stride) {
+    vf4 v = x4[i];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = cap * tanhf(v[j] / cap);
+    x4[i] = v;
+  }
+  for (int64_t i = n / 4 * 4 + first; i < n; i += stride) x[i] = cap * tanhf(x[i] / cap);
+}
+
+DRYFT_API int dryft_cap_values(float* x, int64_t n, float cap, hipStream_t stream) {
+  if (n <= 0) return 0;
+  if (!(cap > 0.f) || ((uintptr_t)x & 15)) return -1;
+  const int64_t blocks = (n / 4 + 255) / 256 + 1;
+  hipLaunchKernelGGL(cap_values_kernel, dim3((unsigned)(blocks < 4096 ? blocks : 4096)), dim3(256), 0, stream, x, n, cap);
+  return DRYFT_LAUNCH_CHECK();
+}
+
 // A gated linear unit with clamped halves: g = min(gu[:, :I], limit), u = clamp(gu[:, I:], -limit, limit),
 // y = T( g * sigmoid(alpha * g) * (u + 1) ), evaluated in float and rounded once.
 template <typename T>

@@ -393,13 +393,24 @@ __host__ __device__ constexpr size_t causal_page_bytes(int head_dim, int units) 
 }
 #define CAUSAL_REL_LDS_BYTES (16 * 1024)     // the most a bias table may take there
 
-template <int KB, bool FULL, int GP, int RP>
+// Two maps of one query head over the same values (differential attention). A key's row holds the two maps' keys side
+// by side, `map_dim` features each (a multiple of 8); query head 2 h + m is map m of output head h. With the two maps'
+// outputs a1 and a2, o = a1 - lambda * a2, divided by its root mean square over the first v_dim features and times
+// `post`. Output rows are [heads / 2, v_dim].
+struct MapPair {
+  int map_dim, v_dim;
+  float lambda, post, eps;
+};
+
+// DIFF: the wave's two units are the two maps of one head (GP = 2), each with keys of its own.
+template <int KB, bool FULL, int GP, int RP, bool DIFF>
 __global__ __launch_bounds__(256, (GP * RP * KB <= 8 && KB <= 4) ? (GP * RP == 1 ? 3 : 2) : 1) void attn_causal_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages,
     const int* __restrict__ page_table, int max_pages, const int* __restrict__ seq_slot,
     const int* __restrict__ cu_rows, const int* __restrict__ tile_cu, const int* __restrict__ seq_start, int n_seqs,
     bf16_t* __restrict__ out, int n_heads, int n_kv, int head_dim, float scale, int window, ScoreOptions opt,
-    int rel_lds) {
+    int rel_lds, MapPair pair) {
+  static_assert(!DIFF || (GP == 2 && RP == 1), "two maps are the two units of a wave");
   extern __shared__ __attribute__((aligned(16))) unsigned char lds_raw[];
   constexpr int U = GP * RP, TILE_ROWS = 64 * RP, WAVE_ROWS = 16 * RP;
   ScoreCap cap = score_cap(opt, scale, n_heads);
@@ -417,7 +428,9 @@ __global__ __launch_bounds__(256, (GP * RP * KB <= 8 && KB <= 4) ? (GP * RP == 1
   // Two heads per wave: a workgroup takes one tile from each end of the list (grid: pairs of tiles x heads / 2).
   // Otherwise: one tile per workgroup, the ones with the most pages first, heads fastest (grid: heads x tiles),
   // so that the short tiles fill the compute units that the long ones leave.
-  constexpr bool PAIRED = GP != 1;
+  constexpr bool PAIRED = GP != 1 && !DIFF;
+  constexpr int KQ = DIFF ? (KB + 1) / 2 : KB;                // blocks of 32 features of a query
+  const int q_dim = DIFF ? pair.map_dim : head_dim;
   const int head0 = (PAIRED ? blockIdx.y : blockIdx.x) * GP;
   const int first_tile = PAIRED ? blockIdx.x : blockIdx.y;
   const int n_tiles = count_tiles<RP>(seq_slot, cu_rows, tile_cu, n_seqs);   // tiles of TILE_ROWS rows over all sequences
@@ -459,7 +472,7 @@ __global__ __launch_bounds__(256, (GP * RP * KB <= 8 && KB <= 4) ? (GP * RP == 1
   RowBlock<KB> st[U];                                         // unit u: head u % GP, rows of tile u / GP
 #pragma unroll
   for (int u = 0; u < U; ++u)
-    init_rows<KB>(st[u], q + (row[u / GP] * n_heads + head0 + u % GP) * head_dim, row_valid[u / GP], head_dim);
+    init_rows<KB>(st[u], q + (row[u / GP] * n_heads + head0 + u % GP) * q_dim, row_valid[u / GP], q_dim);
   const int lo_wave = first_seen(pos_wave, window, chunk);
   const int hi_wave = pos_wave + wave_rows - 1;               // below lo_wave for a wave without rows
   const int lo_tile = first_seen(pos_tile, window, chunk);
@@ -505,7 +518,16 @@ __global__ __launch_bounds__(256, (GP * RP * KB <= 8 && KB <= 4) ? (GP * RP == 1
 #pragma unroll
         for (int u = 0; u < U; ++u) s[u][t] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int kb = 0; kb < KB; ++kb) {
+        for (int kb = 0; kb < KQ; ++kb) {
+          if (DIFF) {                                         // a unit's own keys; behind them the query holds zeros
+            const int d = min(32 * kb + 8 * g, q_dim - 8);
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+              const bf16x8 a = load8(k_lds + (16 * t + c) * (head_dim + K_PAD) + u * q_dim + d);
+              s[u][t] = MFMA16(a, st[u].q[kb], s[u][t]);
+            }
+            continue;
+          }
           const int d = FULL ? 32 * kb + 8 * g : min(32 * kb + 8 * g, head_dim - 8);
           const bf16x8 a = load8(k_lds + (16 * t + c) * (head_dim + K_PAD) + d);
 #pragma unroll
@@ -547,6 +569,47 @@ __global__ __launch_bounds__(256, (GP * RP * KB <= 8 && KB <= 4) ? (GP * RP == 1
   float row_l[U];
 #pragma unroll
   for (int u = 0; u < U; ++u) row_l[u] = row_sum<KB>(st[u]);
+  if (DIFF) {
+    if (row_valid[0]) {
+      if (opt.sink != nullptr) {
+#pragma unroll
+        for (int u = 0; u < U; ++u) row_l[u] += sink_term(opt.sink, head0 + u, st[u].m);
+      }
+    }
+    const float w1 = row_valid[0] ? 1.f / row_l[0] : 0.f, w2 = row_valid[0] ? pair.lambda / row_l[U - 1] : 0.f;
+    float ss = 0.f;
+#pragma unroll
+    for (int dt = 0; dt < 2 * KB; ++dt)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float o = st[0].o[dt][i] * w1 - st[U - 1].o[dt][i] * w2;
+        st[0].o[dt][i] = o;
+        ss += 16 * dt + 4 * g + i < pair.v_dim ? o * o : 0.f;
+      }
+    ss += __shfl_xor(ss, 16, WAVE);                           // the four lanes that share a row
+    ss += __shfl_xor(ss, 32, WAVE);
+    const float r = pair.post / sqrtf(ss / (float)pair.v_dim + pair.eps);
+    if (row_valid[0]) {
+      bf16_t* o = out + (row[0] * (n_heads / 2) + head0 / 2) * pair.v_dim;
+#pragma unroll
+      for (int dt = 0; dt < 2 * KB; ++dt) {
+        const int d0 = 16 * dt + 4 * g;
+        if (pair.v_dim % 4 == 0) {                            // then the address is a multiple of 8 bytes
+          if (d0 < pair.v_dim) {
+            bf16x4 v;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) v[i] = to_bf16(st[0].o[dt][i] * r);
+            *(bf16x4*)(o + d0) = v;
+          }
+        } else {
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            if (d0 + i < pair.v_dim) o[d0 + i] = float_to_bf16(st[0].o[dt][i] * r);
+        }
+      }
+    }
+    continue;
+  }
 #pragma unroll
   for (int u = 0; u < U; ++u) {
     if (!row_valid[u / GP]) continue;
@@ -1130,7 +1193,7 @@ __global__ __launch_bounds__(64 * SPLIT_WAVES, 2) void attn_split_kernel(
       l += wgt * merge_ml[w][r][1];
       o += wgt * merge_o[w][r][d];
     }
-    if (n_splits == 1) {                                   // nothing to combine: this is the result
+    if (n_splits == 1 && out != nullptr) {                 // nothing to combine: this is the result
       if (opt.sink != nullptr && m != -INFINITY) l += sink_term(opt.sink, kvh * group + hb * 16 + r, m);
       out[(row * n_heads + kvh * group + hb * 16 + r) * head_dim + d] = float_to_bf16(l > 0.f ? o / l : 0.f);
       continue;
@@ -1196,6 +1259,69 @@ __global__ __launch_bounds__(COMBINE_THREADS) void attn_combine_kernel(const flo
   }
 }
 
+// The same for the two maps of a head (MapPair above): query heads 2 h and 2 h + 1 of the partial results become one
+// row of v_dim features, o = a1 - lambda * a2 divided by its root mean square and times post.
+template <int COMBINE_HELD>
+__global__ __launch_bounds__(COMBINE_THREADS) void attn_combine_maps_kernel(const float* __restrict__ part_o,
+                                                                const float* __restrict__ part_ml,
+                                                                const int* __restrict__ seq_slot,
+                                                                const int* __restrict__ cu_rows, bf16_t* __restrict__ out,
+                                                                int n_heads, int head_dim, int n_splits,
+                                                                const float* __restrict__ sink, MapPair pair) {
+  __shared__ float wgt[2][COMBINE_MAX_SPLITS];
+  __shared__ float scratch[16];
+  const int seq = blockIdx.x, head = blockIdx.y, tid = threadIdx.x, wave = tid / WAVE, lane = tid % WAVE;
+  const int64_t row = cu_rows[seq];
+  const float* ml = part_ml + ((int64_t)seq * n_heads + 2 * head) * n_splits * 2;
+  const float* po = part_o + ((int64_t)seq * n_heads + 2 * head) * n_splits * head_dim;
+  const int64_t map_stride = (int64_t)n_splits * head_dim;
+  const bool live = seq_slot[seq] >= 0;
+  float held[2][2][COMBINE_HELD];                             // [map][feature of the thread][split]
+#pragma unroll
+  for (int m = 0; m < 2; ++m)
+#pragma unroll
+    for (int k = 0; k < 2; ++k) {
+      const int d = min(tid + k * COMBINE_THREADS, head_dim - 1);
+#pragma unroll
+      for (int s = 0; s < COMBINE_HELD; ++s) held[m][k][s] = po[m * map_stride + min(s, n_splits - 1) * head_dim + d];
+    }
+  {                                       // wave m turns map m's (m_s, l_s) into weights, the sum's inverse included
+    const float* mine = ml + (int64_t)wave * n_splits * 2;
+    const float ms = (live && lane < n_splits) ? mine[2 * lane] : -INFINITY;
+    const float ls = (live && lane < n_splits) ? mine[2 * lane + 1] : 0.f;
+    const float m = wave_max(ms);
+    const float w = (ms == -INFINITY) ? 0.f : exp2f(ms - m);
+    float l = wave_sum(w * ls);
+    if (sink != nullptr && m != -INFINITY) l += sink_term(sink, 2 * head + wave, m);
+    if (lane < n_splits) wgt[wave][lane] = l > 0.f ? w / l : 0.f;
+  }
+  __syncthreads();
+  float o[2], ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < 2; ++k) {
+    const int d = tid + k * COMBINE_THREADS;
+    float a[2];
+#pragma unroll
+    for (int m = 0; m < 2; ++m) {
+      a[m] = 0.f;
+#pragma unroll
+      for (int s = 0; s < COMBINE_HELD; ++s)
+        if (s < n_splits) a[m] += wgt[m][s] * held[m][k][s];
+      if (d < head_dim)
+        for (int s = COMBINE_HELD; s < n_splits; ++s) a[m] += wgt[m][s] * po[m * map_stride + s * head_dim + d];
+    }
+    o[k] = a[0] - pair.lambda * a[1];
+    ss += d < pair.v_dim ? o[k] * o[k] : 0.f;
+  }
+  ss = block_sum(ss, scratch);
+  const float r = pair.post / sqrtf(ss / (float)pair.v_dim + pair.eps);
+#pragma unroll
+  for (int k = 0; k < 2; ++k) {
+    const int d = tid + k * COMBINE_THREADS;
+    if (d < pair.v_dim) out[(row * (n_heads / 2) + head) * pair.v_dim + d] = float_to_bf16(o[k] * r);
+  }
+}
+
 #define DISPATCH_KB(KBV, CALL)                                                      \
   switch (KBV) {                                                                    \
     case 1: { constexpr int KB = 1; CALL; } break;                                  \
@@ -1213,15 +1339,16 @@ static int head_shape_ok(int n_heads, int n_kv, int head_dim) {
   return head_dim > 0 && head_dim % 16 == 0 && head_dim <= 256 && n_kv > 0 && n_heads % n_kv == 0;
 }
 
-template <int GP, int RP>
+template <int GP, int RP, bool DIFF = false>
 static int launch_causal(const void* q, const void* k_pages, const void* v_pages, const int* page_table, int max_pages,
                          const int* seq_slot, const int* cu_rows, const int* tile_cu, const int* seq_start, int n_seqs,
                          int max_tiles, void* out, int n_heads, int n_kv, int head_dim, float scale, int window,
-                         ScoreOptions opt, hipStream_t stream) {
+                         ScoreOptions opt, hipStream_t stream, MapPair pair = {}) {
   dim3 grid((max_tiles + 1) / 2, n_heads / GP), block(256);
   // max_tiles bounds the 64-row tiles of the sequences that take part. Tiles of 128 rows: a sequence with t
   // 64-row tiles has (t + 1) / 2 of them, so all together at most (max_tiles + n_seqs) / 2.
   if (GP == 1) grid = dim3(n_heads, RP == 1 ? max_tiles : (max_tiles + n_seqs + 1) / 2);
+  if (DIFF) grid = dim3(n_heads / 2, max_tiles);
   if (grid.y > 65535) return -1;
   // two pages of keys [64][D+8] and two of values [D][64+8] (one with one unit per wave)
   const size_t rel_bytes = opt.rel != nullptr ? (size_t)GP * opt.n_dist * sizeof(float) : 0;
@@ -1229,13 +1356,13 @@ static int launch_causal(const void* q, const void* k_pages, const void* v_pages
   const size_t lds = causal_page_bytes(head_dim, GP * RP) + (rel_lds ? rel_bytes : 0);
 #define LAUNCH_CAUSAL(FULLV)                                                                                       \
   {                                                                                                                \
-    auto kernel = attn_causal_kernel<KB, FULLV, GP, RP>;                                                           \
+    auto kernel = attn_causal_kernel<KB, FULLV, GP, RP, DIFF>;                                                     \
     if (lds > 64 * 1024 &&                                                                                          \
         hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) \
       return -1;                                                                                                   \
     hipLaunchKernelGGL(kernel, grid, block, lds, stream, (const bf16_t*)q, (const bf16_t*)k_pages,                 \
                        (const bf16_t*)v_pages, page_table, max_pages, seq_slot, cu_rows, tile_cu, seq_start, n_seqs, \
-                       (bf16_t*)out, n_heads, n_kv, head_dim, scale, window, opt, rel_lds);                        \
+                       (bf16_t*)out, n_heads, n_kv, head_dim, scale, window, opt, rel_lds, pair);                  \
   }
   if (head_dim % 32 == 0) {
     DISPATCH_KB(head_dim / 32, LAUNCH_CAUSAL(true));
@@ -1355,7 +1482,8 @@ DRYFT_API int dryft_attn_causal_projected_bf16(const void* qkv, int64_t qkv_stri
 static int launch_split(const void* q, const void* k_pages, const void* v_pages, const int* page_table, int max_pages,
                         const int* seq_slot, const int* cu_rows, const int* kv_len, int n_seqs, float* part_o,
                         float* part_ml, int n_splits, void* out, int n_heads, int n_kv, int head_dim, float scale,
-                        int window, FusedQKV fused, hipStream_t stream, ScoreOptions opt = {0.f, nullptr}) {
+                        int window, FusedQKV fused, hipStream_t stream, ScoreOptions opt = {0.f, nullptr},
+                        const MapPair* pair = nullptr) {
   if (n_seqs <= 0) return 0;
   if (!head_shape_ok(n_heads, n_kv, head_dim) || n_splits < 1 || n_splits > COMBINE_MAX_SPLITS) return -1;
   const int group = n_heads / n_kv, blocks = (group + 15) / 16;
@@ -1365,7 +1493,7 @@ static int launch_split(const void* q, const void* k_pages, const void* v_pages,
   hipLaunchKernelGGL((attn_split_kernel<KB, FULLV>), grid, block, 0, stream, (const bf16_t*)q, (const bf16_t*)k_pages, \
                      (const bf16_t*)v_pages, page_table, max_pages, seq_slot, cu_rows, kv_len, part_o, part_ml,    \
                      n_heads, n_kv, head_dim, scale, window, n_splits, fused, (bf16_t*)k_pages, (bf16_t*)v_pages,       \
-                     (bf16_t*)out, opt)
+                     (bf16_t*)(pair != nullptr ? nullptr : out), opt)
   if (head_dim % 32 == 0) {
     DISPATCH_KB(head_dim / 32, LAUNCH_SPLIT(true));
   } else {
@@ -1373,7 +1501,18 @@ static int launch_split(const void* q, const void* k_pages, const void* v_pages,
   }
 #undef LAUNCH_SPLIT
   int rc = DRYFT_LAUNCH_CHECK();
-  if (rc || n_splits == 1) return rc;
+  if (rc) return rc;
+  if (pair != nullptr) {
+#define COMBINE_MAPS(HELD)                                                                                          \
+  hipLaunchKernelGGL(attn_combine_maps_kernel<HELD>, dim3(n_seqs, n_heads / 2), dim3(COMBINE_THREADS), 0, stream,    \
+                     part_o, part_ml, seq_slot, cu_rows, (bf16_t*)out, n_heads, head_dim, n_splits, opt.sink, *pair)
+    if (n_splits <= 4) COMBINE_MAPS(4);
+    else if (n_splits <= 8) COMBINE_MAPS(8);
+    else COMBINE_MAPS(16);
+#undef COMBINE_MAPS
+    return DRYFT_LAUNCH_CHECK();
+  }
+  if (n_splits == 1) return rc;
 #define COMBINE(HELD)                                                                                              \
   hipLaunchKernelGGL(attn_combine_kernel<HELD>, dim3(n_seqs, n_heads), dim3(COMBINE_THREADS), 0, stream, part_o,   \
                      part_ml, seq_slot, cu_rows, (bf16_t*)out, n_heads, head_dim, n_splits, opt.sink)
@@ -1414,4 +1553,40 @@ DRYFT_API int dryft_attn_decode_fused_bf16(const void* qkv, int64_t qkv_stride, 
                     (const bf16_t*)cos_t, (const bf16_t*)sin_t, rot, write_kv};
   return launch_split(nullptr, k_pages, v_pages, page_table, max_pages, seq_slot, cu_rows, kv_len, n_seqs, part_o,
                       part_ml, n_splits, out, n_heads, n_kv, head_dim, scale, window, fused, stream);
+}
+
+static int pair_ok(const MapPair& p, int n_heads, int n_kv, int head_dim) {
+  return n_kv > 0 && n_heads % (2 * n_kv) == 0 && p.map_dim > 0 && p.map_dim % 8 == 0 && 2 * p.map_dim <= head_dim &&
+         p.v_dim > 0 && p.v_dim <= head_dim;
+}
+
+// Differential attention of steps with many rows per sequence: q [rows, n_heads, map_dim] holds the two maps of every
+// head as neighbouring query heads, pages of keys rows of head_dim values (map 1, map 2, zeros), pages of values
+// head_dim features of which the first v_dim count, out [rows, n_heads / 2, v_dim].
+DRYFT_API int dryft_attn_causal_diff_bf16(const void* q, const void* k_pages, const void* v_pages, const int* page_table,
+                                          int max_pages, const int* seq_slot, const int* cu_rows, const int* tile_cu,
+                                          const int* seq_start, int n_seqs, int max_tiles, void* out, int n_heads,
+                                          int n_kv, int head_dim, int map_dim, int v_dim, float scale, int window,
+                                          float lambda, float post, float eps, hipStream_t stream) {
+  if (n_seqs <= 0 || max_tiles <= 0) return 0;
+  const MapPair pair = {map_dim, v_dim, lambda, post, eps};
+  if (!head_shape_ok(n_heads, n_kv, head_dim) || !pair_ok(pair, n_heads, n_kv, head_dim)) return -1;
+  return launch_causal<2, 1, true>(q, k_pages, v_pages, page_table, max_pages, seq_slot, cu_rows, tile_cu, seq_start,
+                                   n_seqs, max_tiles, out, n_heads, n_kv, head_dim, scale, window,
+                                   ScoreOptions{0.f, nullptr, 0, nullptr, 0}, stream, pair);
+}
+
+// The same for one row per sequence. q is [rows, n_heads, head_dim] here: a map's query sits where its keys sit in a
+// page's row, with zeros around it, so that the maps of all heads of a kv head share the 16 rows of a tile.
+DRYFT_API int dryft_attn_split_diff_bf16(const void* q, const void* k_pages, const void* v_pages, const int* page_table,
+                                         int max_pages, const int* seq_slot, const int* cu_rows, const int* kv_len,
+                                         int n_seqs, float* part_o, float* part_ml, int n_splits, void* out, int n_heads,
+                                         int n_kv, int head_dim, int v_dim, float scale, int window, float lambda,
+                                         float post, float eps, hipStream_t stream) {
+  FusedQKV none = {};
+  const MapPair pair = {8, v_dim, lambda, post, eps};          // where the maps' keys sit is in q
+  if (!pair_ok(pair, n_heads, n_kv, head_dim)) return -1;
+  return launch_split(q, k_pages, v_pages, page_table, max_pages, seq_slot, cu_rows, kv_len, n_seqs, part_o, part_ml,
+                      n_splits, out, n_heads, n_kv, head_dim, scale, window, none, stream,
+                      ScoreOptions{0.f, nullptr, 0, nullptr, 0}, &pair);
 }

@@ -15,7 +15,9 @@
 // float (exact_p), for designs that ask for float attention weights also in bfloat16; chunks, where a row sees
 // the keys of its own run of `chunk` positions only (runs counted from position 0: lo = pos - pos % chunk); and a
 // learned bias by distance, rel[min(pos - j, n_dist - 1)][head] (float32, one row per distance, the last row for
-// every larger one), added to the scaled score.
+// every larger one), added to the scaled score. With `maps` > 1 a key holds several keys of head_dim features side by
+// side and neighbouring query heads read them in turn: head h reads key h % maps of kv head h / (heads / n_kv), and
+// all of them weigh the same values.
 #include "common.h"
 
 #define ROWS_THREADS 256
@@ -27,7 +29,7 @@ __global__ void attn_rows_kernel(const T* __restrict__ q, const T* __restrict__ 
                                  const int* __restrict__ row_pos, T* __restrict__ out, int n_heads, int n_kv,
                                  int head_dim, int v_dim, float scale, int window, float softcap,
                                  const float* __restrict__ sink, int exact_p, int vec, int chunk,
-                                 const float* __restrict__ rel, int n_dist) {
+                                 const float* __restrict__ rel, int n_dist, int maps) {
   __shared__ float qs[ROWS_MAX_HEAD_DIM];
   __shared__ float ps[ROWS_THREADS];
   __shared__ int pages[ROWS_THREADS / PAGE_TOKENS];
@@ -57,7 +59,7 @@ __global__ void attn_rows_kernel(const T* __restrict__ q, const T* __restrict__ 
     const bool seen = j >= lo && j <= pos && page >= 0;
     float s = -INFINITY;
     if (seen) {
-      const T* kp = k_pages + (((int64_t)page * n_kv + kvh) * PAGE_TOKENS + j % PAGE_TOKENS) * head_dim;
+      const T* kp = k_pages + ((((int64_t)page * n_kv + kvh) * PAGE_TOKENS + j % PAGE_TOKENS) * maps + head % maps) * head_dim;
       float d = 0.f;
       if (vec) {                                           // head_dim % 8 == 0, 16-byte aligned: 8 values a load
         for (int i = 0; i < head_dim; i += 8) {
@@ -127,20 +129,22 @@ __global__ void attn_rows_kernel(const T* __restrict__ q, const T* __restrict__ 
 DRYFT_API int dryft_attn_rows(const void* q, const void* k_pages, const void* v_pages, const int* page_table,
                               int max_pages, const int* row_slot, const int* row_pos, void* out, int n_rows,
                               int n_heads, int n_kv, int head_dim, int v_dim, float scale, int window, float softcap,
-                              const float* sink, int exact_p, int chunk, const float* rel, int n_dist, int is_f32,
+                              const float* sink, int exact_p, int chunk, const float* rel, int n_dist, int maps, int is_f32,
                               hipStream_t stream) {
   if (n_rows <= 0) return 0;
   if (chunk < 0 || (rel != nullptr && n_dist <= 0)) return -1;
-  if (head_dim > ROWS_MAX_HEAD_DIM || v_dim <= 0 || v_dim > ROWS_THREADS || n_kv <= 0 || n_heads % n_kv) return -1;
+  if (head_dim > ROWS_MAX_HEAD_DIM || v_dim <= 0 || v_dim > ROWS_THREADS || n_kv <= 0 || n_heads % n_kv ||
+      maps < 1 || (n_heads / n_kv) % maps)
+    return -1;
   dim3 grid(n_rows, n_heads), block(ROWS_THREADS);
   const int vec = head_dim % 8 == 0 && v_dim % 8 == 0 && (((uintptr_t)k_pages | (uintptr_t)v_pages) & 15) == 0;
   if (is_f32)
     hipLaunchKernelGGL(attn_rows_kernel<float>, grid, block, 0, stream, (const float*)q, (const float*)k_pages,
                        (const float*)v_pages, page_table, max_pages, row_slot, row_pos, (float*)out, n_heads, n_kv,
-                       head_dim, v_dim, scale, window, softcap, sink, exact_p, vec, chunk, rel, n_dist);
+                       head_dim, v_dim, scale, window, softcap, sink, exact_p, vec, chunk, rel, n_dist, maps);
   else
     hipLaunchKernelGGL(attn_rows_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)q, (const bf16_t*)k_pages,
                        (const bf16_t*)v_pages, page_table, max_pages, row_slot, row_pos, (bf16_t*)out, n_heads, n_kv,
-                       head_dim, v_dim, scale, window, softcap, sink, exact_p, vec, chunk, rel, n_dist);
+                       head_dim, v_dim, scale, window, softcap, sink, exact_p, vec, chunk, rel, n_dist, maps);
   return DRYFT_LAUNCH_CHECK();
 }

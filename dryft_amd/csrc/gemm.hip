@@ -576,8 +576,10 @@ __device__ __forceinline__ float silu_for_bf16(float g) {
 // y[n + i] = T(T(silu(gate)) * up), two values in one store where N is even.
 // With `act.limit` > 0 the unit is the clamped one instead: g = min(gate, limit), u = clamp(up, -limit, limit),
 // y = T(g * sigmoid(alpha g) * (u + 1)), from the float accumulators, rounded once.
+// With `act.relu` it is T(max(gate, 0) * up), also from the accumulators and rounded once.
 struct GateAct {
   float limit = 0.f, alpha = 0.f;
+  int relu = 0;
 };
 __device__ __forceinline__ float clamped_unit(float gate, float up, const GateAct& act) {
   const float gc = fminf(gate, act.limit), uc = fminf(fmaxf(up, -act.limit), act.limit);
@@ -592,9 +594,11 @@ __device__ __forceinline__ void swiglu_store4(bf16_t* __restrict__ y_row, int fi
   const float up0 = second ? acc[2] : got0, up1 = second ? acc[3] : got1;
   const int n = first + 4 * (g & 1) + (second ? 2 : 0);
   const bool clamped = act.limit > 0.f;
-  const bf16_t v0 = clamped ? float_to_bf16(clamped_unit(gate0, up0, act))
+  const bf16_t v0 = act.relu ? float_to_bf16(fmaxf(gate0, 0.f) * up0)
+                    : clamped ? float_to_bf16(clamped_unit(gate0, up0, act))
                             : float_to_bf16(rounded_as<bf16_t>(silu_for_bf16(rounded_as<bf16_t>(gate0))) * rounded_as<bf16_t>(up0));
-  const bf16_t v1 = clamped ? float_to_bf16(clamped_unit(gate1, up1, act))
+  const bf16_t v1 = act.relu ? float_to_bf16(fmaxf(gate1, 0.f) * up1)
+                    : clamped ? float_to_bf16(clamped_unit(gate1, up1, act))
                             : float_to_bf16(rounded_as<bf16_t>(silu_for_bf16(rounded_as<bf16_t>(gate1))) * rounded_as<bf16_t>(up1));
   if (!row_there || n >= N) return;
   if (N % 2 == 0) {                                        // then n + 1 < N too, and the address is a multiple of 4
@@ -762,14 +766,17 @@ DRYFT_API int dryft_gemm_panel_waves(int N) {
   return best;
 }
 
-// M <= 64. y[M, N] = T(T(silu(x . Wg^T)) * (x . Wu^T)) with W = [Wg; Wu] of 2N rows; K a multiple of 128; x and W
+// M <= 64. y[M, N] = T(T(silu(x . Wg^T)) * (x . Wu^T)) with W = [Wg; Wu] of 2N rows (relu: T(max(x . Wg^T, 0) *
+// (x . Wu^T))); K a multiple of 128; x and W
 // within reach of 32-bit byte offsets; waves: 4 to 8, or 0 for dryft_gemm_panel_waves' choice.
 static int panel_entry(const void* x, int64_t x_stride, const void* w, void* y, int M, int N, int K, int waves,
                        GateAct act, hipStream_t stream);
 
 DRYFT_API int dryft_gemm_panel_swiglu_bf16(const void* x, int64_t x_stride, const void* w, void* y, int M, int N, int K,
-                                           int waves, hipStream_t stream) {
-  return panel_entry(x, x_stride, w, y, M, N, K, waves, GateAct{}, stream);
+                                           int waves, int relu, hipStream_t stream) {
+  GateAct act;
+  act.relu = relu;
+  return panel_entry(x, x_stride, w, y, M, N, K, waves, act, stream);
 }
 
 // The same product with the clamped gated unit in its epilogue: y = T(g sigmoid(alpha g) (u + 1)),
@@ -995,7 +1002,7 @@ struct TallPlan {
 template <int R, int T, bool SWIGLU>
 __global__ __launch_bounds__(64 * (TALL_WAVES + 1)) void gemm_tall_kernel(
     const bf16_t* __restrict__ x, int64_t x_stride, const bf16_t* __restrict__ w, void* __restrict__ y, int M, int N,
-    int K, int per, int blocks, int splits) {
+    int K, int per, int blocks, int splits, GateAct act) {
   extern __shared__ __align__(16) unsigned char tall_lds[];
   using Plan = TallPlan<R, T>;
   constexpr int WAVES = TALL_WAVES, RB = Plan::RB, W_BYTES = Plan::W_BYTES, X_BYTES = Plan::X_BYTES;
@@ -1115,7 +1122,7 @@ __global__ __launch_bounds__(64 * (TALL_WAVES + 1)) void gemm_tall_kernel(
     if (SWIGLU) {                                          // the gate of output 4g + i of the tile in lanes with g < 2,
       bf16_t* y_row = (bf16_t*)y + (int64_t)min(row, M - 1) * N;                    // its up 32 lanes further on
 #pragma unroll
-      for (int t = 0; t < T; ++t) swiglu_store4(y_row, 8 * (tile0 + t), N, g, acc[m][t], row < M);
+      for (int t = 0; t < T; ++t) swiglu_store4(y_row, 8 * (tile0 + t), N, g, acc[m][t], row < M, act);
     } else if (row < M) {
       float* y_row = (float*)y + ((int64_t)run * M + row) * N;
 #pragma unroll
@@ -1135,7 +1142,7 @@ __global__ __launch_bounds__(64 * (TALL_WAVES + 1)) void gemm_tall_kernel(
 
 template <int R, int T, bool SWIGLU>
 static int launch_tall(const void* x, int64_t x_stride, const void* w, void* y, int M, int N, int K, int splits, int per,
-                       hipStream_t stream) {
+                       hipStream_t stream, GateAct act) {
   constexpr int lds = TallPlan<R, T>::LDS;
   static_assert(lds <= TALL_LDS, "the rings must fit a compute unit's LDS");
   static bool raised = false;                              // more dynamic LDS than the default limit allows
@@ -1147,7 +1154,7 @@ static int launch_tall(const void* x, int64_t x_stride, const void* w, void* y, 
   const int outputs = (SWIGLU ? 8 : 16) * T, blocks = (N + outputs - 1) / outputs;
   dim3 grid(8 * ((blocks * splits + 7) / 8)), block(64 * (TALL_WAVES + 1));
   hipLaunchKernelGGL(kernel, grid, block, lds, stream, (const bf16_t*)x, x_stride, (const bf16_t*)w, y, M, N, K, per, blocks,
-                     splits);
+                     splits, act);
   return DRYFT_LAUNCH_CHECK();
 }
 
@@ -1170,13 +1177,13 @@ DRYFT_API int dryft_gemm_tall_tiles(int N) {
 
 template <int R, bool SWIGLU>
 static int tall_tiles(const void* x, int64_t x_stride, const void* w, void* y, int M, int N, int K, int tiles, int splits,
-                      int per, hipStream_t stream) {
+                      int per, hipStream_t stream, GateAct act = {}) {
   switch (tiles) {
-    case 4: return launch_tall<R, 4, SWIGLU>(x, x_stride, w, y, M, N, K, splits, per, stream);
-    case 5: return launch_tall<R, 5, SWIGLU>(x, x_stride, w, y, M, N, K, splits, per, stream);
-    case 6: return launch_tall<R, 6, SWIGLU>(x, x_stride, w, y, M, N, K, splits, per, stream);
-    case 7: return launch_tall<R, 7, SWIGLU>(x, x_stride, w, y, M, N, K, splits, per, stream);
-    case 8: return launch_tall<R, 8, SWIGLU>(x, x_stride, w, y, M, N, K, splits, per, stream);
+    case 4: return launch_tall<R, 4, SWIGLU>(x, x_stride, w, y, M, N, K, splits, per, stream, act);
+    case 5: return launch_tall<R, 5, SWIGLU>(x, x_stride, w, y, M, N, K, splits, per, stream, act);
+    case 6: return launch_tall<R, 6, SWIGLU>(x, x_stride, w, y, M, N, K, splits, per, stream, act);
+    case 7: return launch_tall<R, 7, SWIGLU>(x, x_stride, w, y, M, N, K, splits, per, stream, act);
+    case 8: return launch_tall<R, 8, SWIGLU>(x, x_stride, w, y, M, N, K, splits, per, stream, act);
     default: return -1;
   }
 }
@@ -1186,16 +1193,19 @@ static bool tall_operands_ok(const void* x, int64_t x_stride, const void* w, int
          w_rows * K * 2 < (int64_t)4 << 30 && (int64_t)M * x_stride * 2 < (int64_t)4 << 30;
 }
 
-// M <= 256. y[M, N] = T(T(silu(x . Wg^T)) * (x . Wu^T)) with W = [Wg; Wu] of 2N rows; K a multiple of 64; x and W
+// M <= 256. y[M, N] = T(T(silu(x . Wg^T)) * (x . Wu^T)) with W = [Wg; Wu] of 2N rows (relu: T(max(x . Wg^T, 0) *
+// (x . Wu^T))); K a multiple of 64; x and W
 // within reach of 32-bit byte offsets; tiles: 4 to 8, or 0 for dryft_gemm_tall_tiles' choice.
 DRYFT_API int dryft_gemm_tall_swiglu_bf16(const void* x, int64_t x_stride, const void* w, void* y, int M, int N, int K,
-                                          int tiles, hipStream_t stream) {
+                                          int tiles, int relu, hipStream_t stream) {
   if (M <= 0 || N <= 0) return 0;
+  GateAct act;
+  act.relu = relu;
   if (!tall_operands_ok(x, x_stride, w, M, (int64_t)2 * N, K)) return -1;
   if (tiles == 0) tiles = dryft_gemm_tall_tiles(N);
   const int groups = K / TALL_GROUP;
-  if (M <= 128) return tall_tiles<1, true>(x, x_stride, w, y, M, N, K, tiles, 1, groups, stream);
-  return tall_tiles<2, true>(x, x_stride, w, y, M, N, K, tiles, 1, groups, stream);
+  if (M <= 128) return tall_tiles<1, true>(x, x_stride, w, y, M, N, K, tiles, 1, groups, stream, act);
+  return tall_tiles<2, true>(x, x_stride, w, y, M, N, K, tiles, 1, groups, stream, act);
 }
 
 // M <= 256. partials[s, M, N] = x . W^T over the s-th of `splits` runs of ceil(K / 64 / splits) groups of K (the last

@@ -30,20 +30,22 @@ __device__ __forceinline__ Best wave_best(Best b) {
 // s / (sum of the chosen s + 1e-20) * scale. One wave a row; lane l holds experts l, l + 64, ...
 // Other forms: `softmax` takes s = softmax(z) over all experts instead of the sigmoid; no correction (null): the
 // choice scores are s itself; `group_best`: a group scores as its single largest choice score; without `renorm`
-// the weights are s * scale as they are.
+// the weights are s * scale as they are. `softmax` = 2: no scores at all; the logits themselves (plus `logit_bias`, if
+// there is one) decide, and the weights are the softmax over the chosen logits alone, times scale.
 template <int PER>
 __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ logits, int64_t stride,
                                                         const float* __restrict__ correction, int n_experts, int groups,
                                                         int keep, int top, float scale, int* __restrict__ chosen,
                                                         float* __restrict__ weights, int rows, int softmax,
-                                                        int group_best, int renorm) {
+                                                        int group_best, int renorm,
+                                                        const float* __restrict__ logit_bias) {
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int64_t row = (int64_t)blockIdx.x * 4 + wave;
   if (row >= rows) return;
   const float NEG = -__builtin_inff();
   float s[PER], c[PER];
   float z_max = NEG, z_sum = 0.f;
-  if (softmax) {
+  if (softmax == 1) {
 #pragma unroll
     for (int j = 0; j < PER; ++j) {
       const int e = lane + WAVE * j;
@@ -64,7 +66,9 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
     const int e = lane + WAVE * j;
     if (!softmax) s[j] = 0.f;
     c[j] = NEG;
-    if (e < n_experts) {
+    if (e < n_experts && softmax == 2) {
+      s[j] = c[j] = logits[row * stride + e] + (logit_bias != nullptr ? logit_bias[e] : 0.f);
+    } else if (e < n_experts) {
       s[j] = softmax ? s[j] / z_sum : 1.f / (1.f + expf(-logits[row * stride + e]));
       c[j] = s[j] + (correction != nullptr ? correction[e] : 0.f);
     }
@@ -106,7 +110,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
       if (e < n_experts && !((kept >> (e / size)) & 1)) c[j] = NEG;
     }
   }
-  float total = 0.f;
+  float total = 0.f, first = 0.f;
   for (int i = 0; i < top; ++i) {
     Best a{NEG, 0x7fffffff};
 #pragma unroll
@@ -120,6 +124,10 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
     for (int j = 0; j < PER; ++j)
       if (lane + WAVE * j == a.i) { sv = s[j]; c[j] = NEG; }
     sv = wave_sum(sv);
+    if (softmax == 2) {                // the first chosen logit is the largest
+      if (i == 0) first = sv;
+      sv = expf(sv - first);
+    }
     total += sv;
     if (lane == 0) {
       chosen[row * top + i] = a.i;
@@ -128,7 +136,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
   }
   if (lane == 0)       // the same lane wrote them
     for (int i = 0; i < top; ++i)
-      weights[row * top + i] = renorm ? weights[row * top + i] / (total + 1e-20f) * scale : weights[row * top + i] * scale;
+      weights[row * top + i] = softmax == 2 ? weights[row * top + i] / total * scale : renorm ? weights[row * top + i] / (total + 1e-20f) * scale : weights[row * top + i] * scale;
 }
 
 DRYFT_API int dryft_moe_max_experts() { return MOE_MAX_EXPERTS; }
@@ -136,14 +144,17 @@ DRYFT_API int dryft_moe_tile() { return MOE_TILE; }
 
 DRYFT_API int dryft_moe_route(const float* logits, int64_t stride, const float* correction, int n_experts, int groups,
                               int keep, int top, float scale, int* chosen, float* weights, int rows, int softmax,
-                              int group_best, int renorm, hipStream_t stream) {
+                              int group_best, int renorm, const float* logit_bias, hipStream_t stream) {
   if (rows <= 0) return 0;
+  if (softmax < 0 || softmax > 2 || (softmax == 2 && correction != nullptr) || (softmax != 2 && logit_bias != nullptr))
+    return -1;
   if (n_experts < 1 || n_experts > MOE_MAX_EXPERTS || top < 1 || top > n_experts || groups < 1 || groups > WAVE ||
       n_experts % groups || keep < 1 || keep > groups || keep * (n_experts / groups) < top)
     return -1;
 #define MOE_ROUTE(PER)                                                                                              \
   hipLaunchKernelGGL(moe_route_kernel<PER>, dim3((rows + 3) / 4), dim3(256), 0, stream, logits, stride, correction,   \
-                     n_experts, groups, keep, top, scale, chosen, weights, rows, softmax, group_best, renorm)
+                     n_experts, groups, keep, top, scale, chosen, weights, rows, softmax, group_best, renorm,  \
+                     logit_bias)
   if (n_experts <= WAVE) MOE_ROUTE(1);
   else if (n_experts <= 2 * WAVE) MOE_ROUTE(2);
   else MOE_ROUTE(MOE_PER_LANE);

@@ -193,7 +193,8 @@ DRYFT_API int dryft_add_rows(const void* a, const void* b, void* out, int64_t n,
 // `form` chooses other norms: bit 0, the branch's norm takes the mean off first (a layer norm without bias:
 // (d - mean) * rsqrt(mean((d - mean)^2) + eps) * wb); bit 1, the same for y; bit 2, y is x_new itself, only rounded
 // (a sublayer that reads the stream as it is). With `groups` > 1 the norm of y is an rms norm taken in that many equal
-// consecutive parts of the row, each divided by its own root mean square.
+// consecutive parts of the row, each divided by its own root mean square. `bias` (float, optional) is added to a y that
+// is normed as one part.
 #define STREAM_NORM_MAX_GROUPS 256
 
 // Sums of squares of a row's parts from its values in LDS, by the block's four waves: parts of a row of fewer than
@@ -225,7 +226,7 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(const void* __restrict
                                                           int wb_f32, const T* __restrict__ extra,
                                                           const void* __restrict__ vec, int vec_f32,
                                                           const void* __restrict__ w, int w_f32,
-                                                          float* __restrict__ x_out, T* __restrict__ y, int width,
+                                                          const float* __restrict__ bias, float* __restrict__ x_out, T* __restrict__ y, int width,
                                                           float eps, int form, int groups) {
   extern __shared__ __attribute__((aligned(16))) float held[];
   __shared__ float scratch[16], sums[STREAM_NORM_MAX_GROUPS];
@@ -281,7 +282,7 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(const void* __restrict
   }
   const float inv = rsqrtf(block_sum(ss, scratch) / (float)width + eps);
   for (int i = threadIdx.x; i < width; i += blockDim.x)
-    store_from_float(y + base + i, (held[i] - mean) * inv * load_vector(w, i, w_f32));
+    store_from_float(y + base + i, (held[i] - mean) * inv * load_vector(w, i, w_f32) + (bias ? bias[i] : 0.f));
 }
 
 // The same for rows whose width is a multiple of 8 with 16-byte aligned operands: a thread owns runs of 8
@@ -294,7 +295,7 @@ __global__ __launch_bounds__(256) void stream_norm_vec_kernel(const void* __rest
                                                               int wb_f32, const T* __restrict__ extra,
                                                               const void* __restrict__ vec, int vec_f32,
                                                               const void* __restrict__ w, int w_f32,
-                                                              float* __restrict__ x_out, T* __restrict__ y, int width,
+                                                              const float* __restrict__ bias, float* __restrict__ x_out, T* __restrict__ y, int width,
                                                               float eps, int form, int groups) {
   extern __shared__ __attribute__((aligned(16))) float held[];
   __shared__ float scratch[16], sums[STREAM_NORM_MAX_GROUPS];
@@ -415,6 +416,12 @@ __global__ __launch_bounds__(256) void stream_norm_vec_kernel(const void* __rest
     if (w_f32) load8_as_float((const float*)w + i, wv); else load8_as_float((const bf16_t*)w + i, wv);
 #pragma unroll
     for (int j = 0; j < 8; ++j) v[j] = (v[j] - mean) * inv * wv[j];
+    if (bias != nullptr) {
+      float bv[8];
+      load8_as_float(bias + i, bv);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] += bv[j];
+    }
     store8_from_float(y + base + i, v);
   }
 }
@@ -425,25 +432,26 @@ __global__ __launch_bounds__(256) void stream_norm_vec_kernel(const void* __rest
 // delta_kind: 0 = none, 1 = activation dtype, 2 = float partial sums.
 DRYFT_API int dryft_stream_norm(const void* x_in, int x_kind, const void* delta, int delta_kind, int n_partials,
                                 int64_t partial_stride, const void* wb, int wb_f32, const void* extra,
-                                const void* vec, int vec_f32, const void* w, int w_f32, float* x_out, void* y,
+                                const void* vec, int vec_f32, const void* w, int w_f32, const float* bias, float* x_out, void* y,
                                 int n_rows, int width, float eps, int is_f32, int form, int groups,
                                 hipStream_t stream) {
   if (n_rows <= 0) return 0;
   if (groups < 1 || groups > STREAM_NORM_MAX_GROUPS || width % groups || (groups > 1 && (form & 2))) return -1;
+  if (bias != nullptr && (groups > 1 || (form & 4))) return -1;
   if (width <= 0 || width > STREAM_NORM_MAX_WIDTH || (y != nullptr && w == nullptr && !(form & 4))) return -1;
   if (delta_kind == 0) n_partials = 0;
   dim3 grid(n_rows), block(256);
   const size_t lds = (size_t)width * sizeof(float);
 #define SN(TT, DD)                                                                                                   \
   hipLaunchKernelGGL((stream_norm_kernel<TT, DD>), grid, block, lds, stream, x_in, x_kind, (const DD*)delta,        \
-                     n_partials, partial_stride, wb, wb_f32, (const TT*)extra, vec, vec_f32, w, w_f32, x_out,       \
+                     n_partials, partial_stride, wb, wb_f32, (const TT*)extra, vec, vec_f32, w, w_f32, bias, x_out, \
                      (TT*)y, width, eps, form, groups)
 #define SNV(TT, DD)                                                                                                  \
   hipLaunchKernelGGL((stream_norm_vec_kernel<TT, DD>), grid, block, lds, stream, x_in, x_kind, (const DD*)delta,    \
-                     n_partials, partial_stride, wb, wb_f32, (const TT*)extra, vec, vec_f32, w, w_f32, x_out,       \
+                     n_partials, partial_stride, wb, wb_f32, (const TT*)extra, vec, vec_f32, w, w_f32, bias, x_out, \
                      (TT*)y, width, eps, form, groups)
   const bool aligned = (((uintptr_t)x_in | (uintptr_t)delta | (uintptr_t)wb | (uintptr_t)extra | (uintptr_t)vec |
-                         (uintptr_t)w | (uintptr_t)x_out | (uintptr_t)y) & 15) == 0 && partial_stride % 4 == 0;
+                         (uintptr_t)w | (uintptr_t)bias | (uintptr_t)x_out | (uintptr_t)y) & 15) == 0 && partial_stride % 4 == 0;
   if (width % 8 == 0 && aligned) {
     if (is_f32) SNV(float, float);
     else if (delta_kind == 2) SNV(bf16_t, float);

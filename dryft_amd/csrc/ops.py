@@ -24,10 +24,12 @@ _SIGNATURES = {
               "dryft_embed_scaled": [_P, _P, _P, _I, _I, _I, _F, _I, _P]},
     "norm": {"dryft_add_rmsnorm": [_P, _P, _I, _I, _L, _P, _I, _P, _P, _I, _I, _F, _I, _P],
              "dryft_add_rows": [_P, _P, _P, _L, _I, _P],
-             "dryft_stream_norm": [_P, _I, _P, _I, _I, _L, _P, _I, _P, _P, _I, _P, _I, _P, _P, _I, _I, _F, _I, _I, _I, _P],
+             "dryft_stream_norm": [_P, _I, _P, _I, _I, _L, _P, _I, _P, _P, _I, _P, _I, _P, _P, _P, _I, _I, _F, _I, _I, _I, _P],
              "dryft_scaled_pair": [_P, _I, _I, _L, _P, _F, _P, _I, _I, _L, _P, _F, _P, _I, _I, _I, _P],
              "dryft_rms_pair_mean": [_P, _I, _I, _L, _P, _P, _P, _I, _I, _L, _P, _P, _P, _I, _I, _F, _I, _P]},
     "activation": {"dryft_silu_mul": [_P, _P, _I, _I, _L, _I, _P],
+                   "dryft_relu_mul": [_P, _P, _I, _I, _L, _I, _P],
+                   "dryft_cap_values": [_P, _L, _F, _P],
                    "dryft_glu_clamped": [_P, _P, _I, _I, _L, _F, _F, _I, _P],
                    "dryft_sigmoid_gate": [_P, _L, _P, _L, _P, _I, _I, _I, _P],
                    "dryft_relu_squared": [_P, _L, _P, _I, _I, _I, _P],
@@ -52,11 +54,18 @@ _SIGNATURES = {
                                         _I, _I, _P],
                 "dryft_norm_rope_half_kv": [_P, _L, _I, _I, _I, _P, _P, _F, _P, _P, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I,
                                             _I, _I, _I, _I, _I, _I, _I, _P],
+                "dryft_rope_maps_kv": [_P, _L, _I, _I, _I, _P, _I, _P, _P, _I, _P, _P, _P, _I, _I, _P, _I, _I, _P, _I, _P, _I,
+                                       _I, _I, _I, _I, _I, _I, _I, _P],
+                "dryft_map_difference": [_P, _P, _L, _I, _F, _F, _F, _I, _P],
                 "dryft_rows_to_cache_takes": [_I, _I, _I, _I],
                 "dryft_rows_to_cache_parts": [_P, _I, _L, _P, _P, _I, _I, _F, _P, _P, _I, _P, _P, _P, _P, _P, _P, _I, _I,
                                               _I, _I, _I, _P]},
-    "attn_rows": {"dryft_attn_rows": [_P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _F, _P, _I, _I, _P, _I, _I, _P]},
-    "attn_mfma": {"dryft_attn_causal_bf16": [_P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _I, _P, _I, _I, _I, _F, _I, _I, _F, _P,
+    "attn_rows": {"dryft_attn_rows": [_P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _F, _P, _I, _I, _P, _I, _I, _I, _P]},
+    "attn_mfma": {"dryft_attn_causal_diff_bf16": [_P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _I, _F,
+                                                  _I, _F, _F, _F, _P],
+                  "dryft_attn_split_diff_bf16": [_P, _P, _P, _P, _I, _P, _P, _P, _I, _P, _P, _I, _P, _I, _I, _I, _I, _F, _I,
+                                                 _F, _F, _F, _P],
+                  "dryft_attn_causal_bf16": [_P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _I, _P, _I, _I, _I, _F, _I, _I, _F, _P,
                                              _I, _P, _I, _P],
                   "dryft_attn_causal_takes_projection": [_I, _I],
                   "dryft_attn_causal_projected_bf16": [_P, _L, _P, _I, _I, _F, _P, _P, _P, _P, _P, _I, _P, _P, _P, _P, _I,
@@ -69,10 +78,10 @@ _SIGNATURES = {
              "dryft_gemm_stream_bf16": [_P, _L, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
              "dryft_gemm_stream_swiglu_bf16": [_P, _L, _P, _P, _I, _I, _I, _I, _I, _P],
              "dryft_gemm_wide_bf16": [_P, _L, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
-             "dryft_gemm_panel_swiglu_bf16": [_P, _L, _P, _P, _I, _I, _I, _I, _P],
+             "dryft_gemm_panel_swiglu_bf16": [_P, _L, _P, _P, _I, _I, _I, _I, _I, _P],
              "dryft_gemm_panel_glu_clamped_bf16": [_P, _L, _P, _P, _I, _I, _I, _I, _F, _F, _P],
              "dryft_gemm_panel_waves": [_I],
-             "dryft_gemm_tall_swiglu_bf16": [_P, _L, _P, _P, _I, _I, _I, _I, _P],
+             "dryft_gemm_tall_swiglu_bf16": [_P, _L, _P, _P, _I, _I, _I, _I, _I, _P],
              "dryft_gemm_tall_bf16": [_P, _L, _P, _P, _I, _I, _I, _I, _I, _P],
              "dryft_gemm_tall_tiles": [_I],
              "dryft_gemm_mid_bf16": [_P, _L, _P, _P, _I, _I, _I, _I, _P],
@@ -82,7 +91,7 @@ _SIGNATURES = {
              "dryft_gemm_wide_swiglu_bf16": [_P, _L, _P, _P, _I, _I, _I, _I, _I, _P],
              "dryft_gemm_narrow_bf16": [_P, _L, _P, _P, _I, _I, _I, _P],
              "dryft_sum_partials": [_P, _P, _L, _I, _I, _P]},
-    "hyper": {"dryft_hyper_norm": [_P, _I, _I, _P, _I, _I, _L, _P, _P, _P, _P, _P, _P, _I, _I, _I, _F, _I, _P]},
+    "hyper": {"dryft_hyper_norm": [_P, _I, _I, _P, _I, _I, _L, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _F, _I, _P]},
     "wkv": {"dryft_wkv_blend": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _P],
             "dryft_wkv_decay": [_P, _P, _P, _P, _I, _I, _I, _I, _P],
             "dryft_log_decay": [_P, _P, _P, _P, _I, _I, _I, _F, _I, _P],
@@ -93,7 +102,7 @@ _SIGNATURES = {
                "dryft_latent_rope_kv": [_P, _P, _P, _L, _I, _P, _P, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I,
                                         _I, _I, _I, _I, _I, _P],
                "dryft_head_gate": [_P, _P, _L, _I, _P, _I, _I, _I, _I, _I, _I, _P]},
-    "moe": {"dryft_moe_route": [_P, _L, _P, _I, _I, _I, _I, _F, _P, _P, _I, _I, _I, _I, _P],
+    "moe": {"dryft_moe_route": [_P, _L, _P, _I, _I, _I, _I, _F, _P, _P, _I, _I, _I, _I, _P, _P],
             "dryft_moe_plan": [_P, _I, _I, _P, _P, _P, _P, _P, _P, _I, _P],
             "dryft_moe_product": [_P, _L, _P, _P, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _F, _F, _F, _I, _I, _I, _P],
             "dryft_moe_table_route": [_P, _P, _P, _P, _I, _I, _I, _I, _P],
@@ -281,7 +290,8 @@ STREAM_NORM_MAX_GROUPS = 256
 
 
 def stream_norm(x, delta, post_weight, extra, vec, weight, eps: float, x_out, y, act: torch.dtype,
-                post_centred: bool = False, centred: bool = False, plain_read: bool = False, groups: int = 1) -> None:
+                post_centred: bool = False, centred: bool = False, plain_read: bool = False, groups: int = 1,
+                bias=None) -> None:
     """The norms of a float32 residual stream in one launch, per row (``post_centred`` / ``centred``: the norm of
     ``d`` / of ``x_out`` takes the mean off first and divides by the standard deviation, a layer norm without bias;
     ``plain_read``: ``y`` is ``x_out`` itself in the activation dtype, no weight):
@@ -289,7 +299,8 @@ def stream_norm(x, delta, post_weight, extra, vec, weight, eps: float, x_out, y,
     ``x_out = x + rmsnorm(d) * post_weight + extra + vec`` (each term optional; without ``post_weight`` ``d`` is added
     as it is); ``y = rmsnorm(x_out) * weight`` in the activation dtype (optional). ``x`` is float32, or in the
     activation dtype ``act`` (a stream that starts), or None; ``x_out`` is float32 (may be ``x`` itself) or None.
-    ``groups`` > 1: the norm of ``y`` is taken in so many equal consecutive parts of the row, each by itself."""
+    ``groups`` > 1: the norm of ``y`` is taken in so many equal consecutive parts of the row, each by itself. ``bias``
+    (float32 ``[width]``): added to ``y`` behind its weight."""
     ref = y if y is not None else (x_out if x_out is not None else x)
     rows, width = ref.shape
     if groups < 1 or groups > STREAM_NORM_MAX_GROUPS or width % groups or (groups > 1 and centred):
@@ -321,6 +332,10 @@ def stream_norm(x, delta, post_weight, extra, vec, weight, eps: float, x_out, y,
             _float_flag(t, name)
             if not (t.shape == (width,) and t.is_contiguous()):
                 raise KernelError(f"stream_norm: {name} must be [{width}]")
+    if bias is not None:
+        _f32_vector(bias, "bias", width)
+        if groups > 1 or plain_read or y is None:
+            raise KernelError("stream_norm: a bias goes with a y that is normed as one part")
     is_f32 = 1 if act == torch.float32 else 0
     if kind == 1 and delta.dtype != act or x_kind == 2 and x.dtype != torch.float32:
         raise KernelError("stream_norm: delta must be in the activation dtype, the stream in it or in float32")
@@ -339,7 +354,7 @@ def stream_norm(x, delta, post_weight, extra, vec, weight, eps: float, x_out, y,
     flag = lambda t: 0 if t is None else _float_flag(t, "vector")      # noqa: E731
     _check(_fn("norm", "dryft_stream_norm")(
         _ptr(x), x_kind, _ptr(delta), kind, n_partials, stride, _ptr(post_weight), flag(post_weight), _ptr(extra),
-        _ptr(vec), flag(vec), _ptr(weight), flag(weight), _ptr(x_out), _ptr(y), rows, width, float(eps), is_f32,
+        _ptr(vec), flag(vec), _ptr(weight), flag(weight), _ptr(bias), _ptr(x_out), _ptr(y), rows, width, float(eps), is_f32,
         (1 if post_centred else 0) | (2 if centred else 0) | (4 if plain_read else 0), int(groups), _stream()), "stream_norm")
 
 
@@ -439,16 +454,35 @@ def blend_columns(a: torch.Tensor, b: torch.Tensor, lam: torch.Tensor) -> torch.
     return a
 
 
+def cap_values(x: torch.Tensor, cap: float) -> torch.Tensor:
+    """``x <- cap * tanh(x / cap)`` in place (float32)."""
+    _gpu(x, "x", torch.float32)
+    if not (x.is_contiguous() and x.data_ptr() % 16 == 0 and cap > 0):
+        raise KernelError("cap_values: x must be contiguous and 16-byte aligned, the cap positive")
+    _check(_fn("activation", "dryft_cap_values")(_ptr(x), x.numel(), float(cap), _stream()), "cap_values")
+    return x
+
+
+def relu_mul(gate_up: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """``out = relu(gate_up[:, :I]) * gate_up[:, I:]``."""
+    return _gate_mul("relu_mul", gate_up, out)
+
+
 def silu_mul(gate_up: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """``out = silu(gate_up[:, :I]) * gate_up[:, I:]``."""
+    return _gate_mul("silu_mul", gate_up, out)
+
+
+def _gate_mul(name: str, gate_up: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
     _gpu(gate_up, "gate_up")
     _gpu(out, "out", gate_up.dtype)
     rows, two_i = gate_up.shape
     if not (two_i % 2 == 0 and out.shape == (rows, two_i // 2)):
-        raise KernelError("silu_mul: out must be [rows, width / 2]")
+        raise KernelError(f"{name}: out must be [rows, width / 2]")
     if not (gate_up.stride(1) == 1 and out.is_contiguous()):
-        raise KernelError("silu_mul: unit stride along the width")
-    _check(_fn("activation", "dryft_silu_mul")(_ptr(gate_up), _ptr(out), rows, two_i // 2, gate_up.stride(0),
-                                               _float_flag(gate_up, "gate_up"), _stream()), "silu_mul")
+        raise KernelError(f"{name}: unit stride along the width")
+    _check(_fn("activation", "dryft_" + name)(_ptr(gate_up), _ptr(out), rows, two_i // 2, gate_up.stride(0),
+                                              _float_flag(gate_up, "gate_up"), _stream()), name)
     return out
 
 
@@ -569,12 +603,14 @@ def _check_pages(k_pages, v_pages, page_table, n_kv: int, head_dim: int, dtype, 
 # --------------------------------------------------------------------------------------- attention
 def attn_rows(q, k_pages, v_pages, page_table, row_slot, row_pos, out, n_heads: int, n_kv: int, head_dim: int,
               scale: float, window: int, *, v_dim: int | None = None, softcap: float = 0.0, sink=None,
-              exact_p: bool = False, chunk: int = 0, rel=None) -> None:
+              exact_p: bool = False, chunk: int = 0, rel=None, maps: int = 1) -> None:
     """``v_dim``: the values' width where it differs from the keys'; ``softcap`` > 0: scores become
     ``cap * tanh(s / cap)``; ``sink``: float32 ``[heads]`` whose exp() joins each head's denominator; ``exact_p``:
     the probabilities weigh the values unrounded; ``chunk`` > 0: a row sees the keys of its own run of so many
     positions instead of a window; ``rel``: float32 ``[distances, heads]``, a bias by distance added to the scaled
-    score (the last row serves every larger distance)."""
+    score (the last row serves every larger distance). ``maps`` > 1: a row of a page of keys holds so many keys of
+    ``head_dim`` features side by side, and query head ``h`` reads key ``h % maps`` of its kv head; the values are one
+    for all maps."""
     _gpu(q, "q")
     is_f32 = _float_flag(q, "q")
     v_dim = head_dim if v_dim is None else int(v_dim)
@@ -584,7 +620,7 @@ def attn_rows(q, k_pages, v_pages, page_table, row_slot, row_pos, out, n_heads: 
     _gpu(out, "out", q.dtype)
     if not (out.is_contiguous() and out.numel() == rows * n_heads * v_dim):
         raise KernelError("attn_rows: out must be [rows, heads, v_dim]")
-    _check_pages(k_pages, v_pages, page_table, n_kv, head_dim, q.dtype, v_dim)
+    _check_pages(k_pages, v_pages, page_table, n_kv, maps * head_dim, q.dtype, v_dim)
     if sink is not None:
         _gpu(sink, "sink", torch.float32)
         if not (sink.is_contiguous() and sink.numel() == n_heads):
@@ -599,8 +635,8 @@ def attn_rows(q, k_pages, v_pages, page_table, row_slot, row_pos, out, n_heads: 
     _check(_fn("attn_rows", "dryft_attn_rows")(
         _ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(page_table), page_table.shape[1], _ptr(row_slot), _ptr(row_pos),
         _ptr(out), rows, n_heads, n_kv, head_dim, v_dim, float(scale), int(window), float(softcap), _ptr(sink),
-        int(bool(exact_p)), int(chunk), _ptr(rel), rel.shape[0] if rel is not None else 0, is_f32, _stream()),
-        "attn_rows")
+        int(bool(exact_p)), int(chunk), _ptr(rel), rel.shape[0] if rel is not None else 0, int(maps), is_f32,
+        _stream()), "attn_rows")
 
 
 def _check_rel(rel, n_heads: int) -> None:
@@ -905,11 +941,15 @@ def gemm_panel_waves(n_outputs: int) -> int:
     return int(_fn("gemm", "dryft_gemm_panel_waves")(int(n_outputs)))
 
 
-def gemm_panel_swiglu_bf16(x, w_gate_up, out, waves: int = 0, clamped: tuple[float, float] | None = None) -> torch.Tensor:
+def gemm_panel_swiglu_bf16(x, w_gate_up, out, waves: int = 0, clamped: tuple[float, float] | None = None,
+                           relu: bool = False) -> torch.Tensor:
     """``silu(x @ Wg.T) * (x @ Wu.T)`` for ``w_gate_up = [Wg; Wu]``, at most 64 rows, by the kernel whose operands go
     from memory straight into LDS. K must be a multiple of 128. ``waves`` (4 to 8, 8 outputs each) per workgroup;
     0 lets the library choose. ``clamped = (limit, alpha)``: the clamped gated unit in the epilogue instead,
-    ``g * sigmoid(alpha * g) * (u + 1)`` with ``g = min(x @ Wg.T, limit)`` and ``u = clamp(x @ Wu.T, -limit, limit)``."""
+    ``g * sigmoid(alpha * g) * (u + 1)`` with ``g = min(x @ Wg.T, limit)`` and ``u = clamp(x @ Wu.T, -limit, limit)``.
+    ``relu``: relu in the place of silu."""
+    if relu and clamped is not None:
+        raise KernelError("gemm_panel_swiglu: relu or the clamped unit, not both")
     _gpu(x, "x", torch.bfloat16)
     _gpu(w_gate_up, "w_gate_up", torch.bfloat16)
     _gpu(out, "out", torch.bfloat16)
@@ -934,7 +974,7 @@ def gemm_panel_swiglu_bf16(x, w_gate_up, out, waves: int = 0, clamped: tuple[flo
             _stream()), "gemm_panel_glu_clamped_bf16")
         return out
     _check(_fn("gemm", "dryft_gemm_panel_swiglu_bf16")(_ptr(x), x.stride(0), _ptr(w_gate_up), _ptr(out), m, two_n // 2, k,
-                                                       int(waves), _stream()), "gemm_panel_swiglu_bf16")
+                                                       int(waves), int(bool(relu)), _stream()), "gemm_panel_swiglu_bf16")
     return out
 
 
@@ -942,10 +982,11 @@ TALL_ROWS = 256     # the most rows gemm_tall_swiglu takes
 TALL_GROUP = 64     # values of K it moves at a time; K must be a multiple of it
 
 
-def gemm_tall_swiglu_bf16(x, w_gate_up, out, tiles: int = 0) -> torch.Tensor:
+def gemm_tall_swiglu_bf16(x, w_gate_up, out, tiles: int = 0, relu: bool = False) -> torch.Tensor:
     """``silu(x @ Wg.T) * (x @ Wu.T)`` for ``w_gate_up = [Wg; Wu]``, at most 256 rows, by the kernel whose waves each own
     rows of x and multiply them with all of the workgroup's rows of W (operands straight into LDS). K must be a multiple
-    of 64. ``tiles`` (4 to 8, 8 outputs each) per workgroup; 0 lets the library choose."""
+    of 64. ``tiles`` (4 to 8, 8 outputs each) per workgroup; 0 lets the library choose. ``relu``: relu in the place of
+    silu."""
     _gpu(x, "x", torch.bfloat16)
     _gpu(w_gate_up, "w_gate_up", torch.bfloat16)
     _gpu(out, "out", torch.bfloat16)
@@ -962,7 +1003,7 @@ def gemm_tall_swiglu_bf16(x, w_gate_up, out, tiles: int = 0) -> torch.Tensor:
     if not (tiles == 0 or 4 <= tiles <= 8):
         raise KernelError("gemm_tall_swiglu: tiles 4 to 8, or 0")
     _check(_fn("gemm", "dryft_gemm_tall_swiglu_bf16")(_ptr(x), x.stride(0), _ptr(w_gate_up), _ptr(out), m, two_n // 2, k,
-                                                      int(tiles), _stream()), "gemm_tall_swiglu_bf16")
+                                                      int(tiles), int(bool(relu)), _stream()), "gemm_tall_swiglu_bf16")
     return out
 
 
@@ -1228,6 +1269,129 @@ def rope_pairs_kv(proj, q_col: int, k_col: int, v_col: int, cos, sin, rot: int, 
         n_heads, n_kv, head_dim, v_dim, is_f32, _stream()), "rope_pairs_kv")
 
 
+# ------------------------------------------------------------------------------------------ two maps a head
+def rope_maps_kv(proj, q_col: int, k_col: int, v_col: int, bias, cos, sin, rot: int, row_slot, row_pos, q_out, q_step: int,
+                 k_pages, map_dim: int, v_pages, page_table, write_kv: bool, n_heads: int, n_kv: int, dim: int,
+                 v_dim: int) -> None:
+    """Queries, keys and values of differential attention from a fused projection (a tensor, or ``(partials, count)``):
+    adds ``bias`` (float32, one number a column of the projection), turns the first ``rot`` features of both maps of
+    every q and k head pair by pair ``(2i, 2i + 1)`` with float32 tables ``[positions, rot / 2]``, writes the queries to
+    ``q_out [rows, heads, 2, q_width]`` (map ``m`` at ``m * q_step``, zeros elsewhere) and, when ``write_kv``, the keys'
+    maps at 0 and ``map_dim`` of their pages' rows and the values to the first ``v_dim`` features of theirs."""
+    data, parts = proj if isinstance(proj, tuple) else (proj, 0)
+    _gpu(data, "proj")
+    if isinstance(proj, tuple):
+        if not (data.dtype == torch.float32 and data.dim() == 3 and data.is_contiguous() and data.shape[0] >= parts >= 1 and
+                q_out.dtype == torch.bfloat16):
+            raise KernelError("rope_maps_kv: partial sums must be contiguous float32 [n, rows, columns], for bfloat16 queries")
+    elif not (data.dim() == 2 and data.stride(1) == 1 and data.dtype == q_out.dtype):
+        raise KernelError("rope_maps_kv: proj must be [rows, columns] with unit column stride in the queries' dtype")
+    rows, columns = data.shape[-2:]
+    is_f32 = _float_flag(q_out, "q_out")
+    ends = (q_col + 2 * n_heads * dim, k_col + 2 * n_kv * dim, v_col + n_kv * v_dim)
+    if min(q_col, k_col, v_col) < 0 or max(ends) > columns:
+        raise KernelError("rope_maps_kv: q, k or v lie outside the projection's columns")
+    if bias is not None:
+        _f32_vector(bias, "bias", columns)
+    if rot % 2 or not 0 <= rot <= dim:
+        raise KernelError(f"rope_maps_kv: the rotated width must be even and at most {dim}, got {rot}")
+    if rot:
+        for name, t in (("cos", cos), ("sin", sin)):
+            _gpu(t, name, torch.float32)
+            if not (t.dim() == 2 and t.shape[1] == rot // 2 and t.is_contiguous()):
+                raise KernelError(f"{name}: must be contiguous float32 [positions, {rot // 2}]")
+    _gpu(q_out, "q_out")
+    if not (q_out.dim() == 4 and q_out.shape[:3] == (rows, n_heads, 2) and q_out.is_contiguous() and
+            0 <= q_step and q_step + dim <= q_out.shape[3]):
+        raise KernelError("rope_maps_kv: q_out must be contiguous [rows, heads, 2, width] with room for both maps")
+    page_dim, v_page = k_pages.shape[3], v_pages.shape[2]
+    _check_pages(k_pages, v_pages, page_table, n_kv, page_dim, q_out.dtype, v_page)
+    if k_pages.shape[2] != 64 or v_pages.shape[3] != 64 or map_dim < dim or map_dim + dim > page_dim or v_page < v_dim:
+        raise KernelError("rope_maps_kv: pages too narrow for the maps or the values")
+    for name, t in (("row_slot", row_slot), ("row_pos", row_pos)):
+        _gpu(t, name, torch.int32)
+        if not (t.numel() >= rows):
+            raise KernelError(f"{name}: needs {rows} entries")
+    _check(_fn("rope_kv", "dryft_rope_maps_kv")(
+        _ptr(data), data.stride(-2), q_col, k_col, v_col, _ptr(bias), parts, _ptr(cos), _ptr(sin), rot, _ptr(row_slot),
+        _ptr(row_pos), _ptr(q_out), q_out.shape[3], int(q_step), _ptr(k_pages), page_dim, int(map_dim), _ptr(v_pages), v_page,
+        _ptr(page_table), page_table.shape[1], int(bool(write_kv)), rows, n_heads, n_kv, dim, v_dim, is_f32, _stream()),
+        "rope_maps_kv")
+
+
+def map_difference(a, out, v_dim: int, lam: float, post: float, eps: float) -> torch.Tensor:
+    """``a [rows, heads, 2, v_dim]``: ``out = o / sqrt(mean(o^2) + eps) * post`` with ``o = a1 - lam * a2``."""
+    _gpu(a, "a")
+    _gpu(out, "out", a.dtype)
+    if not (a.is_contiguous() and out.is_contiguous() and a.numel() == 2 * out.numel() and out.numel() % v_dim == 0 and
+            0 < v_dim <= 256):
+        raise KernelError("map_difference: a [rows, heads, 2, v_dim] and out [rows, heads, v_dim], contiguous, v_dim at most 256")
+    _check(_fn("rope_kv", "dryft_map_difference")(_ptr(a), _ptr(out), out.numel() // v_dim, v_dim, float(lam), float(post),
+                                                  float(eps), _float_flag(a, "a"), _stream()), "map_difference")
+    return out
+
+
+def attn_causal_diff_bf16(q, k_pages, v_pages, page_table, seq_slot, cu_rows, tile_cu, seq_start, n_seqs: int,
+                          max_tiles: int, out, n_heads: int, n_kv: int, map_dim: int, v_dim: int, scale: float,
+                          window: int, lam: float, post: float, eps: float) -> None:
+    """Differential attention of steps with many rows per sequence, on the matrix cores. ``q [rows, heads, 2, map_dim]``;
+    pages of keys and of values of one width (a multiple of 16), a key's maps at 0 and ``map_dim`` (a multiple of 8) of
+    its row, a value's ``v_dim`` features first; ``out [rows, heads, v_dim]`` receives the maps' difference, normed."""
+    page_dim = _diff_operands("attn_causal_diff", q, k_pages, v_pages, page_table, out, n_heads, n_kv, map_dim, v_dim, map_dim)
+    for name, t, n in (("seq_slot", seq_slot, n_seqs), ("cu_rows", cu_rows, n_seqs + 1),
+                       ("tile_cu", tile_cu, n_seqs + 1), ("seq_start", seq_start, n_seqs)):
+        _gpu(t, name, torch.int32)
+        if not (t.numel() >= n):
+            raise KernelError(f"{name}: needs {n} entries")
+    _check(_fn("attn_mfma", "dryft_attn_causal_diff_bf16")(
+        _ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(page_table), page_table.shape[1], _ptr(seq_slot), _ptr(cu_rows),
+        _ptr(tile_cu), _ptr(seq_start), n_seqs, max_tiles, _ptr(out), 2 * n_heads, n_kv, page_dim, map_dim, v_dim,
+        float(scale), int(window), float(lam), float(post), float(eps), _stream()), "attn_causal_diff_bf16")
+
+
+def attn_split_diff_bf16(q, k_pages, v_pages, page_table, seq_slot, cu_rows, kv_len, n_seqs: int, part_o, part_ml,
+                         n_splits: int, out, n_heads: int, n_kv: int, map_dim: int, v_dim: int, scale: float, window: int,
+                         lam: float, post: float, eps: float) -> None:
+    """The same for steps of one row per sequence; ``q [rows, heads, 2, page width]`` holds map ``m`` at ``m * map_dim`` and
+    zeros elsewhere."""
+    page_dim = _diff_operands("attn_split_diff", q, k_pages, v_pages, page_table, out, n_heads, n_kv, map_dim, v_dim,
+                              k_pages.shape[3])
+    for name, t, n in (("seq_slot", seq_slot, n_seqs), ("cu_rows", cu_rows, n_seqs + 1), ("kv_len", kv_len, n_seqs)):
+        _gpu(t, name, torch.int32)
+        if not (t.numel() >= n):
+            raise KernelError(f"{name}: needs {n} entries")
+    _gpu(part_o, "part_o", torch.float32)
+    _gpu(part_ml, "part_ml", torch.float32)
+    entries = n_seqs * 2 * n_heads * n_splits
+    if part_o.numel() < entries * page_dim or part_ml.numel() < entries * 2:
+        raise KernelError("attn_split_diff: partial buffers too small")
+    if not (n_splits <= 65535 and n_kv * ((2 * n_heads // n_kv + 15) // 16) <= 65535):
+        raise KernelError("attn_split_diff: grid too large")
+    _check(_fn("attn_mfma", "dryft_attn_split_diff_bf16")(
+        _ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(page_table), page_table.shape[1], _ptr(seq_slot), _ptr(cu_rows),
+        _ptr(kv_len), n_seqs, _ptr(part_o), _ptr(part_ml), n_splits, _ptr(out), 2 * n_heads, n_kv, page_dim, v_dim,
+        float(scale), int(window), float(lam), float(post), float(eps), _stream()), "attn_split_diff_bf16")
+
+
+def _diff_operands(who: str, q, k_pages, v_pages, page_table, out, n_heads: int, n_kv: int, map_dim: int, v_dim: int,
+                   q_width: int) -> int:
+    _gpu(q, "q", torch.bfloat16)
+    _gpu(out, "out", torch.bfloat16)
+    page_dim = k_pages.shape[3]
+    _check_pages(k_pages, v_pages, page_table, n_kv, page_dim, torch.bfloat16)
+    rows = q.shape[0]
+    if not (q.shape == (rows, n_heads, 2, q_width) and q.is_contiguous()):
+        raise KernelError(f"{who}: q must be contiguous [rows, {n_heads}, 2, {q_width}]")
+    if not (out.is_contiguous() and out.numel() == rows * n_heads * v_dim):
+        raise KernelError(f"{who}: out must be contiguous [rows, {n_heads}, {v_dim}]")
+    if not (n_kv > 0 and n_heads % n_kv == 0 and map_dim > 0 and map_dim % 8 == 0 and 2 * map_dim <= page_dim and
+            0 < v_dim <= page_dim and page_dim % 16 == 0 and page_dim <= 256 and n_heads <= 32767):
+        raise KernelError(f"{who}: sizes the matrix-core kernels do not take")
+    if (q.data_ptr() | k_pages.data_ptr() | v_pages.data_ptr() | out.data_ptr()) & 15:
+        raise KernelError(f"{who}: operands must be 16-byte aligned")
+    return page_dim
+
+
 # ------------------------------------------------------------------------------------------ recurrent mixers
 def _f32_vector(t, name: str, n: int) -> None:
     _gpu(t, name, torch.float32)
@@ -1453,14 +1617,16 @@ def rglru_scan_tiles(coef, proj, x_col: int, y_col: int, x_bias, y_bias, taps: i
 HYPER_MAX_STREAMS = 8
 
 
-def hyper_norm(x, n: int, delta, mix, write, read, weight, eps: float, x_out, y, *, normed: bool, act=None) -> None:
+def hyper_norm(x, n: int, delta, mix, write, read, weight, eps: float, x_out, y, *, normed: bool, act=None,
+               centred: bool = False, bias=None) -> None:
     """One launch for a residual stream of ``n`` copies: ``x'_t = sum_s mix[s, t] x_s + write[t] * delta`` (skipped
     without ``delta``), written to ``x_out [n, rows, width]`` (float32, may be ``x``; None: not kept);
     ``u = sum_t read[t] x'_t`` (``read`` None: the plain sum); ``y = rmsnorm(u) * weight`` in the activation dtype
     when ``normed``, else ``y = u`` in float32. ``x`` is the copies in float32 or one ``[rows, width]`` tensor in the
     activation dtype that every copy equals; ``delta`` a tensor in the activation dtype or ``(partials, count)``
     (partial sums are rounded to the activation dtype once added up, as the product itself would have stored them;
-    ``act`` names that dtype where no operand shows it)."""
+    ``act`` names that dtype where no operand shows it). ``centred``: the norm of ``u`` takes its mean off first (a
+    layer norm); ``bias`` (float32 ``[width]``) is added behind its weight."""
     _gpu(x, "x")
     rows, width = x.shape[-2:]
     copies = x.dim() == 3
@@ -1509,9 +1675,11 @@ def hyper_norm(x, n: int, delta, mix, write, read, weight, eps: float, x_out, y,
             raise KernelError("hyper_norm: y must be contiguous [rows, width]")
         if normed:
             _f32_vector(weight, "weight", width)
+            if bias is not None:
+                _f32_vector(bias, "bias", width)
     _check(_fn("hyper", "dryft_hyper_norm")(
         _ptr(x), int(copies), n, _ptr(delta), kind, n_partials, stride, _ptr(mix), _ptr(write), _ptr(read), _ptr(weight),
-        _ptr(x_out), _ptr(y), int(bool(normed)), rows, width, float(eps), 1 if act == torch.float32 else 0, _stream()),
+        _ptr(bias), _ptr(x_out), _ptr(y), int(bool(normed)), int(bool(centred)), rows, width, float(eps), 1 if act == torch.float32 else 0, _stream()),
         "hyper_norm")
 
 
@@ -1735,12 +1903,19 @@ MOE_TILE = 64
 
 
 def moe_route(logits, correction, n_experts: int, groups: int, keep: int, scale: float, chosen, weights, *,
-              softmax: bool = False, group_best: bool = False, renorm: bool = True) -> None:
+              softmax: bool = False, group_best: bool = False, renorm: bool = True, chosen_softmax: bool = False,
+              logit_bias=None) -> None:
     """Per row of float32 ``logits`` (their first ``n_experts`` columns): the ``top`` experts by ``sigmoid + correction``
     among the ``keep`` best of ``groups`` groups (a group's score: its two largest such scores), and their weights
     ``sigmoid / (sum of the chosen sigmoids + 1e-20) * scale``. ``chosen`` int32 and ``weights`` float32 ``[rows, top]``.
     ``softmax``: scores are the softmax over all experts instead; ``correction`` None: none; ``group_best``: a group
-    scores as its best expert; ``renorm`` off: the weights are the scores times ``scale`` as they are."""
+    scores as its best expert; ``renorm`` off: the weights are the scores times ``scale`` as they are.
+    ``chosen_softmax``: the logits plus ``logit_bias`` (float32 ``[experts]``, optional) decide, and the weights are the
+    softmax over the chosen ones alone, times ``scale``."""
+    if chosen_softmax and (softmax or correction is not None) or (logit_bias is not None and not chosen_softmax):
+        raise KernelError("moe_route: chosen_softmax goes alone, and a bias on the logits only with it")
+    if logit_bias is not None:
+        _f32_vector(logit_bias, "logit_bias", n_experts)
     _gpu(logits, "logits", torch.float32)
     rows, top = chosen.shape
     if not (logits.dim() == 2 and logits.shape[0] == rows and logits.stride(1) == 1 and logits.shape[1] >= n_experts):
@@ -1755,8 +1930,9 @@ def moe_route(logits, correction, n_experts: int, groups: int, keep: int, scale:
             keep * (n_experts // groups) >= top):
         raise KernelError("moe_route: sizes the router does not take")
     _check(_fn("moe", "dryft_moe_route")(_ptr(logits), logits.stride(0), _ptr(correction), n_experts, groups, keep, top,
-                                         float(scale), _ptr(chosen), _ptr(weights), rows, int(bool(softmax)),
-                                         int(bool(group_best)), int(bool(renorm)), _stream()), "moe_route")
+                                         float(scale), _ptr(chosen), _ptr(weights), rows,
+                                         2 if chosen_softmax else int(bool(softmax)), int(bool(group_best)),
+                                         int(bool(renorm)), _ptr(logit_bias), _stream()), "moe_route")
 
 
 class MoePlan:

@@ -269,7 +269,8 @@ __device__ __forceinline__ void qk_norm_rope_row(int64_t row, const T* __restric
 // LDS. Where 32 consecutive rows are one aligned block of 32 positions of one page (the usual case in a long
 // prompt), a thread writes 8 columns of a feature's row with one 16-byte store: they are two runs of four
 // consecutive positions (see value_column). Otherwise values go one by one. (The per-row kernel above writes a
-// row's values 128 bytes apart.) head_dim must be a multiple of 8.
+// row's values 128 bytes apart.) head_dim must be a multiple of 8. `bias` (float, the values' own columns) is added
+// first; `page_dim` > head_dim: pages hold so many features, those behind head_dim are not written.
 #define V_TILE_ROWS 64
 #define V_TILE_LD (V_TILE_ROWS + 8)
 extern __shared__ __attribute__((aligned(16))) unsigned char v_tile_raw[];
@@ -279,7 +280,8 @@ __device__ __forceinline__ void v_tile_write(int tile_index, int kvh, const T* _
                                              int v_col0, const int* __restrict__ row_slot,
                                              const int* __restrict__ row_pos, T* __restrict__ v_pages,
                                              const int* __restrict__ page_table, int max_pages, int n_rows, int n_kv,
-                                             int head_dim, int parts, int64_t part_stride) {
+                                             int head_dim, int parts, int64_t part_stride,
+                                             const float* __restrict__ bias = nullptr, int page_dim = 0) {
   __shared__ int64_t base[V_TILE_ROWS];                     // start of the row's page for this kv head, or -1
   __shared__ int in_page[V_TILE_ROWS];                      // the row's position within its page
   __shared__ int block_ok[V_TILE_ROWS / 32];
@@ -291,6 +293,10 @@ __device__ __forceinline__ void v_tile_write(int tile_index, int kvh, const T* _
     const int t = e / chunks, ch = e % chunks;
     float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
     if (t < rows) load8_projected(qkv, (int64_t)(r0 + t) * qkv_stride + v_col0 + kvh * head_dim + 8 * ch, parts, part_stride, v);
+    if (bias != nullptr) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] += bias[kvh * head_dim + 8 * ch + j];
+    }
 #pragma unroll
     for (int j = 0; j < 8; ++j) store_from_float(tile + (8 * ch + j) * V_TILE_LD + t, v[j]);
   }
@@ -301,7 +307,7 @@ __device__ __forceinline__ void v_tile_write(int tile_index, int kvh, const T* _
       const int slot = row_slot[r0 + threadIdx.x], pos = row_pos[r0 + threadIdx.x];
       if (slot >= 0) {
         const int page = page_of(page_table, max_pages, slot, pos);
-        if (page >= 0) where = ((int64_t)page * n_kv + kvh) * head_dim * PAGE_TOKENS;
+        if (page >= 0) where = ((int64_t)page * n_kv + kvh) * (page_dim > 0 ? page_dim : head_dim) * PAGE_TOKENS;
         at = pos % PAGE_TOKENS;
       }
     }
@@ -776,5 +782,262 @@ DRYFT_API int dryft_norm_rope_half_kv(const void* src, int64_t src_stride, int q
   else
     hipLaunchKernelGGL(v_tile_write_kernel<bf16_t>, vgrid, dim3(256), v_lds, stream, (const bf16_t*)src, src_stride,
                        v_col, row_slot, row_pos, (bf16_t*)v_pages, page_table, max_pages, n_rows, n_kv, v_dim);
+  return DRYFT_LAUNCH_CHECK();
+}
+
+// ---------------------------------------------------------------------------------------------------
+// Queries and keys of two maps per head (differential attention), turned over neighbouring pairs with float tables
+// and brought to the paged cache together with the values that both maps weigh. The projection holds, behind q_col,
+// k_col and v_col, the query heads [n_heads][2][dim], the keys [n_kv][2][dim] and the values [n_kv][v_dim]; `bias`
+// (float, one number a column of the projection, or null) is added first. Of the first `rot` features of every map,
+// 2i and 2i + 1 turn together (as above), in float, rounded once.
+//
+//   q_out  [rows][n_heads][2][q_width]   map m's features at m * q_step, zeros elsewhere
+//   pages of keys    [.., 64, page_dim]  a row: map 1 at 0, map 2 at map_dim; what lies between and behind is not
+//                                        written (it holds the zeros it started with)
+//   pages of values  [.., v_page, 64]    the first v_dim features
+//
+// The projection may also be `parts` float partial sums (bfloat16 activations), added up and rounded on the way in.
+struct MapLayout {
+  int n_heads, n_kv, dim, v_dim, rot;
+  int q_width, q_step, page_dim, map_dim, v_page;
+};
+
+__device__ __forceinline__ float projected_at(const float* p, int64_t at, int parts, int64_t part_stride) { return p[at]; }
+__device__ __forceinline__ float projected_at(const bf16_t* p, int64_t at, int parts, int64_t part_stride) {
+  if (parts == 0) return bf16_to_float(p[at]);
+  const float* f = (const float*)p + at;
+  float v = f[0];
+  for (int s = 1; s < parts; ++s) v += f[s * part_stride];
+  return rounded_as<bf16_t>(v);
+}
+
+// Any sizes: a wave takes one map of a query head, one map of a key, or one head of values.
+template <typename T>
+__global__ __launch_bounds__(256) void rope_maps_kernel(const T* __restrict__ proj, int64_t stride, int q_col, int k_col,
+                                                        int v_col, const float* __restrict__ bias, int parts,
+                                                        int64_t part_stride, const float* __restrict__ cos_t,
+                                                        const float* __restrict__ sin_t, const int* __restrict__ row_slot,
+                                                        const int* __restrict__ row_pos, T* __restrict__ q_out,
+                                                        T* __restrict__ k_pages, T* __restrict__ v_pages,
+                                                        const int* __restrict__ page_table, int max_pages, int write_kv,
+                                                        int skip_v, MapLayout m) {
+  const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
+  const int64_t row = blockIdx.x;
+  const int job = blockIdx.y * 4 + wave, q_jobs = 2 * m.n_heads, k_jobs = 2 * m.n_kv;
+  if (job >= q_jobs + k_jobs + (skip_v ? 0 : m.n_kv)) return;
+  const int slot = row_slot[row], pos = row_pos[row];
+  const bool is_q = job < q_jobs, is_k = !is_q && job < q_jobs + k_jobs;
+  if (is_q) {
+    T* dst = q_out + (row * q_jobs + job) * m.q_width;
+    const int first = (job & 1) * m.q_step;
+    for (int i = lane; i < m.q_width; i += WAVE)
+      if (slot < 0 || i < first || i >= first + m.dim) store_from_float(dst + i, 0.f);
+    if (slot < 0) return;
+  } else if (slot < 0 || !write_kv) {
+    return;
+  }
+  int page = 0;
+  const int in_page = pos % PAGE_TOKENS;
+  if (!is_q) {
+    page = page_of(page_table, max_pages, slot, pos);
+    if (page < 0) return;  // no page: the host reserves one before the step; never write through a bad index
+  }
+  const int64_t row_at = row * stride;
+  if (!is_q && !is_k) {
+    const int kvh = job - q_jobs - k_jobs, col = v_col + kvh * m.v_dim;
+    T* dst = v_pages + ((int64_t)page * m.n_kv + kvh) * m.v_page * PAGE_TOKENS + value_column(in_page);
+    for (int i = lane; i < m.v_dim; i += WAVE)
+      store_from_float(dst + (int64_t)i * PAGE_TOKENS,
+                       projected_at(proj, row_at + col + i, parts, part_stride) + (bias ? bias[col + i] : 0.f));
+    return;
+  }
+  const int kj = job - q_jobs;
+  const int col = is_q ? q_col + job * m.dim : k_col + kj * m.dim;
+  T* dst = is_q ? q_out + (row * q_jobs + job) * m.q_width + (job & 1) * m.q_step
+                : k_pages + (((int64_t)page * m.n_kv + kj / 2) * PAGE_TOKENS + in_page) * m.page_dim + (kj & 1) * m.map_dim;
+  const int half = m.rot / 2;
+  for (int i = lane; i < half; i += WAVE) {
+    const float c = cos_t[(int64_t)pos * half + i], s = sin_t[(int64_t)pos * half + i];
+    const float a = projected_at(proj, row_at + col + 2 * i, parts, part_stride) + (bias ? bias[col + 2 * i] : 0.f);
+    const float b = projected_at(proj, row_at + col + 2 * i + 1, parts, part_stride) + (bias ? bias[col + 2 * i + 1] : 0.f);
+    store_from_float(dst + 2 * i, a * c - b * s);
+    store_from_float(dst + 2 * i + 1, b * c + a * s);
+  }
+  for (int i = m.rot + lane; i < m.dim; i += WAVE)
+    store_from_float(dst + i, projected_at(proj, row_at + col + i, parts, part_stride) + (bias ? bias[col + i] : 0.f));
+}
+
+// Sizes in steps of 8 (dim, v_dim, widths, columns; 16-byte aligned operands): a thread takes 8 neighbouring features
+// of a query, a key or a value. Values go to their pages one by one here (few rows) or through the tile kernel.
+template <typename T>
+__global__ __launch_bounds__(256) void rope_maps_vec_kernel(const T* __restrict__ proj, int64_t stride, int q_col,
+                                                            int k_col, int v_col, const float* __restrict__ bias,
+                                                            int parts, int64_t part_stride,
+                                                            const float* __restrict__ cos_t,
+                                                            const float* __restrict__ sin_t,
+                                                            const int* __restrict__ row_slot,
+                                                            const int* __restrict__ row_pos, T* __restrict__ q_out,
+                                                            T* __restrict__ k_pages, T* __restrict__ v_pages,
+                                                            const int* __restrict__ page_table, int max_pages,
+                                                            int write_kv, int skip_v, MapLayout m) {
+  const int64_t row = blockIdx.x;
+  const int q_pieces = m.q_width / 8, d_pieces = m.dim / 8, v_pieces = m.v_dim / 8;
+  const int q_lanes = 2 * m.n_heads * q_pieces, k_lanes = 2 * m.n_kv * d_pieces;
+  int at = blockIdx.y * blockDim.x + threadIdx.x;
+  if (at >= q_lanes + (write_kv ? k_lanes + (skip_v ? 0 : m.n_kv * v_pieces) : 0)) return;
+  const int slot = row_slot[row], pos = row_pos[row];
+  float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+  T* dst;
+  int col, part;                                              // first column of the map; the thread's piece of it
+  bool is_v = false;
+  if (at < q_lanes) {
+    const int job = at / q_pieces, piece = at % q_pieces;
+    dst = q_out + (row * 2 * m.n_heads + job) * m.q_width + 8 * piece;
+    part = piece - (job & 1) * (m.q_step / 8);
+    if (slot < 0 || part < 0 || part >= d_pieces) {
+      store8_from_float(dst, v);
+      return;
+    }
+    col = q_col + job * m.dim;
+  } else {
+    if (slot < 0) return;
+    const int page = page_of(page_table, max_pages, slot, pos), in_page = pos % PAGE_TOKENS;
+    if (page < 0) return;
+    at -= q_lanes;
+    if (at < k_lanes) {
+      const int job = at / d_pieces;
+      part = at % d_pieces;
+      col = k_col + job * m.dim;
+      dst = k_pages + (((int64_t)page * m.n_kv + job / 2) * PAGE_TOKENS + in_page) * m.page_dim + (job & 1) * m.map_dim + 8 * part;
+    } else {
+      at -= k_lanes;
+      const int kvh = at / v_pieces;
+      part = at % v_pieces;
+      col = v_col + kvh * m.v_dim;
+      dst = v_pages + (((int64_t)page * m.n_kv + kvh) * m.v_page + 8 * part) * PAGE_TOKENS + value_column(in_page);
+      is_v = true;
+    }
+  }
+  col += 8 * part;
+  load8_projected(proj, row * stride + col, parts, part_stride, v);
+  if (bias != nullptr) {
+    float b[8];
+    load8_as_float(bias + col, b);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] += b[j];
+  }
+  if (is_v) {
+#pragma unroll
+    for (int j = 0; j < 8; ++j) store_from_float(dst + (int64_t)j * PAGE_TOKENS, v[j]);
+    return;
+  }
+  const int half = m.rot / 2;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int i = 4 * part + j;
+    if (i < half) {
+      const float c = cos_t[(int64_t)pos * half + i], s = sin_t[(int64_t)pos * half + i];
+      const float a = v[2 * j], b = v[2 * j + 1];
+      v[2 * j] = a * c - b * s;
+      v[2 * j + 1] = b * c + a * s;
+    }
+  }
+  store8_from_float(dst, v);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void v_tile_biased_kernel(const T* __restrict__ proj, int64_t stride, int v_col,
+                                                            const float* __restrict__ bias, int parts,
+                                                            int64_t part_stride, const int* __restrict__ row_slot,
+                                                            const int* __restrict__ row_pos, T* __restrict__ v_pages,
+                                                            const int* __restrict__ page_table, int max_pages, int n_rows,
+                                                            int n_kv, int v_dim, int v_page) {
+  v_tile_write<T>(blockIdx.x, blockIdx.y, proj, stride, v_col, row_slot, row_pos, v_pages, page_table, max_pages, n_rows,
+                  n_kv, v_dim, parts, part_stride, bias ? bias + v_col : nullptr, v_page);
+}
+
+DRYFT_API int dryft_rope_maps_kv(const void* proj, int64_t stride, int q_col, int k_col, int v_col, const float* bias,
+                                 int parts, const float* cos_t, const float* sin_t, int rot, const int* row_slot,
+                                 const int* row_pos, void* q_out, int q_width, int q_step, void* k_pages, int page_dim,
+                                 int map_dim, void* v_pages, int v_page, const int* page_table, int max_pages,
+                                 int write_kv, int n_rows, int n_heads, int n_kv, int dim, int v_dim, int is_f32,
+                                 hipStream_t stream) {
+  if (n_rows <= 0) return 0;
+  if (n_heads <= 0 || n_kv <= 0 || dim <= 0 || v_dim <= 0 || rot < 0 || rot % 2 || rot > dim || q_out == nullptr ||
+      q_step < 0 || q_step + dim > q_width || map_dim < dim || map_dim + dim > page_dim || v_page < v_dim || parts < 0 ||
+      (parts > 0 && is_f32))
+    return -1;
+  const MapLayout m = {n_heads, n_kv, dim, v_dim, rot, q_width, q_step, page_dim, map_dim, v_page};
+  const int64_t part_stride = (int64_t)n_rows * stride;
+  const uintptr_t all = (uintptr_t)proj | (uintptr_t)bias | (uintptr_t)q_out | (uintptr_t)k_pages | (uintptr_t)v_pages;
+  const bool by8 = ((dim | v_dim | q_width | q_step | page_dim | map_dim | q_col | k_col | v_col) % 8) == 0 &&
+                   stride % 8 == 0 && (all & 15) == 0;
+  const size_t v_lds = (size_t)v_dim * V_TILE_LD * (is_f32 ? 4 : 2);
+  const int skip_v = (write_kv && n_rows >= 32 && by8 && v_lds <= 64 * 1024) ? 1 : 0;
+#define ROPE_MAPS(KERNEL, TT, GRID)                                                                                  \
+  hipLaunchKernelGGL(KERNEL<TT>, GRID, dim3(256), 0, stream, (const TT*)proj, stride, q_col, k_col, v_col, bias, parts, \
+                     part_stride, cos_t, sin_t, row_slot, row_pos, (TT*)q_out, (TT*)k_pages, (TT*)v_pages, page_table, \
+                     max_pages, write_kv, skip_v, m)
+  if (by8) {
+    const int lanes = 2 * n_heads * (q_width / 8) + (write_kv ? 2 * n_kv * (dim / 8) + (skip_v ? 0 : n_kv * (v_dim / 8)) : 0);
+    const dim3 grid(n_rows, (lanes + 255) / 256);
+    if (is_f32) ROPE_MAPS(rope_maps_vec_kernel, float, grid);
+    else ROPE_MAPS(rope_maps_vec_kernel, bf16_t, grid);
+  } else {
+    const dim3 grid(n_rows, (2 * n_heads + 3 * n_kv + 3) / 4);
+    if (is_f32) ROPE_MAPS(rope_maps_kernel, float, grid);
+    else ROPE_MAPS(rope_maps_kernel, bf16_t, grid);
+  }
+#undef ROPE_MAPS
+  int rc = DRYFT_LAUNCH_CHECK();
+  if (rc || !skip_v) return rc;
+  const dim3 vgrid((n_rows + V_TILE_ROWS - 1) / V_TILE_ROWS, n_kv);
+#define V_BIASED(TT)                                                                                                 \
+  hipLaunchKernelGGL(v_tile_biased_kernel<TT>, vgrid, dim3(256), v_lds, stream, (const TT*)proj, stride, v_col, bias,  \
+                     parts, part_stride, row_slot, row_pos, (TT*)v_pages, page_table, max_pages, n_rows, n_kv, v_dim, v_page)
+  if (is_f32) V_BIASED(float);
+  else V_BIASED(bf16_t);
+#undef V_BIASED
+  return DRYFT_LAUNCH_CHECK();
+}
+
+// ---------------------------------------------------------------------------------------------------
+// The two maps' outputs a [rows][heads][2][v_dim] of attention kernels that keep them apart:
+// out[row][head] = o / sqrt(mean(o^2) + eps) * post with o = a1 - lambda * a2, in float, rounded once. A wave a head.
+template <typename T>
+__global__ __launch_bounds__(256) void map_difference_kernel(const T* __restrict__ a, T* __restrict__ out, int64_t n,
+                                                             int v_dim, float lambda, float post, float eps) {
+  const int64_t at = (int64_t)blockIdx.x * 4 + threadIdx.x / WAVE;
+  const int lane = threadIdx.x % WAVE;
+  if (at >= n) return;
+  const T* a1 = a + at * 2 * v_dim;
+  const T* a2 = a1 + v_dim;
+  float o[4], ss = 0.f;                                       // v_dim <= 256
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    const int i = lane + WAVE * k;
+    o[k] = i < v_dim ? load_as_float(a1 + i) - lambda * load_as_float(a2 + i) : 0.f;
+    ss += o[k] * o[k];
+  }
+  const float r = post / sqrtf(wave_sum(ss) / (float)v_dim + eps);
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    const int i = lane + WAVE * k;
+    if (i < v_dim) store_from_float(out + at * v_dim + i, o[k] * r);
+  }
+}
+
+DRYFT_API int dryft_map_difference(const void* a, void* out, int64_t n, int v_dim, float lambda, float post, float eps,
+                                   int is_f32, hipStream_t stream) {
+  if (n <= 0) return 0;
+  if (v_dim <= 0 || v_dim > 4 * WAVE) return -1;
+  const dim3 grid((unsigned)((n + 3) / 4)), block(256);
+  if (is_f32)
+    hipLaunchKernelGGL(map_difference_kernel<float>, grid, block, 0, stream, (const float*)a, (float*)out, n, v_dim, lambda,
+                       post, eps);
+  else
+    hipLaunchKernelGGL(map_difference_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)a, (bf16_t*)out, n, v_dim,
+                       lambda, post, eps);
   return DRYFT_LAUNCH_CHECK();
 }

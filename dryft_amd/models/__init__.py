@@ -79,3 +79,4 @@ from . import fetedra as _fetedra  # noqa: E402,F401  (registers Fetedra)
 from . import barilix as _barilix  # noqa: E402,F401  (registers Barilix)
 from . import podenex as _podenex  # noqa: E402,F401  (registers Podenex)
 from . import fubinex as _fubinex  # noqa: E402,F401  (registers Fubinex)
+from . import kaditar as _kaditar  # noqa: E402,F401  (registers Kaditar)

@@ -16,6 +16,7 @@ Checkpoint names: ``embed``, ``final.norm``, ``loop.step``, and per layer ``l<i>
 
 from __future__ import annotations
 
+from ..config.base import layer_order
 from ..config.piralix import PiralixConfig
 from ..config.plan import LayerSpec, ModelPlan, PartSpec, Run
 from . import register_architecture
@@ -76,19 +77,11 @@ def piralix_plan(cfg: PiralixConfig) -> ModelPlan:
         layers.append(LayerSpec("sandwich", parts))
     # the schedule: layers before the loop, the looped run once per pass (each pass with cache lines of its own,
     # its first run entering through the pass entry), the layers after it
-    n = len(cfg.layers)
-    order: list[tuple[int, tuple[str, int] | None]] = []
     stream_parts = {}
-    if cfg.loop is None:
-        order = [(i, None) for i in range(n)]
-    else:
-        lp = cfg.loop
-        stream_parts["loop"] = PartSpec("pass_entry", dict(passes=lp.times, size=cfg.width), {"steps": "loop.step"})
-        order += [(i, None) for i in range(lp.start)]
-        for t in range(lp.times):
-            order += [(i, ("loop", t) if i == lp.start else None) for i in range(lp.start, lp.stop)]
-        order += [(i, None) for i in range(lp.stop, n)]
-    schedule = tuple(Run(layer, line, True, enter) for line, (layer, enter) in enumerate(order))
+    if cfg.loop is not None:
+        stream_parts["loop"] = PartSpec("pass_entry", dict(passes=cfg.loop.times, size=cfg.width), {"steps": "loop.step"})
+    schedule = tuple(Run(layer, line, True, ("loop", t) if t is not None else None)
+                     for line, (layer, t) in enumerate(layer_order(len(cfg.layers), cfg.loop)))
     return ModelPlan(
         vocab_size=cfg.vocab,
         hidden_size=cfg.width,

@@ -68,6 +68,29 @@ def add_bias(delta, bias: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
     return out
 
 
+def keys_seen(spans: list[tuple[int, int]], window: int | None, chunk: int | None = None) -> int:
+    """The keys that the rows of a step see together; ``spans`` holds ``(start, q)`` per sequence."""
+    seen = 0
+    for start, q in spans:
+        first, last = start + 1, start + q                  # keys that the span's first and last row see
+        if window:
+            full = max(0, min(last, window) - first + 1)               # rows that still see every key
+            seen += (2 * first + full - 1) * full // 2 + (q - full) * window
+        elif chunk:
+            seen += sum(p % chunk + 1 for p in range(start, start + q))
+        else:
+            seen += (first + last) * q // 2
+    return seen
+
+
+def key_splits(n_seqs: int, blocks: int, span: int) -> int:
+    """How many ways each sequence's keys are split in decoding (``blocks`` workgroups a sequence and split, ``span`` keys
+    at most): as many as run at the same time, and no more. Workgroups beyond what the chip holds at once start when
+    the first ones end, which costs more than the longer walk of fewer, larger splits."""
+    pages = max(1, (span + 63) // 64)
+    return max(1, min(_RESIDENT_WORKGROUPS // (n_seqs * blocks), _MAX_SPLITS, pages))
+
+
 def distance_row(n: int, rows: int, far: int) -> int:
     """The row of a bias table that distance ``n`` reads: its own below half the table, then
     ``half + floor(log(n / half) / log(far / half) * (rows - half))``, at most the last."""
@@ -402,29 +425,12 @@ class GQAAttention(Mixer):
 
     def flops(self, rows, spans):
         """The projections, and both attention products over the keys each row sees."""
-        seen = 0
-        for start, q in spans:
-            first, last = start + 1, start + q                  # keys that the span's first and last row see
-            if self.window:
-                full = max(0, min(last, self.window) - first + 1)          # rows that still see every key
-                seen += (2 * first + full - 1) * full // 2 + (q - full) * self.window
-            elif self.chunk:
-                seen += sum(p % self.chunk + 1 for p in range(start, start + q))
-            else:
-                seen += (first + last) * q // 2
+        seen = keys_seen(spans, self.window, self.chunk)
         return super().flops(rows, spans) + 2.0 * (self.q_dim + self.o_dim) * seen
 
     def decode_splits(self, n_seqs: int, max_kv_len: int) -> int:
-        """How many ways each sequence's keys are split: as many as run at the same time, and no more.
-
-        Workgroups beyond what the chip holds at once start when the first ones end, which costs more than
-        the longer walk of fewer, larger splits.
-        """
         blocks = self.n_kv * ((self.n_heads // self.n_kv + 15) // 16)
-        want = _RESIDENT_WORKGROUPS // (n_seqs * blocks)
-        span = self.window or getattr(self, "chunk", None) or max_kv_len
-        pages = max(1, (span + 63) // 64)
-        return max(1, min(want, _MAX_SPLITS, pages))
+        return key_splits(n_seqs, blocks, self.window or getattr(self, "chunk", None) or max_kv_len)
 
 
 register_part("gqa_attention", GQAAttention)

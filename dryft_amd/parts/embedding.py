@@ -2,7 +2,7 @@
 
 Embedding: a row gather without scaling (reference: engine/dryft_qwen3/model.py:132); with ``scale`` the rows are
 multiplied by it and come out as float32, the start of a float32 residual stream.
-Head: ``logits = h @ W.T`` as float32. A tied head is a plan that gives the head the
+Head: ``logits = h @ W.T`` as float32, with ``softcap`` ``logits <- cap * tanh(logits / cap)``. A tied head is a plan that gives the head the
 embedding's tensor name (weights.py:47-49): both parts then hold the same tensor. The reference keeps bfloat16 logits (model.py:186, 261); here the
 float accumulators are stored directly.
 """
@@ -44,8 +44,9 @@ class TokenEmbedding(Part):
 
 
 class LMHead(Part):
-    def __init__(self, vocab_size: int, hidden_size: int):
+    def __init__(self, vocab_size: int, hidden_size: int, softcap: float | None = None):
         self.vocab, self.hidden = int(vocab_size), int(hidden_size)
+        self.softcap = float(softcap) if softcap else None
         self.weight: torch.Tensor | None = None
 
     def tensor_specs(self):
@@ -55,10 +56,11 @@ class LMHead(Part):
         self.weight = tensors["weight"]
 
     def kernel_modules(self, dtype):
-        return ("gemm",)
+        return ("gemm",) + (("activation",) if self.softcap else ())
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
-        return linear(h, self.weight, out_dtype=torch.float32)
+        logits = linear(h, self.weight, out_dtype=torch.float32)
+        return ops.cap_values(logits, self.softcap) if self.softcap else logits
 
 
 register_part("token_embedding", TokenEmbedding)

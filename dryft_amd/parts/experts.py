@@ -10,12 +10,15 @@ shared expert, of the same form with sizes of its own, runs for every row and is
 
 Other forms, by constructor arguments. ``router="table"``: no scores at all; an integer table ``[vocab, top]`` (the
 entries of a row differ) names each token id's experts, every one with weight ``1 / top`` (the step's token ids come
-with the step context). ``unit="silu"``: an expert is ``down(silu(gate(h)) * up(h))``, nothing clamped, and so is
-the shared expert, which is then added as it is.
+with the step context), and the shared expert is added as it is. ``unit="silu"``: an expert is ``down(silu(gate(h)) *
+up(h))``, nothing clamped, and so is the shared expert.
 
 ``score="softmax"``: the scores are the softmax of ``z`` over all experts; ``correction=False``: no correction, the
 scores themselves decide; ``group_score="best"``: a group scores as its best expert; ``renormalize=False``: the weights
 are the chosen scores times ``route_scale`` as they are; ``shared_gate=False``: the shared expert is added as it is.
+``score="chosen_softmax"``: the logits themselves decide, with ``logit_bias`` after one learned number per expert has been
+added to them (tensor ``router_bias``), and the weights are the softmax over the chosen logits alone times
+``route_scale``.
 ``unit="relu2"``: an expert has no gate, ``down(relu(up(h))^2)``, and so has the shared expert.
 
 On the device throughout, so a step can be captured: the router picks, a small kernel sorts the (row, expert) pairs
@@ -40,14 +43,19 @@ class RoutedExperts(FeedForward):
                  route_scale: float = 1.0, groups: tuple[int, int] | None = None,
                  shared: tuple | None = None, alpha: float = 1.702, router: str = "scores", unit: str = "clamped",
                  vocab_size: int | None = None, score: str = "sigmoid", correction: bool = True,
-                 group_score: str = "top2", renormalize: bool = True, shared_gate: bool = True):
+                 group_score: str = "top2", renormalize: bool = True, shared_gate: bool = True,
+                 logit_bias: bool = False):
         self.hidden, self.n_experts, self.top, self.inter = int(hidden_size), int(experts), int(top), int(intermediate_size)
         if router not in ("scores", "table") or unit not in ("clamped", "silu", "relu2"):
             raise ValueError(f"router is 'scores' or 'table', unit 'clamped', 'silu' or 'relu2'; got {router!r}, {unit!r}")
-        if score not in ("sigmoid", "softmax") or group_score not in ("top2", "best"):
-            raise ValueError(f"score is 'sigmoid' or 'softmax', group_score 'top2' or 'best'; got {score!r}, {group_score!r}")
+        if score not in ("sigmoid", "softmax", "chosen_softmax") or group_score not in ("top2", "best"):
+            raise ValueError(f"score is 'sigmoid', 'softmax' or 'chosen_softmax', group_score 'top2' or 'best'; got {score!r}, {group_score!r}")
         self.score, self.has_correction, self.group_score = score, bool(correction), group_score
         self.renormalize, self.shared_gate = bool(renormalize), bool(shared_gate) and router == "scores"
+        self.has_logit_bias = bool(logit_bias)
+        if score == "chosen_softmax" and (correction or groups) or (logit_bias and score != "chosen_softmax"):
+            raise ValueError("scores of the chosen logits alone go without a correction and groups, and only they take a "
+                             "bias on the logits")
         self.gated = unit != "relu2"
         if router == "table" and not vocab_size:
             raise ValueError("a table router needs the vocabulary's size")
@@ -67,7 +75,7 @@ class RoutedExperts(FeedForward):
         if shared:
             self.shared = ClampedGLU(hidden_size, shared[0], shared[1], alpha) if unit == "clamped" else \
                 SwiGLU(hidden_size, shared[0]) if unit == "silu" else SquaredReLU(hidden_size, shared[0])
-        self.w_router = self.correction = self.w_gate_up = self.w_down = self.table = None
+        self.w_router = self.correction = self.router_bias = self.w_gate_up = self.w_down = self.table = None
 
     def tensor_specs(self):
         if self.router == "table":
@@ -76,6 +84,8 @@ class RoutedExperts(FeedForward):
             specs = {"router": matrix((self.n_experts, self.hidden))}
             if self.has_correction:
                 specs["correction"] = ((self.n_experts,), VECTOR, "zeros")
+            if self.has_logit_bias:
+                specs["router_bias"] = ((self.n_experts,), VECTOR, "zeros")
         for e in range(self.n_experts):
             if self.gated:
                 specs[f"e{e}_gate"] = matrix((self.inter, self.hidden))
@@ -104,6 +114,8 @@ class RoutedExperts(FeedForward):
             return
         if self.has_correction:
             self.correction = tensors["correction"].float().contiguous()
+        if self.has_logit_bias:
+            self.router_bias = tensors["router_bias"].float().contiguous()
         router = [tensors["router"]]
         if self.shared is not None and self.shared_gate:
             router.append(tensors["shared_weight"])
@@ -124,7 +136,8 @@ class RoutedExperts(FeedForward):
             logits = linear(h, self.w_router, out_dtype=torch.float32)
             ops.moe_route(logits, self.correction, E, self.groups[0], self.groups[1], self.route_scale, chosen, weights,
                           softmax=self.score == "softmax", group_best=self.group_score == "best",
-                          renorm=self.renormalize)
+                          renorm=self.renormalize, chosen_softmax=self.score == "chosen_softmax",
+                          logit_bias=self.router_bias)
         plan = ops.moe_plan(chosen, E)
         act = torch.empty((rows * top, self.inter), dtype=h.dtype, device=dev)
         if self.gated:

@@ -56,7 +56,7 @@ def read_streams(x: torch.Tensor, pending: Deferred, route: StreamRoute | None, 
     """``(copies, h)``: the copies after ``pending`` has entered them (float32 ``[n, rows, width]``; updated in place
     where ``x`` already is such a tensor, None when not kept), and ``h = norm(sum_s read[s] x_s)`` in ``act``
     (``route`` None: the plain sum). ``x`` may still be the embedding's output ``[rows, width]``, which every copy
-    equals."""
+    equals. The norm may be a layer norm, with or without a bias."""
     if pending.norm is not None or pending.rows is not None or pending.vector is not None:
         raise ValueError("a stream of several copies takes a sublayer's output and nothing else")
     n = copies or (route.streams if route is not None else _copies(x, pending))
@@ -71,7 +71,8 @@ def read_streams(x: torch.Tensor, pending: Deferred, route: StreamRoute | None, 
         delta = (delta.data, delta.count)
     taken = pending.route
     ops.hyper_norm(x, n, delta, taken.mix if taken else None, taken.write if taken else None,
-                   route.read if route is not None else None, norm.weight, norm.eps, out, h, normed=True)
+                   route.read if route is not None else None, norm.weight, norm.eps, out, h, normed=True,
+                   centred=norm.centred, bias=norm.bias)
     return out, h
 
 

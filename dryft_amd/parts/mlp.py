@@ -16,6 +16,8 @@ from .linear import STREAM_ROWS, few_rows_ok, linear, panel_swiglu_ok, tall_swig
 
 
 class SwiGLU(FeedForward):
+    relu = False              # relu in the place of silu (``ReGLU``)
+
     def __init__(self, hidden_size: int, intermediate_size: int):
         self.hidden, self.inter = int(hidden_size), int(intermediate_size)
         self.w_gate_up: torch.Tensor | None = None
@@ -35,14 +37,22 @@ class SwiGLU(FeedForward):
     def forward(self, h, ctx):
         act = torch.empty((h.shape[0], self.inter), dtype=h.dtype, device=h.device)
         if h.dtype == torch.bfloat16 and panel_swiglu_ok(h, self.w_gate_up):
-            ops.gemm_panel_swiglu_bf16(h, self.w_gate_up, act)        # product and activation in one kernel
+            ops.gemm_panel_swiglu_bf16(h, self.w_gate_up, act, relu=self.relu)        # product and activation in one kernel
         elif h.dtype == torch.bfloat16 and tall_swiglu_ok(h, self.w_gate_up):
-            ops.gemm_tall_swiglu_bf16(h, self.w_gate_up, act)         # the same at 65 to 256 rows
+            ops.gemm_tall_swiglu_bf16(h, self.w_gate_up, act, relu=self.relu)         # the same at 65 to 256 rows
+        elif self.relu:
+            ops.relu_mul(linear(h, self.w_gate_up), act)
         elif h.dtype == torch.bfloat16 and h.shape[0] <= STREAM_ROWS and few_rows_ok(h, self.w_gate_up):
             ops.gemm_stream_swiglu_bf16(h, self.w_gate_up, act)       # the same for any K that is a multiple of 8
         else:
             ops.silu_mul(linear(h, self.w_gate_up), act)
         return linear(act, self.w_down, allow_partials=True)
+
+
+class ReGLU(SwiGLU):
+    """``down( relu(gate(h)) * up(h) )``, dense, no bias."""
+
+    relu = True
 
 
 class ClampedGLU(FeedForward):
@@ -127,6 +137,7 @@ class PolyNormMLP(FeedForward):
 
 
 register_part("swiglu", SwiGLU)
+register_part("reglu", ReGLU)
 register_part("poly_norm_mlp", PolyNormMLP)
 register_part("squared_relu", SquaredReLU)
 register_part("clamped_glu", ClampedGLU)

@@ -8,7 +8,7 @@ unadded (``Deferred``), and the next block's first kernel norms it, adds it, add
 due meanwhile, and norms the stream for its own first branch, in one launch.
 
 ``StreamRMSNorm``    the norm itself: ``x / sqrt(mean(x^2) + eps) * w`` in float, rounded once.
-``StreamLayerNorm``  the same with the mean taken off first: ``(x - mean) / sqrt(var + eps) * w``, no bias.
+``StreamLayerNorm``  the same with the mean taken off first: ``(x - mean) / sqrt(var + eps) * w``, and ``+ b`` if it has one.
 ``SandwichBlock``    mixer and feed-forward, each between two norms; ``SandwichMixerBlock`` has the mixer alone.
 ``PostNormBlock``    ``x <- x + norm(branch(x))``: the branches read the stream as it is, only their outputs are
                      normed; ``PostNormMixerBlock`` has the mixer alone.
@@ -37,6 +37,7 @@ class StreamRMSNorm(Norm):
     parts of the vector, each divided by its own root mean square. A stream of several copies ``[copies, rows, width]``
     (``parts/hyper.py``) is normed as the sum of its copies."""
 
+    bias: torch.Tensor | None = None      # added behind the weight, where the norm has one
     centred = False           # does the norm take the mean off first (a layer norm without bias)?
 
     def __init__(self, size: int, eps: float, offset: float = 0.0, scale: float = 1.0, groups: int = 1):
@@ -60,7 +61,7 @@ class StreamRMSNorm(Norm):
             return self.add_forward(x, None, dtype)[1]
         y = torch.empty(x.shape, dtype=dtype or self.compute_dtype or x.dtype, device=x.device)
         ops.stream_norm(x, None, None, None, None, self.weight, self.eps, None, y, y.dtype, centred=self.centred,
-                        groups=self.groups)
+                        groups=self.groups, bias=self.bias)
         return y
 
     def add_forward(self, res: torch.Tensor, delta, dtype: torch.dtype | None = None, in_place: bool = True):
@@ -77,14 +78,30 @@ class StreamRMSNorm(Norm):
         own = in_place and res.dtype == torch.float32 and res.is_contiguous()
         out = res if own else torch.empty(res.shape, dtype=torch.float32, device=res.device)
         y = torch.empty(res.shape, dtype=act, device=res.device)
-        _launch(res, pending, self.weight, self.eps, out, y, act, centred=self.centred, groups=self.groups)
+        _launch(res, pending, self.weight, self.eps, out, y, act, centred=self.centred, groups=self.groups, bias=self.bias)
         return out, y
 
 
 class StreamLayerNorm(StreamRMSNorm):
-    """``(x - mean(x)) / sqrt(mean((x - mean(x))^2) + eps) * w`` in float, without a bias."""
+    """``(x - mean(x)) / sqrt(mean((x - mean(x))^2) + eps) * w`` in float; with ``bias`` (tensor ``bias``) ``+ b``. A norm
+    with a bias stands in front of a reader."""
 
     centred = True
+
+    def __init__(self, size: int, eps: float, offset: float = 0.0, scale: float = 1.0, bias: bool = False):
+        super().__init__(size, eps, offset, scale)
+        self.has_bias = bool(bias)
+
+    def tensor_specs(self):
+        specs = super().tensor_specs()
+        if self.has_bias:
+            specs["bias"] = ((self.size,), VECTOR, "zeros")
+        return specs
+
+    def load(self, tensors):
+        super().load(tensors)
+        if self.has_bias:
+            self.bias = (tensors["bias"].float() * self.scale).contiguous()
 
 
 def as_deferred(pending) -> Deferred:
@@ -103,18 +120,20 @@ def _activation_dtype(x: torch.Tensor, pending: Deferred) -> torch.dtype:
 
 
 def _launch(x, pending: Deferred, weight, eps, x_out, y, act, centred: bool = False, plain_read: bool = False,
-            groups: int = 1) -> None:
+            groups: int = 1, bias=None) -> None:
     delta = pending.delta
     if isinstance(delta, Partials):
         delta = (delta.data, delta.count)
     post = pending.norm.weight if pending.norm is not None else None
+    if getattr(pending.norm, "bias", None) is not None:
+        raise NotImplementedError("a norm with a bias stands in front of a reader, not behind a sublayer")
     if getattr(pending.norm, "groups", 1) > 1:
         raise NotImplementedError("a norm in parts stands in front of a reader, not behind a sublayer")
     if pending.norm is not None and pending.norm.eps != eps:
         raise ValueError("the norms around one residual sum differ in eps; one launch takes one")
     ops.stream_norm(x, delta, post, pending.rows, pending.vector, weight, eps, x_out, y, act,
                     post_centred=bool(getattr(pending.norm, "centred", False)), centred=centred, plain_read=plain_read,
-                    groups=groups)
+                    groups=groups, bias=bias)
 
 
 def read_plain(x: torch.Tensor, pending, act: torch.dtype):
