@@ -137,7 +137,8 @@ def compare_fetedra(args, design: str = "fetedra", relative: str = "piralix") ->
     float32 stream, as many layers of the same widths), ``--design podenex`` for Podenex beside it (three kinds of
     windowed or chunked attention, one of them Fetedra's latent kind, with routed experts on a float32 stream),
     ``--design fubinex`` for Fubinex beside Barilix (attention and a recurrence side by side, and a second recurrent
-    kind, on a float32 stream)."""
+    kind, on a float32 stream), ``--design kaditar`` for Kaditar beside Fetedra (windowed attention and routed experts with
+    a gated shared one on several copies of a float32 stream, as many runs of layers of the same widths)."""
     import torch
 
     from dryft_amd import Engine
@@ -149,6 +150,8 @@ def compare_fetedra(args, design: str = "fetedra", relative: str = "piralix") ->
         kw = dict(seed=args.seed, dtype="bfloat16", max_batch=args.batch, max_len=args.prompt_len + 2 * (args.steps + args.warmup) + 64,
                   use_graph=not args.no_graph)
         entry = {"preset": name, "width": raw["width"], "layers": len(raw["layers"])}
+        if raw.get("loop"):
+            entry["layer_runs"] = len(raw["layers"]) + (raw["loop"]["times"] - 1) * (raw["loop"]["stop"] - raw["loop"]["start"])
         for key, cfg in ((design, raw), (relative, load_preset(f"{relative}-w{raw['width']}"))):
             engine = Engine(config=cfg, **kw)
             entry[key] = measure(engine, args.prompt_len, args.batch, args.steps, args.warmup, args.seed)
@@ -165,10 +168,10 @@ def compare_fetedra(args, design: str = "fetedra", relative: str = "piralix") ->
 def main() -> int:
     global PROMPT, SLOT
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", default=None, choices=["piralix", "fetedra", "barilix", "podenex", "fubinex"],
+    ap.add_argument("--design", default=None, choices=["piralix", "fetedra", "barilix", "podenex", "fubinex", "kaditar"],
                     help="instead of the default workload: that design beside its closest relative in the library at "
-                         "equal size (Piralix beside Qwen3, Fetedra beside Piralix, Barilix and Podenex beside Fetedra, Fubinex beside "
-                         "Barilix; one JSON line)")
+                         "equal size (Piralix beside Qwen3, Fetedra beside Piralix, Barilix, Podenex and Kaditar beside Fetedra, "
+                         "Fubinex beside Barilix; one JSON line)")
     ap.add_argument("--sizes", default=None, help="presets for --design (default: the design's presets)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=128)
@@ -194,8 +197,9 @@ def main() -> int:
                                     "fetedra": "fetedra-w1024,fetedra-w2048",
                                     "barilix": "barilix-w1024,barilix-w2048",
                                     "podenex": "podenex-w1024,podenex-w2048",
-                                    "fubinex": "fubinex-w1024,fubinex-w2048"}[args.design]
-        if args.design in ("barilix", "podenex"):
+                                    "fubinex": "fubinex-w1024,fubinex-w2048",
+                                    "kaditar": "kaditar-w1024,kaditar-w2048"}[args.design]
+        if args.design in ("barilix", "podenex", "kaditar"):
             return compare_fetedra(args, args.design, "fetedra")
         if args.design == "fubinex":
             return compare_fetedra(args, "fubinex", "barilix")
