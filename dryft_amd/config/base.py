@@ -93,7 +93,7 @@ class KeyReader:
 
 @dataclass(frozen=True)
 class LoopConfig:
-    """Layers ``start`` .. ``stop - 1`` run ``times`` times in a row with the same weights."""
+    """A run of layers, ``start`` inclusive to ``stop`` exclusive, that is gone through ``times`` times over one set of weights."""
 
     start: int
     stop: int

@@ -2,8 +2,8 @@
 
 A Kaditar ``config.json`` is nested: ``vocab``, ``width``, ``streams`` (copies of the residual stream that the layers
 read from and write to through learned weights), ``norm.eps``, optionally ``logit_softcap``, optionally ``loop``
-(``start``, ``stop``, ``times``: layers ``start`` .. ``stop - 1`` run ``times`` times in a row with the same weights), and a
-list ``layers`` whose entries each name a mixer ``type`` with that mixer's sizes under ``mixer`` and a feed-forward
+(``start``, ``stop``, ``times``: the layers from ``start`` up to ``stop``, not included, are gone through ``times`` times),
+and a list ``layers`` whose entries each name a mixer ``type`` with that mixer's sizes under ``mixer`` and a feed-forward
 under ``mlp`` (or null):
 
 * ``attention``: ``heads``, ``kv_heads``, ``dim`` (one map's query and key), ``vdim``, ``scale``, ``diff``; optionally

@@ -402,6 +402,44 @@ struct MapPair {
   float lambda, post, eps;
 };
 
+// The end of both prompt kernels' forms for two maps: `a` and `b` hold the maps' unnormalised outputs of the lane's row,
+// l1 and l2 the row's sums; all lanes of the wave must call it. `o` is the row's place in the output.
+template <int KB>
+__device__ __forceinline__ void store_difference(RowBlock<KB>& a, const RowBlock<KB>& b, float l1, float l2, bool row_valid,
+                                                 bf16_t* __restrict__ o, const MapPair& pair) {
+  const int g = (threadIdx.x % WAVE) / 16;
+  const float w1 = row_valid ? 1.f / l1 : 0.f, w2 = row_valid ? pair.lambda / l2 : 0.f;
+  float ss = 0.f;
+#pragma unroll
+  for (int dt = 0; dt < 2 * KB; ++dt)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float d = a.o[dt][i] * w1 - b.o[dt][i] * w2;
+      a.o[dt][i] = d;
+      ss += 16 * dt + 4 * g + i < pair.v_dim ? d * d : 0.f;
+    }
+  ss += __shfl_xor(ss, 16, WAVE);                             // the four lanes that share a row
+  ss += __shfl_xor(ss, 32, WAVE);
+  const float r = pair.post / sqrtf(ss / (float)pair.v_dim + pair.eps);
+  if (!row_valid) return;
+#pragma unroll
+  for (int dt = 0; dt < 2 * KB; ++dt) {
+    const int d0 = 16 * dt + 4 * g;
+    if (pair.v_dim % 4 == 0) {                                // then the address is a multiple of 8 bytes
+      if (d0 < pair.v_dim) {
+        bf16x4 v;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = to_bf16(a.o[dt][i] * r);
+        *(bf16x4*)(o + d0) = v;
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (d0 + i < pair.v_dim) o[d0 + i] = float_to_bf16(a.o[dt][i] * r);
+    }
+  }
+}
+
 // DIFF: the wave's two units are the two maps of one head (GP = 2), each with keys of its own.
 template <int KB, bool FULL, int GP, int RP, bool DIFF>
 __global__ __launch_bounds__(256, (GP * RP * KB <= 8 && KB <= 4) ? (GP * RP == 1 ? 3 : 2) : 1) void attn_causal_kernel(
@@ -576,38 +614,8 @@ __global__ __launch_bounds__(256, (GP * RP * KB <= 8 && KB <= 4) ? (GP * RP == 1
         for (int u = 0; u < U; ++u) row_l[u] += sink_term(opt.sink, head0 + u, st[u].m);
       }
     }
-    const float w1 = row_valid[0] ? 1.f / row_l[0] : 0.f, w2 = row_valid[0] ? pair.lambda / row_l[U - 1] : 0.f;
-    float ss = 0.f;
-#pragma unroll
-    for (int dt = 0; dt < 2 * KB; ++dt)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const float o = st[0].o[dt][i] * w1 - st[U - 1].o[dt][i] * w2;
-        st[0].o[dt][i] = o;
-        ss += 16 * dt + 4 * g + i < pair.v_dim ? o * o : 0.f;
-      }
-    ss += __shfl_xor(ss, 16, WAVE);                           // the four lanes that share a row
-    ss += __shfl_xor(ss, 32, WAVE);
-    const float r = pair.post / sqrtf(ss / (float)pair.v_dim + pair.eps);
-    if (row_valid[0]) {
-      bf16_t* o = out + (row[0] * (n_heads / 2) + head0 / 2) * pair.v_dim;
-#pragma unroll
-      for (int dt = 0; dt < 2 * KB; ++dt) {
-        const int d0 = 16 * dt + 4 * g;
-        if (pair.v_dim % 4 == 0) {                            // then the address is a multiple of 8 bytes
-          if (d0 < pair.v_dim) {
-            bf16x4 v;
-#pragma unroll
-            for (int i = 0; i < 4; ++i) v[i] = to_bf16(st[0].o[dt][i] * r);
-            *(bf16x4*)(o + d0) = v;
-          }
-        } else {
-#pragma unroll
-          for (int i = 0; i < 4; ++i)
-            if (d0 + i < pair.v_dim) o[d0 + i] = float_to_bf16(st[0].o[dt][i] * r);
-        }
-      }
-    }
+    store_difference<KB>(st[0], st[U - 1], row_l[0], row_l[U - 1], row_valid[0],
+                         out + (row[0] * (n_heads / 2) + head0 / 2) * pair.v_dim, pair);
     continue;
   }
 #pragma unroll
@@ -755,18 +763,22 @@ __device__ __forceinline__ void init_rows_projected(RowBlock<4>& st, const Proje
 // the same at 2,048). With 32 rows a wave the registers allow two workgroups a unit anyway, so both have two
 // buffers and a page takes one barrier.
 // EXTRA: the form that also knows chunks and a sink (a build of its own, so that the plain form keeps its registers).
-template <int RP, bool EXTRA>
-__global__ __launch_bounds__(256, RP == 1 ? 4 : 2) void attn_causal_direct_kernel(
+// DIFF: two maps a head (MapPair above) of 64 features each; a wave's two units are the maps of its 16 rows, every piece
+// of the values read from LDS serves both, and grid x counts output heads. Two buffers, as with 32 rows a wave.
+template <int RP, bool EXTRA, bool DIFF = false>
+__global__ __launch_bounds__(256, RP == 1 && !DIFF ? 4 : 2) void attn_causal_direct_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages,
     const int* __restrict__ page_table, int max_pages, const int* __restrict__ seq_slot,
     const int* __restrict__ cu_rows, const int* __restrict__ tile_cu, const int* __restrict__ seq_start, int n_seqs,
     bf16_t* __restrict__ out, int n_heads, int n_kv, float scale, int window, ProjectedQ projected, int chunk_given,
-    const float* __restrict__ sink, const float* __restrict__ rel, int n_dist) {
+    const float* __restrict__ sink, const float* __restrict__ rel, int n_dist, MapPair pair) {
+  static_assert(!DIFF || (RP == 1 && !EXTRA), "two maps: 16 rows a wave, no other options");
   const int chunk = EXTRA ? chunk_given : 0;
   extern __shared__ __attribute__((aligned(16))) unsigned char lds_raw[];
   constexpr int KB = DIRECT_D / 32, TILE_ROWS = 64 * RP, WAVE_ROWS = 16 * RP, head_dim = DIRECT_D;
-  constexpr bool TWO = RP != 1;                               // two buffers each for keys and values
-  const int head = blockIdx.x;
+  constexpr bool TWO = RP != 1 || DIFF;                               // two buffers each for keys and values
+  constexpr int U = DIFF ? 2 : RP, KQ = DIFF ? KB / 2 : KB;   // units of a wave; blocks of 32 features of a query
+  const int head = DIFF ? 2 * (int)blockIdx.x : (int)blockIdx.x;
   const int n_tiles = count_tiles<RP>(seq_slot, cu_rows, tile_cu, n_seqs);
   const int tile = n_tiles - 1 - (int)blockIdx.y;
   if (tile < 0) return;
@@ -784,7 +796,7 @@ __global__ __launch_bounds__(256, RP == 1 ? 4 : 2) void attn_causal_direct_kerne
   int rows[RP], pos0[RP], pos_row[RP], lo_row[RP];
   bool row_valid[RP];
   int64_t row[RP];
-  RowBlock<KB> st[RP];
+  RowBlock<KB> st[U];
 #pragma unroll
   for (int rt = 0; rt < RP; ++rt) {
     const int first = wave_first + 16 * rt;
@@ -794,7 +806,11 @@ __global__ __launch_bounds__(256, RP == 1 ? 4 : 2) void attn_causal_direct_kerne
     pos0[rt] = pos_wave + 16 * rt;
     pos_row[rt] = row_valid[rt] ? pos0[rt] + c : -1;
     lo_row[rt] = first_seen(pos_row[rt], window, chunk);
-    if (projected.qkv != nullptr)
+    if (DIFF) {
+#pragma unroll
+      for (int u = 0; u < U; ++u)
+        init_rows<KB>(st[u], q + (row[rt] * n_heads + head + u) * (DIRECT_D / 2), row_valid[rt], DIRECT_D / 2);
+    } else if (projected.qkv != nullptr)
       init_rows_projected(st[rt], projected, row[rt], head, pos0[rt] + c, row_valid[rt]);
     else
       init_rows<KB>(st[rt], q + (row[rt] * n_heads + head) * head_dim, row_valid[rt], head_dim);
@@ -849,31 +865,38 @@ __global__ __launch_bounds__(256, RP == 1 ? 4 : 2) void attn_causal_direct_kerne
     }
     const int key0 = pg * PAGE_TOKENS;
     const bool sees = page_now >= 0 && key0 <= hi_wave && key0 + PAGE_TOKENS > lo_wave;   // some row sees some key
-    bf16x8 p[RP][2];
+    bf16x8 p[U][2];
     if (sees) {
-      float alpha[RP];
-      bool moved[RP];
-      f32x4 s[RP][4];
+      float alpha[U];
+      bool moved[U];
+      f32x4 s[U][4];
 #pragma unroll
       for (int t = 0; t < 4; ++t) {
 #pragma unroll
-        for (int u = 0; u < RP; ++u) s[u][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int u = 0; u < U; ++u) s[u][t] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int kb = 0; kb < KB; ++kb) {
+        for (int kb = 0; kb < KQ; ++kb) {
+          if (DIFF) {                                         // map u's keys begin 64 features into the row
+#pragma unroll
+            for (int u = 0; u < U; ++u)
+              s[u][t] = MFMA16(*(const bf16x8*)(k_lds + 16 * t * (2 * DIRECT_D) + k_at[KQ * u + kb]), st[u].q[kb], s[u][t]);
+            continue;
+          }
           const bf16x8 a = *(const bf16x8*)(k_lds + 16 * t * (2 * DIRECT_D) + k_at[kb]);
 #pragma unroll
-          for (int u = 0; u < RP; ++u) s[u][t] = MFMA16(a, st[u].q[kb], s[u][t]);
+          for (int u = 0; u < U; ++u) s[u][t] = MFMA16(a, st[u].q[kb], s[u][t]);
         }
       }
 #pragma unroll
-      for (int u = 0; u < RP; ++u) {
-        const bool masked = key0 + PAGE_TOKENS - 1 > pos0[u] || rows[u] < 16 ||
-                            key0 < first_seen(pos0[u] + 15, window, chunk);
-        alpha[u] = masked ? page_softmax<KB, true>(st[u], s[u], p[u], scale_log2, key0, lo_row[u], pos_row[u], moved[u], EXTRA ? cap : ScoreCap{})
-                          : page_softmax<KB, false>(st[u], s[u], p[u], scale_log2, key0, lo_row[u], pos_row[u], moved[u], EXTRA ? cap : ScoreCap{});
+      for (int u = 0; u < U; ++u) {
+        const int rt = DIFF ? 0 : u;
+        const bool masked = key0 + PAGE_TOKENS - 1 > pos0[rt] || rows[rt] < 16 ||
+                            key0 < first_seen(pos0[rt] + 15, window, chunk);
+        alpha[u] = masked ? page_softmax<KB, true>(st[u], s[u], p[u], scale_log2, key0, lo_row[rt], pos_row[rt], moved[u], EXTRA ? cap : ScoreCap{})
+                          : page_softmax<KB, false>(st[u], s[u], p[u], scale_log2, key0, lo_row[rt], pos_row[rt], moved[u], EXTRA ? cap : ScoreCap{});
       }
 #pragma unroll
-      for (int u = 0; u < RP; ++u)
+      for (int u = 0; u < U; ++u)
         if (moved[u]) {                                       // rare once the maxima have settled
 #pragma unroll
           for (int dt = 0; dt < 2 * KB; ++dt) st[u].o[dt] *= alpha[u];
@@ -891,13 +914,18 @@ __global__ __launch_bounds__(256, RP == 1 ? 4 : 2) void attn_causal_direct_kerne
         for (int h = 0; h < 2; ++h) {
           const bf16x8 a = *(const bf16x8*)(v_lds + 16 * dt * (2 * PAGE_TOKENS) + v_at[h]);
 #pragma unroll
-          for (int u = 0; u < RP; ++u) st[u].o[dt] = MFMA16(a, p[u][h], st[u].o[dt]);
+          for (int u = 0; u < U; ++u) st[u].o[dt] = MFMA16(a, p[u][h], st[u].o[dt]);
         }
     }
   }
-  float row_l[RP];
+  float row_l[U];
 #pragma unroll
-  for (int u = 0; u < RP; ++u) row_l[u] = row_sum<KB>(st[u]);
+  for (int u = 0; u < U; ++u) row_l[u] = row_sum<KB>(st[u]);
+  if (DIFF) {
+    store_difference<KB>(st[0], st[U - 1], row_l[0], row_l[U - 1], row_valid[0],
+                         out + (row[0] * (n_heads / 2) + head / 2) * pair.v_dim, pair);
+    return;
+  }
 #pragma unroll
   for (int u = 0; u < RP; ++u) {
     if (!row_valid[u]) continue;
@@ -1389,11 +1417,12 @@ static int launch_causal_direct(const void* q, const void* k_pages, const void* 
   if (chunk > 0 || sink != nullptr || rel != nullptr)
     hipLaunchKernelGGL((attn_causal_direct_kernel<RP, true>), grid, block, lds, stream, (const bf16_t*)q,
                        (const bf16_t*)k_pages, (const bf16_t*)v_pages, page_table, max_pages, seq_slot, cu_rows, tile_cu,
-                       seq_start, n_seqs, (bf16_t*)out, n_heads, n_kv, scale, window, projected, chunk, sink, rel, n_dist);
+                       seq_start, n_seqs, (bf16_t*)out, n_heads, n_kv, scale, window, projected, chunk, sink, rel, n_dist,
+                       MapPair{});
   else
     hipLaunchKernelGGL((attn_causal_direct_kernel<RP, false>), grid, block, lds, stream, (const bf16_t*)q,
                        (const bf16_t*)k_pages, (const bf16_t*)v_pages, page_table, max_pages, seq_slot, cu_rows, tile_cu,
-                       seq_start, n_seqs, (bf16_t*)out, n_heads, n_kv, scale, window, projected, 0, nullptr, nullptr, 0);
+                       seq_start, n_seqs, (bf16_t*)out, n_heads, n_kv, scale, window, projected, 0, nullptr, nullptr, 0, MapPair{});
   return DRYFT_LAUNCH_CHECK();
 }
 
@@ -1567,10 +1596,20 @@ DRYFT_API int dryft_attn_causal_diff_bf16(const void* q, const void* k_pages, co
                                           int max_pages, const int* seq_slot, const int* cu_rows, const int* tile_cu,
                                           const int* seq_start, int n_seqs, int max_tiles, void* out, int n_heads,
                                           int n_kv, int head_dim, int map_dim, int v_dim, float scale, int window,
-                                          float lambda, float post, float eps, hipStream_t stream) {
+                                          float lambda, float post, float eps, int staged, hipStream_t stream) {
   if (n_seqs <= 0 || max_tiles <= 0) return 0;
   const MapPair pair = {map_dim, v_dim, lambda, post, eps};
   if (!head_shape_ok(n_heads, n_kv, head_dim) || !pair_ok(pair, n_heads, n_kv, head_dim)) return -1;
+  // maps of 64 features with values of 128: the pages go straight into LDS (`staged` keeps them in registers on the way)
+  if (!staged && head_dim == DIRECT_D && map_dim == DIRECT_D / 2 && (((uintptr_t)k_pages | (uintptr_t)v_pages) & 15) == 0) {
+    if (max_tiles > 65535) return -1;
+    const size_t lds = 4 * DIRECT_PAGE_BYTES;
+    hipLaunchKernelGGL((attn_causal_direct_kernel<1, false, true>), dim3(n_heads / 2, max_tiles), dim3(256), lds, stream,
+                       (const bf16_t*)q, (const bf16_t*)k_pages, (const bf16_t*)v_pages, page_table, max_pages, seq_slot,
+                       cu_rows, tile_cu, seq_start, n_seqs, (bf16_t*)out, n_heads, n_kv, scale, window, ProjectedQ{}, 0,
+                       nullptr, nullptr, 0, pair);
+    return DRYFT_LAUNCH_CHECK();
+  }
   return launch_causal<2, 1, true>(q, k_pages, v_pages, page_table, max_pages, seq_slot, cu_rows, tile_cu, seq_start,
                                    n_seqs, max_tiles, out, n_heads, n_kv, head_dim, scale, window,
                                    ScoreOptions{0.f, nullptr, 0, nullptr, 0}, stream, pair);

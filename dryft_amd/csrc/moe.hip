@@ -31,7 +31,7 @@ __device__ __forceinline__ Best wave_best(Best b) {
 // Other forms: `softmax` takes s = softmax(z) over all experts instead of the sigmoid; no correction (null): the
 // choice scores are s itself; `group_best`: a group scores as its single largest choice score; without `renorm`
 // the weights are s * scale as they are. `softmax` = 2: no scores at all; the logits themselves (plus `logit_bias`, if
-// there is one) decide, and the weights are the softmax over the chosen logits alone, times scale.
+// there is one) decide; a chosen expert weighs exp(its logit) over the sum of the chosen ones' exponentials, times scale.
 template <int PER>
 __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ logits, int64_t stride,
                                                         const float* __restrict__ correction, int n_experts, int groups,

@@ -62,7 +62,7 @@ _SIGNATURES = {
                                               _I, _I, _I, _P]},
     "attn_rows": {"dryft_attn_rows": [_P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _F, _P, _I, _I, _P, _I, _I, _I, _P]},
     "attn_mfma": {"dryft_attn_causal_diff_bf16": [_P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _I, _F,
-                                                  _I, _F, _F, _F, _P],
+                                                  _I, _F, _F, _F, _I, _P],
                   "dryft_attn_split_diff_bf16": [_P, _P, _P, _P, _I, _P, _P, _P, _I, _P, _P, _I, _P, _I, _I, _I, _I, _F, _I,
                                                  _F, _F, _F, _P],
                   "dryft_attn_causal_bf16": [_P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _I, _P, _I, _I, _I, _F, _I, _I, _F, _P,
@@ -1333,10 +1333,11 @@ def map_difference(a, out, v_dim: int, lam: float, post: float, eps: float) -> t
 
 def attn_causal_diff_bf16(q, k_pages, v_pages, page_table, seq_slot, cu_rows, tile_cu, seq_start, n_seqs: int,
                           max_tiles: int, out, n_heads: int, n_kv: int, map_dim: int, v_dim: int, scale: float,
-                          window: int, lam: float, post: float, eps: float) -> None:
+                          window: int, lam: float, post: float, eps: float, staged: bool = False) -> None:
     """Differential attention of steps with many rows per sequence, on the matrix cores. ``q [rows, heads, 2, map_dim]``;
     pages of keys and of values of one width (a multiple of 16), a key's maps at 0 and ``map_dim`` (a multiple of 8) of
-    its row, a value's ``v_dim`` features first; ``out [rows, heads, v_dim]`` receives the maps' difference, normed."""
+    its row, a value's ``v_dim`` features first; ``out [rows, heads, v_dim]`` receives the maps' difference, normed.
+    Pages 128 wide with maps of 64 go straight into LDS, others through registers (``staged``: those too)."""
     page_dim = _diff_operands("attn_causal_diff", q, k_pages, v_pages, page_table, out, n_heads, n_kv, map_dim, v_dim, map_dim)
     for name, t, n in (("seq_slot", seq_slot, n_seqs), ("cu_rows", cu_rows, n_seqs + 1),
                        ("tile_cu", tile_cu, n_seqs + 1), ("seq_start", seq_start, n_seqs)):
@@ -1346,7 +1347,7 @@ def attn_causal_diff_bf16(q, k_pages, v_pages, page_table, seq_slot, cu_rows, ti
     _check(_fn("attn_mfma", "dryft_attn_causal_diff_bf16")(
         _ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(page_table), page_table.shape[1], _ptr(seq_slot), _ptr(cu_rows),
         _ptr(tile_cu), _ptr(seq_start), n_seqs, max_tiles, _ptr(out), 2 * n_heads, n_kv, page_dim, map_dim, v_dim,
-        float(scale), int(window), float(lam), float(post), float(eps), _stream()), "attn_causal_diff_bf16")
+        float(scale), int(window), float(lam), float(post), float(eps), int(bool(staged)), _stream()), "attn_causal_diff_bf16")
 
 
 def attn_split_diff_bf16(q, k_pages, v_pages, page_table, seq_slot, cu_rows, kv_len, n_seqs: int, part_o, part_ml,
@@ -1910,8 +1911,8 @@ def moe_route(logits, correction, n_experts: int, groups: int, keep: int, scale:
     ``sigmoid / (sum of the chosen sigmoids + 1e-20) * scale``. ``chosen`` int32 and ``weights`` float32 ``[rows, top]``.
     ``softmax``: scores are the softmax over all experts instead; ``correction`` None: none; ``group_best``: a group
     scores as its best expert; ``renorm`` off: the weights are the scores times ``scale`` as they are.
-    ``chosen_softmax``: the logits plus ``logit_bias`` (float32 ``[experts]``, optional) decide, and the weights are the
-    softmax over the chosen ones alone, times ``scale``."""
+    ``chosen_softmax``: the logits plus ``logit_bias`` (float32 ``[experts]``, optional) decide, and a chosen expert weighs
+    ``exp(its logit)`` over the sum of the chosen ones' exponentials, times ``scale``."""
     if chosen_softmax and (softmax or correction is not None) or (logit_bias is not None and not chosen_softmax):
         raise KernelError("moe_route: chosen_softmax goes alone, and a bias on the logits only with it")
     if logit_bias is not None:

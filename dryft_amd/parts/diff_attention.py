@@ -2,14 +2,14 @@
 
 Every head has two maps, each with a query and a key of its own (``dim`` features each, projected side by side: head by
 head ``[map 1, map 2]``); the values, of a width of their own, are one for both. Query head ``h`` reads kv head
-``h // group``. q, k and v have biases, added before anything else; of each map's first features neighbouring pairs turn
-with the position. A row sees the keys up to its own position, or the last ``window`` of them; each map's weights are
-an ordinary softmax of ``scale * (q . k)``. With the maps' outputs ``a1`` and ``a2``
+``h // group``. The three projections in carry biases, added before anything else; of each map's first features
+neighbouring pairs turn with the position. A row sees the keys up to its own position, or the last ``window`` of them;
+each map's weights are an ordinary softmax of ``scale * (q . k)``. With the maps' outputs ``a1`` and ``a2``, per head,
 
-    lambda = exp(sum(lq1 * lk1)) - exp(sum(lq2 * lk2)) + diff           (one number for the layer)
-    o      = a1 - lambda * a2,   o <- o / sqrt(mean(o^2) + eps) * (1 - diff)
+    c = e^(lq1 . lk1) - e^(lq2 . lk2) + diff,      d = a1 - c a2,      out = (1 - diff) d / rms(d)
 
-per head, no weight in the norm, and an output projection without a bias.
+(``c`` is the layer's, from four learned vectors as long as a map's key; ``rms`` with ``eps`` under the root), and an output
+projection without a bias.
 
 A key is cached as one row that holds both maps, so a page serves both with one read and the values are kept once. In
 bfloat16 the matrix-core kernels take pages of one width for keys and values, a multiple of 16: the wider of twice a

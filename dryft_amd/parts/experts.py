@@ -17,8 +17,8 @@ up(h))``, nothing clamped, and so is the shared expert.
 scores themselves decide; ``group_score="best"``: a group scores as its best expert; ``renormalize=False``: the weights
 are the chosen scores times ``route_scale`` as they are; ``shared_gate=False``: the shared expert is added as it is.
 ``score="chosen_softmax"``: the logits themselves decide, with ``logit_bias`` after one learned number per expert has been
-added to them (tensor ``router_bias``), and the weights are the softmax over the chosen logits alone times
-``route_scale``.
+added to them (tensor ``router_bias``), and a chosen expert weighs its logit's exponential over the sum of the chosen ones',
+times ``route_scale``.
 ``unit="relu2"``: an expert has no gate, ``down(relu(up(h))^2)``, and so has the shared expert.
 
 On the device throughout, so a step can be captured: the router picks, a small kernel sorts the (row, expert) pairs

@@ -334,6 +334,37 @@ def test_one_key_stands_out(dtype, which, at, window):
         assert rel_err(got, want) <= 2 * MIXER_TOL[dtype], cuts[:3]
 
 
+@pytest.mark.parametrize("window", [0, 100])
+def test_pages_straight_into_lds_or_through_registers(window):
+    """Maps of 64 features with values of 128 have two prompt kernels: the same numbers, in a step of sequences that go on
+    (one sits out), with pages that are not in order."""
+    from dryft_amd.csrc import ops
+    g = torch.Generator().manual_seed(5)
+    H, G, starts, rows = 6, 2, [70, 0, 3], [150, 65, 64]
+    n = sum(rows)
+    k, v = torch.randn(12, G, 64, 128, generator=g).bfloat16(), torch.randn(12, G, 128, 64, generator=g).bfloat16()
+    q = torch.randn(n, H, 2, 64, generator=g).bfloat16()
+    table = i32([[7, 2, 9, 0], [1, 3, -1, -1], [5, 8, -1, -1]])
+    slots = [0, -1, 2]
+    tiles = [-(-r // 64) if s >= 0 else 0 for s, r in zip(slots, rows)]
+    got = []
+    for staged in (True, False):
+        out = torch.zeros(n, H, 128, dtype=torch.bfloat16, device=DEV)
+        ops.attn_causal_diff_bf16(dev(q), dev(k), dev(v), table, i32(slots), i32([0, 150, 215, 279]), i32([0, 3, 3, 4]), i32(starts), 3,
+                                  sum(tiles), out, H, G, 64, 128, 0.3, window, 0.45, 0.6, EPS, staged=staged)
+        got.append(out.cpu())
+    assert torch.equal(got[0], got[1]) and float(got[0][150:215].abs().max()) == 0.0
+    cols = value_columns()
+    for s, first, r, pages in ((0, 0, 150, [7, 2, 9, 0]), (2, 215, 64, [5, 8])):
+        kd = torch.cat([k[p] for p in pages], 1).double()                       # [G, positions, 128]
+        vd = torch.cat([v[p][:, :, cols].transpose(1, 2) for p in pages], 1).double()
+        pos = torch.arange(starts[s], starts[s] + r)
+        seen = P.visible(pos, torch.arange(kd.shape[1]), window)
+        for h in range(H):
+            a = [P.one_map(q[first:first + r, h, m].double(), kd[h // 3][:, 64 * m:64 * m + 64], vd[h // 3], seen, 0.3) for m in (0, 1)]
+            assert rel_err(got[0][first:first + r, h], P.combine(a[0], a[1], 0.45, 0.4, EPS)) <= MIXER_TOL["bfloat16"], (s, h)
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_the_first_tokens(dtype):
     """Row 0 sees itself alone: both maps give its value, whatever the scores; row 1 two keys. With a factor of nearly
