@@ -40,15 +40,15 @@ def dev(t):
 
 # ------------------------------------------------------------------------------------------ kernels alone
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("n,width", [(1, 60), (3, 256), (4, 1000), (8, 64), (5, 77)])
+@pytest.mark.parametrize("n,width", [(1, 60), (3, 256), (4, 1000), (8, 64), (5, 77), (4, 2048), (2, 4608), (2, 8200)])
 def test_copies_behind_a_layer_norm(dtype, n, width):
     from dryft_amd.csrc import ops
     T = TORCH[dtype]
     g = torch.Generator().manual_seed(width + n)
-    rows = 7
+    rows = 130 if width == 2048 else 7                        # many rows of many columns: two runs of columns a thread
     copies = torch.randn(n, rows, width, generator=g) * 3 + 4                  # a mean that is not zero
     start = (torch.randn(rows, width, generator=g) + 1).to(T)
-    delta, parts = torch.randn(rows, width, generator=g).to(T), torch.randn(3, rows, width, generator=g)
+    delta, parts = torch.randn(rows, width, generator=g).to(T), torch.randn(6, rows, width, generator=g)
     mix, write, read, w, b = (torch.randn(s, generator=g) for s in ((n, n), (n,), (n,), (width,), (width,)))
     for x in (copies, start):
         xs = x.double() if x.dim() == 3 else x.double()[None].expand(n, -1, -1)
@@ -62,7 +62,7 @@ def test_copies_behind_a_layer_norm(dtype, n, width):
                 for bias in (None, b):
                     x_out = torch.empty(n, rows, width, dtype=torch.float32, device=DEV)
                     y = torch.empty(rows, width, dtype=T, device=DEV)
-                    ops.hyper_norm(dev(x), n, (dev(d), 3) if d is not None and d.dim() == 3 else dev(d),
+                    ops.hyper_norm(dev(x), n, (dev(d), 6) if d is not None and d.dim() == 3 else dev(d),
                                    dev(mix) if d is not None else None, dev(write) if d is not None else None, dev(rd), dev(w),
                                    EPS, x_out, y, normed=True, centred=True, bias=dev(bias))
                     assert torch.allclose(x_out.cpu().double(), want, atol=3e-5, rtol=1e-6)
